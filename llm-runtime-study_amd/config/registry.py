@@ -74,10 +74,12 @@ def _load_builtin() -> None:
     from ..text.chat import format_qwen3_chat
     from ..models.felosun import build_spec as build_felosun
     from ..models.kaposun import build_spec as build_kaposun
+    from ..models.mutolix import build_spec as build_mutolix
     from ..models.napizen import build_spec as build_napizen
     from ..models.nobodra import build_spec as build_nobodra
     from .felosun import FelosunConfig
     from .kaposun import KaposunConfig
+    from .mutolix import MutolixConfig
     from .napizen import NapizenConfig
     from .nobodra import NobodraConfig
     from .qwen3 import Qwen3Config
@@ -92,6 +94,8 @@ def _load_builtin() -> None:
         register_architecture(KaposunConfig.ARCHITECTURE, KaposunConfig, build_kaposun)      # token ids only
     if FelosunConfig.ARCHITECTURE not in _ARCHITECTURES:
         register_architecture(FelosunConfig.ARCHITECTURE, FelosunConfig, build_felosun)      # token ids only
+    if MutolixConfig.ARCHITECTURE not in _ARCHITECTURES:
+        register_architecture(MutolixConfig.ARCHITECTURE, MutolixConfig, build_mutolix)      # token ids only
     import importlib
     import os
 

@@ -42,6 +42,15 @@ __device__ __forceinline__ float with_sink(float sink2, float top, float& total)
 }
 constexpr float LOG2E = 1.4426950408889634f;
 
+// A bias by distance: a score of query head h loses rate_h * ln(1 + reach_h * (i - j)), i the query's position, j the key's.
+// `distance` holds the rates of all nq heads, then their reaches (null: no bias).  In the bfloat16 kernels the logarithm is the
+// hardware's (base 2, a unit in the last place), and the distance from a query to the first key of a lane's four (or eight) is
+// taken in whole positions before it meets the reach, so that a near key's distance is exact however far on the sequence is.
+__device__ __forceinline__ float distance_loss(float rate2, float reach, float distance) {       // rate2: for base-2 logarithms
+  return rate2 * __builtin_amdgcn_logf(fmaf(reach, distance, 1.f));
+}
+constexpr float LN2 = 0.6931471805599453f;
+
 // A gate a head: the head's output times sigmoid(gates[token, head]), the gate values lying in rows of their own stride (the
 // columns of the projection that made them).  Null: no gate.
 template <typename T>
@@ -58,7 +67,8 @@ __global__ __launch_bounds__(THREADS) void attention_generic_kernel(
     const T* __restrict__ k_pages, const T* __restrict__ v_pages,
     const int* __restrict__ block_table, int table_stride, const int* __restrict__ token_request,
     const int* __restrict__ positions, int nq, int nkv, int d, int dv, int page_size, float scale,
-    int window, int keep_first, const float* __restrict__ sinks, float softcap, const T* __restrict__ gates, int gate_stride) {
+    int window, int keep_first, const float* __restrict__ sinks, float softcap, const T* __restrict__ gates, int gate_stride,
+    const float* __restrict__ distance) {
   extern __shared__ __attribute__((aligned(16))) float smem[];
   float* qs = smem;                           // [d]
   float* probs = qs + d + d % 2;              // [THREADS]
@@ -109,6 +119,7 @@ __global__ __launch_bounds__(THREADS) void attention_generic_kernel(
       }
       score = dot * scale;
       if (softcap > 0.f) score = softcap * tanhf(score / softcap);
+      if (distance) score -= distance[head] * logf(1.f + distance[nq + head] * (float)(pos - key));
     }
     const float tile_max = block_max(score, scratch);
     const float new_max = fmaxf(running_max, tile_max);
@@ -270,7 +281,7 @@ __global__ __launch_bounds__(WAVES * 64) void attention_decode_bf16_kernel(
     bf16* __restrict__ v_pages, const int* __restrict__ block_table, int table_stride,
     const int* __restrict__ token_request, const int* __restrict__ positions, int nq, int nkv,
     int page_size, float scale, int window, int splits, int slots, DecodePrep prep, const float* __restrict__ sinks,
-    float softcap, const bf16* __restrict__ gates, int gate_stride) {
+    float softcap, const bf16* __restrict__ gates, int gate_stride, int dv, const float* __restrict__ distance) {
   constexpr int DS = D / 32, DB = D / 16, THREADS = WAVES * 64;
   __shared__ float sm_m[WAVES][16], sm_l[WAVES][16];
   __shared__ float sm_o[WAVES][D][16];
@@ -334,9 +345,10 @@ __global__ __launch_bounds__(WAVES * 64) void attention_decode_bf16_kernel(
     const int key8 = tile * 32 + g * 8;                        // this lane's eight keys; pages hold multiples of 16
     if (key8 <= pos && key8 + 7 >= lo) {
       const int64_t page = page_ids[key8 / page_size - first_block];
-      const bf16* vp = v_pages + (page * nkv + kvh) * (int64_t)D * page_size + (int64_t)col * page_size + key8 % page_size;
+      const bf16* vp = v_pages + (page * nkv + kvh) * (int64_t)dv * page_size + (int64_t)col * page_size + key8 % page_size;
+      // (values narrower than keys: the blocks behind them repeat the last one, and nothing of them is written)
 #pragma unroll
-      for (int b = 0; b < DB; ++b) vf[b] = *(const bf16x8*)(vp + (int64_t)b * 16 * page_size);
+      for (int b = 0; b < DB; ++b) vf[b] = *(const bf16x8*)(vp + (int64_t)(b * 16 < dv ? b * 16 : dv - 16) * page_size);
     } else {
 #pragma unroll
       for (int b = 0; b < DB; ++b) vf[b] = zero8;
@@ -406,6 +418,9 @@ __global__ __launch_bounds__(WAVES * 64) void attention_decode_bf16_kernel(
   for (int b = 0; b < DB; ++b) o[b] = floatx4{0.f, 0.f, 0.f, 0.f};
   float run_max = -INFINITY, run_sum = 0.f;
   const float scale2 = scale * 1.4426950408889634f;
+  // the column's head's bias by distance, in the base-2 units of the scores below
+  const int biased = kvh * group + (col < group ? col : 0);
+  const float rate2 = distance ? distance[biased] : 0.f, reach = distance ? distance[nq + biased] : 0.f;
 
   auto work = [&](int tile, bf16x8 (&kf)[2][DS], bf16x8 (&vf)[DB]) {
     if (holds_own && tile == last_tile) {
@@ -439,7 +454,8 @@ __global__ __launch_bounds__(WAVES * 64) void attention_decode_bf16_kernel(
       for (int i = 0; i < 4; ++i) {
         const int key = tile * 32 + g * 8 + h * 4 + i;
         const bool valid = key <= pos && key >= lo;
-        const float scaled = softcap > 0.f ? capped(s[h][i] * scale, softcap) * LOG2E : s[h][i] * scale2;
+        float scaled = softcap > 0.f ? capped(s[h][i] * scale, softcap) * LOG2E : s[h][i] * scale2;
+        if (distance) scaled -= distance_loss(rate2, reach, (float)(pos - key));
         s[h][i] = valid ? scaled : -INFINITY;
         tile_max = fmaxf(tile_max, s[h][i]);
       }
@@ -496,7 +512,7 @@ __global__ __launch_bounds__(WAVES * 64) void attention_decode_bf16_kernel(
 #pragma unroll
     for (int i = 0; i < 4; ++i) sm_o[wave][b * 16 + g * 4 + i][col] = o[b][i];
   __syncthreads();
-  for (int e = tid; e < D * 16; e += THREADS) {
+  for (int e = tid; e < dv * 16; e += THREADS) {
     const int dim = e / 16, h = e % 16;
     if (h >= group) continue;
     float top = sm_m[0][h];
@@ -512,10 +528,10 @@ __global__ __launch_bounds__(WAVES * 64) void attention_decode_bf16_kernel(
     const int head = kvh * group + h;
     if (slots <= 1) {
       if (sinks) acc *= with_sink(sinks[head] * LOG2E, top, total);
-      out[(int64_t)token * out_stride + (int64_t)head * D + dim] = (bf16)(acc / total * head_gate(gates, gate_stride, token, head));
+      out[(int64_t)token * out_stride + (int64_t)head * dv + dim] = (bf16)(acc / total * head_gate(gates, gate_stride, token, head));
     } else {
       const int64_t slot = ((int64_t)token * nq + head) * slots + split;
-      part_o[slot * D + dim] = acc;
+      part_o[slot * dv + dim] = acc;
       if (dim == 0) {
         part_ml[slot * 2] = top;
         part_ml[slot * 2 + 1] = total;
@@ -642,7 +658,7 @@ __global__ __launch_bounds__(WAVE) void attention_kept_bf16_kernel(
     const bf16* __restrict__ q, int q_stride, const bf16* __restrict__ k_pages, const bf16* __restrict__ v_pages,
     const int* __restrict__ block_table, int table_stride, const int* __restrict__ token_request,
     const int* __restrict__ positions, int nq, int nkv, int d, int page_size, float scale, int window, int keep_first,
-    int slots, float* __restrict__ part_o, float* __restrict__ part_ml, float softcap) {
+    int slots, float* __restrict__ part_o, float* __restrict__ part_ml, float softcap, int dv, const float* __restrict__ distance) {
   constexpr int PER_LANE = 4;                                     // heads of up to 256 dims
   const int token = blockIdx.x, head = blockIdx.y, lane = threadIdx.x;
   const int kvh = head / (nq / nkv);
@@ -664,17 +680,18 @@ __global__ __launch_bounds__(WAVE) void attention_kept_bf16_kernel(
     const int64_t page = table[key / page_size];
     const int off = key % page_size;
     const bf16* kp = k_pages + ((page * nkv + kvh) * page_size + off) * (int64_t)d;
-    const bf16* vp = v_pages + (page * nkv + kvh) * (int64_t)d * page_size + off;
+    const bf16* vp = v_pages + (page * nkv + kvh) * (int64_t)dv * page_size + off;
     float dot = 0.f, vv[PER_LANE];
 #pragma unroll
     for (int n = 0; n < PER_LANE; ++n) {
       const int dim = lane + n * WAVE;
       dot += dim < d ? qv[n] * (float)kp[dim] : 0.f;
-      vv[n] = dim < d ? (float)vp[(int64_t)dim * page_size] : 0.f;
+      vv[n] = dim < dv ? (float)vp[(int64_t)dim * page_size] : 0.f;
     }
 #pragma unroll
     for (int step = 1; step < WAVE; step *= 2) dot += __shfl_xor(dot, step, WAVE);
-    const float score = softcap > 0.f ? capped(dot * scale, softcap) * LOG2E : dot * scale2;
+    float score = softcap > 0.f ? capped(dot * scale, softcap) * LOG2E : dot * scale2;
+    if (distance) score -= distance_loss(distance[head], distance[nq + head], (float)(pos - key));
     const float new_top = fmaxf(top, score);
     const float keep = top == -INFINITY ? 0.f : fast_exp2(top - new_top);
     const float weight = fast_exp2(score - new_top);
@@ -686,7 +703,7 @@ __global__ __launch_bounds__(WAVE) void attention_kept_bf16_kernel(
 #pragma unroll
   for (int n = 0; n < PER_LANE; ++n) {
     const int dim = lane + n * WAVE;
-    if (dim < d) part_o[slot * d + dim] = acc[n];
+    if (dim < dv) part_o[slot * dv + dim] = acc[n];
   }
   if (lane == 0) {
     part_ml[slot * 2] = top;
@@ -697,10 +714,10 @@ __global__ __launch_bounds__(WAVE) void attention_kept_bf16_kernel(
 static void launch_attention_kept(const bf16* q, int q_stride, const bf16* k_pages, const bf16* v_pages, const int* block_table,
                                   int table_stride, const int* token_request, const int* positions, int tokens, int nq, int nkv, int d,
                                   int page_size, float scale, int window, int keep_first, int slots, float* part_o, float* part_ml,
-                                  float softcap, hipStream_t s) {
+                                  float softcap, int dv, const float* distance, hipStream_t s) {
   attention_kept_bf16_kernel<<<dim3(tokens, nq), WAVE, 0, s>>>(q, q_stride, k_pages, v_pages, block_table, table_stride, token_request,
                                                                positions, nq, nkv, d, page_size, scale, window, keep_first, slots, part_o,
-                                                               part_ml, softcap);
+                                                               part_ml, softcap, dv, distance);
 }
 
 // Decode step in bf16: one query token per request.  part_o [tokens, nq, splits, d] and part_ml
@@ -717,7 +734,9 @@ LRS_API int lrs_attention_decode(void* out, int out_stride, float* part_o, float
                                  int page_size, float scale, int window, int keep_first, int splits, int form, int prepare,
                                  const void* q_weight, const void* k_weight, int w_dtype, float eps,
                                  const float* cosv, const float* sinv, int kv_columns, const float* sinks, float softcap,
-                                 const void* gates, int gate_stride, void* stream) {
+                                 const void* gates, int gate_stride, int dv, const float* distance, void* stream) {
+  LRS_REQUIRE(dv > 0 && dv % 16 == 0 && dv <= d && (dv == d || !prepare),
+              "attention_decode: values of %d dims beside keys of %d are not served (a multiple of 16, at most the keys', heads that come prepared)", dv, d);
   LRS_REQUIRE(tokens > 0 && nq > 0 && nkv > 0 && nq % nkv == 0, "attention_decode: bad sizes tokens=%d nq=%d nkv=%d", tokens, nq, nkv);
   LRS_REQUIRE(nq / nkv <= 16, "attention_decode: %d query heads per kv head, at most 16 fit a tile", nq / nkv);
   LRS_REQUIRE(page_size % 16 == 0, "attention_decode: page size %d is not a multiple of 16", page_size);
@@ -751,7 +770,7 @@ LRS_API int lrs_attention_decode(void* out, int out_stride, float* part_o, float
 #define ARGS                                                                                                 \
   (bf16*)out, out_stride, part_o, part_ml, (const bf16*)q, q_stride, (bf16*)k_pages, (bf16*)v_pages, block_table, \
       table_stride, token_request, positions, nq, nkv, page_size, scale, window, splits, slots, prep, slots == 1 ? sinks : nullptr, softcap, \
-      slots == 1 ? (const bf16*)gates : nullptr, gate_stride
+      slots == 1 ? (const bf16*)gates : nullptr, gate_stride, dv, distance
 #define LAUNCH_PREP(D, PREP)                                                                                 \
   do {                                                                                                       \
     if (form == 2 && D <= 128) attention_decode_bf16_kernel<D, PREP, 8, (D <= 128)><<<grid, 512, table_lds, s>>>(ARGS); \
@@ -777,11 +796,11 @@ LRS_API int lrs_attention_decode(void* out, int out_stride, float* part_o, float
   if (lrs_check_launch("attention_decode")) return 1;
   if (keep_first > 0) {
     launch_attention_kept((const bf16*)q, q_stride, (const bf16*)k_pages, (const bf16*)v_pages, block_table, table_stride, token_request,
-                          positions, tokens, nq, nkv, d, page_size, scale, window, keep_first, slots, part_o, part_ml, softcap, s);
+                          positions, tokens, nq, nkv, d, page_size, scale, window, keep_first, slots, part_o, part_ml, softcap, dv, distance, s);
     if (lrs_check_launch("attention_kept")) return 1;
   }
   if (slots > 1) {
-    launch_attention_merge((bf16*)out, out_stride, part_o, part_ml, tokens, nq, d, slots, sinks, (const bf16*)gates, gate_stride, s);
+    launch_attention_merge((bf16*)out, out_stride, part_o, part_ml, tokens, nq, dv, slots, sinks, (const bf16*)gates, gate_stride, s);
     return lrs_check_launch("attention_merge");
   }
   return 0;
@@ -815,7 +834,8 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void attention_prefill_bf16_
     const int* __restrict__ positions, const int* __restrict__ qblock_token0,
     const int* __restrict__ qblock_count, int n_blocks, int chunk, int nq, int nkv, int page_size, float scale,
     int window, int splits, int slots, float* __restrict__ part_o, float* __restrict__ part_ml,
-    const float* __restrict__ sinks, float softcap, const bf16* __restrict__ gates, int gate_stride) {
+    const float* __restrict__ sinks, float softcap, const bf16* __restrict__ gates, int gate_stride, int dv,
+    const float* __restrict__ distance) {
   constexpr int DS = D / 32, DB = D / 16;
   // Padded LDS rows.  Every fragment is read 16 bytes a lane, 16 rows at a time (the lane's row is col, its
   // piece g), which the LDS serves at its full 256 bytes a cycle when rows lie 32 bytes more than a multiple
@@ -876,7 +896,10 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void attention_prefill_bf16_
 #pragma unroll
   for (int i = 0; i < KPT; ++i) koff[i] = (unsigned)(((t1 + i * TPR) / KPIECES) * D + ((t1 + i * TPR) % KPIECES) * 8);
 #pragma unroll
-  for (int i = 0; i < VPT; ++i) voff[i] = (unsigned)(((t1 + i * TPR) / 2) * page_size + ((t1 + i * TPR) % 2) * 8);
+  for (int i = 0; i < VPT; ++i) {                                 // (values narrower than keys: the dims behind them repeat the last one)
+    const int dim = (t1 + i * TPR) / 2 < dv ? (t1 + i * TPR) / 2 : dv - 1;
+    voff[i] = (unsigned)(dim * page_size + ((t1 + i * TPR) % 2) * 8);
+  }
   auto fetch = [&](int tile, bf16x8 (&kreg)[KPT], bf16x8 (&vreg)[VPT]) {
     const int run = tile * 2 + wrun, key0 = run * 16;
     const bool present = key0 <= pos_last && key0 + 15 >= lo_first;
@@ -885,7 +908,7 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void attention_prefill_bf16_
       const int64_t page = __builtin_amdgcn_readfirstlane(page_ids[block - first_block]);
       const int off = (run - block * pages16) * 16;
       const bf16* kbase = k_pages + ((page * nkv + kvh) * page_size + off) * D;
-      const bf16* vbase = v_pages + (page * nkv + kvh) * (int64_t)D * page_size + off;
+      const bf16* vbase = v_pages + (page * nkv + kvh) * (int64_t)dv * page_size + off;
 #pragma unroll
       for (int i = 0; i < KPT; ++i) kreg[i] = t1 + i * TPR < RUN_CHUNKS ? *(const bf16x8*)(kbase + koff[i]) : zero8;
 #pragma unroll
@@ -939,9 +962,12 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void attention_prefill_bf16_
       for (int e = 0; e < DB; ++e) o[b][e] = floatx4{0.f, 0.f, 0.f, 0.f};
     }
 
+    // the head's bias by distance, in units of the unscaled scores
+    const int biased = active ? head : head0;
+    const float rate = distance ? distance[biased] * LN2 / scale : 0.f, reach = distance ? distance[nq + biased] : 0.f;
     // The three parts of a tile's work.
     // scores: S[key, query] = K Q^T, unscaled (the scale enters with the exponent).
-    auto scores = [&](int buffer, floatx4 (&sc)[QB][2]) {
+    auto scores = [&](int tile, int buffer, floatx4 (&sc)[QB][2]) {
       const bf16* kt = ks[buffer];
 #pragma unroll
       for (int b = 0; b < QB; ++b) sc[b][0] = sc[b][1] = floatx4{0.f, 0.f, 0.f, 0.f};
@@ -961,6 +987,16 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void attention_prefill_bf16_
           for (int h = 0; h < 2; ++h)
 #pragma unroll
             for (int i = 0; i < 4; ++i) sc[b][h][i] = capped(sc[b][h][i], cap);
+      }
+      if (distance) {            // (a key ahead of the query gives no number here; the mask takes it out)
+#pragma unroll
+        for (int b = 0; b < QB; ++b)
+#pragma unroll
+          for (int h = 0; h < 2; ++h) {
+            const float behind = (float)((live[b] ? pos[b] : pos_last) - (tile * 32 + h * 16 + g * 4));
+#pragma unroll
+            for (int i = 0; i < 4; ++i) sc[b][h][i] -= distance_loss(rate, reach, behind - (float)i);
+          }
       }
     };
     // weights: one step of the running softmax, p = 2^(s * scale2 - reference * scale2) as bfloat16 operands.
@@ -1077,7 +1113,7 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void attention_prefill_bf16_
       for (; tile <= last_tile; ++tile) {
         const int buffer = (tile - first_tile) & 1;
         if (tile < last_tile) fetch(tile + 1, kreg_a, vreg_a);
-        scores(buffer, sc);
+        scores(tile, buffer, sc);
         if (tile < whole_begin || tile >= whole_end || !weights(sc, pf)) {
           unfinished = true;
           break;
@@ -1103,7 +1139,8 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void attention_prefill_bf16_
       if (live[b] && slots > 1) {
         const int64_t slot = ((int64_t)(token0 + b * 16 + col) * nq + head) * slots + split;
 #pragma unroll
-        for (int e = 0; e < DB; ++e) *(floatx4*)(part_o + slot * D + e * 16 + g * 4) = o[b][e];
+        for (int e = 0; e < DB; ++e)
+          if (e * 16 < dv) *(floatx4*)(part_o + slot * dv + e * 16 + g * 4) = o[b][e];
         if (g == 0) {
           part_ml[slot * 2] = run_max[b] * scale2;               // -inf stays -inf: no key seen
           part_ml[slot * 2 + 1] = total;
@@ -1111,9 +1148,10 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void attention_prefill_bf16_
       } else if (live[b]) {
         const float keep = sinks ? with_sink(sinks[head] * LOG2E, run_max[b] * scale2, total) : 1.f;
         const float inv = keep / total * head_gate(gates, gate_stride, token0 + b * 16 + col, head);
-        bf16* dst = out + (int64_t)(token0 + b * 16 + col) * out_stride + (int64_t)head * D + g * 4;
+        bf16* dst = out + (int64_t)(token0 + b * 16 + col) * out_stride + (int64_t)head * dv + g * 4;
 #pragma unroll
         for (int e = 0; e < DB; ++e) {
+          if (e * 16 >= dv) break;
           const bf16x4 packed = {(bf16)(o[b][e][0] * inv), (bf16)(o[b][e][1] * inv), (bf16)(o[b][e][2] * inv), (bf16)(o[b][e][3] * inv)};
           *(bf16x4*)(dst + e * 16) = packed;
         }
@@ -1144,8 +1182,10 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void attention_prefill_bf16_
 // The wave that fetched a tile waits for its own fetches (vmcnt) before the barrier that opens the
 // tile to the others; the fetches of the tile after it stay in flight.  The fetches are written in
 // assembly because the compiler would wait for all of them before any LDS read it cannot tell apart.
-// CAPPED: the scaled scores pass softcap * tanh(score / softcap) (an instance of its own, so that the others keep their registers).
-template <int QB, bool MANY_WAVES, bool IDLE_WAVES, bool CAPPED>
+// SCORES: what happens to the scores before the softmax, by instances of their own so that the others keep their registers:
+// nothing, a cap (softcap * tanh(score / softcap) of the scaled scores), a bias by distance, or the cap and then the bias.
+enum { SCORES_PLAIN = 0, SCORES_CAPPED = 1, SCORES_DISTANCE = 2, SCORES_BOTH = 3 };
+template <int QB, bool MANY_WAVES, bool IDLE_WAVES, int SCORES>
 __global__ __launch_bounds__(MANY_WAVES ? 512 : 256, MANY_WAVES ? 1 : 2) void attention_prefill_d128_bf16_kernel(
     bf16* __restrict__ out, int out_stride, const bf16* __restrict__ q, int q_stride,
     const bf16* __restrict__ k_pages, const bf16* __restrict__ v_pages,
@@ -1153,7 +1193,9 @@ __global__ __launch_bounds__(MANY_WAVES ? 512 : 256, MANY_WAVES ? 1 : 2) void at
     const int* __restrict__ positions, const int* __restrict__ qblock_token0,
     const int* __restrict__ qblock_count, int n_blocks, int chunk, int nq, int nkv, int page_size, float scale,
     int window, int splits, int slots, float* __restrict__ part_o, float* __restrict__ part_ml, int prepare_q, DecodePrep prep,
-    const float* __restrict__ sinks, float softcap, const bf16* __restrict__ gates, int gate_stride) {
+    const float* __restrict__ sinks, float softcap, const bf16* __restrict__ gates, int gate_stride, int dv,
+    const float* __restrict__ distance) {
+  constexpr bool CAPPED = (SCORES & SCORES_CAPPED) != 0, DISTANCE = (SCORES & SCORES_DISTANCE) != 0;
   constexpr int D = 128, DS = D / 32, DB = D / 16, STAGES = 3;
   constexpr int KBLOCK = 1024 + 32, KBYTES = 8 * KBLOCK, VHALF = 16 * D * 2 + 16, VBYTES = 2 * VHALF;
   constexpr int VSTAGE = (VBYTES + 63) / 64 * 64;
@@ -1194,16 +1236,19 @@ __global__ __launch_bounds__(MANY_WAVES ? 512 : 256, MANY_WAVES ? 1 : 2) void at
   // lane l of a key block brings row l / 16 (h = row / 2, k = row % 2), piece l % 16: key 8 k + 4 h + wave of its run
   const unsigned key_offset = (unsigned)(((((lane >> 4) & 1) * 8 + (lane >> 5) * 4 + wave) * D + (lane & 15) * 8) * 2);
   // lane l of a value block brings dimension 32 wave + l / 2, keys 8 (l % 2) .. + 7 of the run
-  const unsigned value_offset = (unsigned)((((wave * 32 + (lane >> 1)) * page_size) + (lane & 1) * 8) * 2);
+  // (values narrower than keys: the dims behind them repeat the last one)
+  const int value_dim = wave * 32 + (lane >> 1) < dv ? wave * 32 + (lane >> 1) : dv - 1;
+  const unsigned value_offset = (unsigned)(((value_dim * page_size) + (lane & 1) * 8) * 2);
   const unsigned keys_address = (unsigned)(uintptr_t)(__attribute__((address_space(3))) unsigned char*)key_tiles;
   const unsigned values_address = (unsigned)(uintptr_t)(__attribute__((address_space(3))) unsigned char*)value_tiles;
   // Where a run of 16 keys lies in memory.  Everything about it is the same for the whole workgroup, so the
   // page comes from the block table by a scalar load and the rest is a handful of scalar instructions; a
   // tile's two pages are asked for a turn before its addresses are wanted.  A run no query sees is masked:
   // any page with numbers in it will do, so runs are clamped to those the queries do see.
-  const unsigned page_bytes = (unsigned)(nkv * page_size * D * 2);   // from page to page, keys and values alike
+  const unsigned page_bytes = (unsigned)(nkv * page_size * D * 2);   // from page to page of keys ...
+  const unsigned value_page_bytes = (unsigned)(nkv * page_size * dv * 2);   // ... and of values
   const char* const k_head = (const char*)(k_pages + (int64_t)kvh * page_size * D);
-  const char* const v_head = (const char*)(v_pages + (int64_t)kvh * page_size * D);
+  const char* const v_head = (const char*)(v_pages + (int64_t)kvh * page_size * dv);
   // INSIDE: the tile lies behind the first of the walk, so that only the far end needs the clamp
   auto run_in_reach = [&](auto inside, int tile, int half) {
     const int run = tile * 2 + half;
@@ -1220,15 +1265,15 @@ __global__ __launch_bounds__(MANY_WAVES ? 512 : 256, MANY_WAVES ? 1 : 2) void at
   auto locate = [&](auto inside, int tile, const int (&pages)[2], const char* (&kbase)[2], const char* (&vbase)[2]) {
 #pragma unroll
     for (int half = 0; half < 2; ++half) {
-      const uint64_t at = (uint64_t)(unsigned)pages[half] * page_bytes;
+      const uint64_t at = (uint64_t)(unsigned)pages[half] * page_bytes, value_at = (uint64_t)(unsigned)pages[half] * value_page_bytes;
       if (pages16 > 1) {
         const int run = run_in_reach(inside, tile, half);
         const unsigned off = (unsigned)(run - (int)__umulhi((unsigned)run, magic) * pages16) * 16u;
         kbase[half] = k_head + at + off * (unsigned)(D * 2);
-        vbase[half] = v_head + at + off * 2u;
+        vbase[half] = v_head + value_at + off * 2u;
       } else {
         kbase[half] = k_head + at;
-        vbase[half] = v_head + at;
+        vbase[half] = v_head + value_at;
       }
     }
   };
@@ -1295,8 +1340,27 @@ __global__ __launch_bounds__(MANY_WAVES ? 512 : 256, MANY_WAVES ? 1 : 2) void at
 #pragma unroll
           for (int i = 0; i < 4; ++i) sc[b][h][i] = capped(sc[b][h][i], cap);
     };
+    // the bias by distance, likewise; sc[b][h][i] belongs to key tile * 32 + 8 m + 4 h + i (a key ahead of the query gives no
+    // number here; the mask takes it out)
+    float rate = 0.f, reach = 0.f;
+    if constexpr (DISTANCE) {
+      const int biased = active ? head : head0;
+      rate = distance[biased] * LN2 / scale;
+      reach = distance[nq + biased];
+    }
+    auto take_off_distance = [&](int tile, floatx4 (&sc)[QB][2]) {
+#pragma unroll
+      for (int b = 0; b < QB; ++b) {
+        const float behind = (float)((live[b] ? pos[b] : pos_last) - (tile * 32 + key_chunk * 8));
+        const float first = fmaf(reach, behind, 1.f);
+#pragma unroll
+        for (int h = 0; h < 2; ++h)
+#pragma unroll
+          for (int i = 0; i < 4; ++i) sc[b][h][i] = fmaf(-rate, __builtin_amdgcn_logf(fmaf(-reach, (float)(4 * h + i), first)), sc[b][h][i]);
+      }
+    };
     // scores: S[key, query] = K Q^T, unscaled (the scale enters with the exponent)
-    auto scores = [&](int stage, floatx4 (&sc)[QB][2]) {
+    auto scores = [&](int tile, int stage, floatx4 (&sc)[QB][2]) {
       const unsigned char* kt = key_tiles + stage * KBYTES + key_fragment;
 #pragma unroll
       for (int b = 0; b < QB; ++b) sc[b][0] = sc[b][1] = floatx4{0.f, 0.f, 0.f, 0.f};
@@ -1309,6 +1373,7 @@ __global__ __launch_bounds__(MANY_WAVES ? 512 : 256, MANY_WAVES ? 1 : 2) void at
           for (int b = 0; b < QB; ++b) sc[b][h] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kfrag, qf[b][c], sc[b][h], 0, 0, 0);
         }
       if constexpr (CAPPED) cap_scores(sc);
+      if constexpr (DISTANCE) take_off_distance(tile, sc);
     };
     // weights: as in attention_prefill_bf16_kernel; sc[b][h][i] belongs to key tile * 32 + 8 m + 4 h + i
     auto weights_with_maximum = [&](int tile, floatx4 (&sc)[QB][2], auto masked, bf16x8 (&pf)[QB]) {
@@ -1363,7 +1428,7 @@ __global__ __launch_bounds__(MANY_WAVES ? 512 : 256, MANY_WAVES ? 1 : 2) void at
     // three or four vector instructions of a weight cost nothing.  A head of 128 has as many products a tile
     // (8 for every 16 queries) as a lane has weights.  Returns false, and has changed nothing but pf and
     // next, if a weight sum says the reference point will not do.
-    auto weights_beside_scores = [&](int stage, floatx4 (&sc)[QB][2], floatx4 (&next)[QB][2], bf16x8 (&pf)[QB]) -> bool {
+    auto weights_beside_scores = [&](int next_tile, int stage, floatx4 (&sc)[QB][2], floatx4 (&next)[QB][2], bf16x8 (&pf)[QB]) -> bool {
       const unsigned char* kt = key_tiles + stage * KBYTES + key_fragment;
       constexpr int FRAGMENTS = 2 * DS, READ_AHEAD = 3;
       static_assert(FRAGMENTS * QB == QB * 8, "one weight for every product");
@@ -1400,6 +1465,7 @@ __global__ __launch_bounds__(MANY_WAVES ? 512 : 256, MANY_WAVES ? 1 : 2) void at
 #pragma unroll
       for (int b = 0; b < QB; ++b) run_sum[b] += tile_sum[b];
       if constexpr (CAPPED) cap_scores(next);
+      if constexpr (DISTANCE) take_off_distance(next_tile, next);
       return true;
     };
     // values: O^T[dim, query] += V^T P
@@ -1450,7 +1516,7 @@ __global__ __launch_bounds__(MANY_WAVES ? 512 : 256, MANY_WAVES ? 1 : 2) void at
       if (pending == 4) fetched_then_barrier<4>();
       else if (pending == 2) fetched_then_barrier<2>();
       else fetched_then_barrier<0>();
-      if (!IDLE_WAVES || active) scores(0, sa);
+      if (!IDLE_WAVES || active) scores(first_tile, 0, sa);
       asm volatile("s_barrier" ::: "memory");                  // everyone has read the first keys: their stage may be filled again
     }
     int tile = first_tile, stage = 0;                          // stage = (tile - first_tile) % 3
@@ -1491,7 +1557,7 @@ __global__ __launch_bounds__(MANY_WAVES ? 512 : 256, MANY_WAVES ? 1 : 2) void at
       for (;;) {
         if (asked || tile < fast_begin || tile >= fast_end) break;
         ask_ahead(std::true_type{});
-        if (!weights_beside_scores(stage == STAGES - 1 ? 0 : stage + 1, sa, sb, pf)) {
+        if (!weights_beside_scores(tile + 1, stage == STAGES - 1 ? 0 : stage + 1, sa, sb, pf)) {
           asked = true;
           continue;
         }
@@ -1503,7 +1569,7 @@ __global__ __launch_bounds__(MANY_WAVES ? 512 : 256, MANY_WAVES ? 1 : 2) void at
       const bool unfinished = tile <= last_tile;
       if (!unfinished) break;
       const int pending = asked ? 4 : ask_ahead(std::false_type{});
-      if (tile < last_tile) scores(stage == STAGES - 1 ? 0 : stage + 1, sb);
+      if (tile < last_tile) scores(tile + 1, stage == STAGES - 1 ? 0 : stage + 1, sb);
       if (tile >= whole_begin && tile < whole_end) weights_with_maximum(tile, sa, std::false_type{}, pf);
       else weights_with_maximum(tile, sa, std::true_type{}, pf);
       values(stage, pf);
@@ -1519,7 +1585,8 @@ __global__ __launch_bounds__(MANY_WAVES ? 512 : 256, MANY_WAVES ? 1 : 2) void at
       if (live[b] && slots > 1) {
         const int64_t slot = ((int64_t)(token0 + b * 16 + col) * nq + head) * slots + split;
 #pragma unroll
-        for (int e = 0; e < DB; ++e) *(floatx4*)(part_o + slot * D + e * 16 + g * 4) = o[b][e];
+        for (int e = 0; e < DB; ++e)
+          if (e * 16 < dv) *(floatx4*)(part_o + slot * dv + e * 16 + g * 4) = o[b][e];
         if (g == 0) {
           part_ml[slot * 2] = run_max[b] * scale2;               // -inf stays -inf: no key seen
           part_ml[slot * 2 + 1] = total;
@@ -1527,9 +1594,10 @@ __global__ __launch_bounds__(MANY_WAVES ? 512 : 256, MANY_WAVES ? 1 : 2) void at
       } else if (live[b]) {
         const float keep = sinks ? with_sink(sinks[head] * LOG2E, run_max[b] * scale2, total) : 1.f;
         const float inv = keep / total * head_gate(gates, gate_stride, token0 + b * 16 + col, head);
-        bf16* dst = out + (int64_t)(token0 + b * 16 + col) * out_stride + (int64_t)head * D + g * 4;
+        bf16* dst = out + (int64_t)(token0 + b * 16 + col) * out_stride + (int64_t)head * dv + g * 4;
 #pragma unroll
         for (int e = 0; e < DB; ++e) {
+          if (e * 16 >= dv) break;
           const bf16x4 packed = {(bf16)(o[b][e][0] * inv), (bf16)(o[b][e][1] * inv), (bf16)(o[b][e][2] * inv), (bf16)(o[b][e][3] * inv)};
           *(bf16x4*)(dst + e * 16) = packed;
         }
@@ -1585,7 +1653,8 @@ LRS_API int lrs_attention_prefill(void* out, int out_stride, const void* q, int 
                                   int nkv, int d, int page_size, float scale, int window, int keep_first, int tokens, int splits,
                                   float* part_o, float* part_ml, int prepare, const void* q_weight, int w_dtype, float eps,
                                   const float* cosv, const float* sinv, const float* sinks, float softcap, const void* gates,
-                                  int gate_stride, void* stream) {
+                                  int gate_stride, int dv, const float* distance, void* stream) {
+  LRS_REQUIRE(dv > 0 && dv % 16 == 0 && dv <= d, "attention_prefill: values of %d dims beside keys of %d are not served (a multiple of 16, at most the keys')", dv, d);
   LRS_REQUIRE(n_blocks > 0 && nq > 0 && nkv > 0 && nq % nkv == 0, "attention_prefill: bad sizes blocks=%d nq=%d nkv=%d", n_blocks, nq, nkv);
   if (prepare) {
     LRS_REQUIRE(lrs_attention_prefill_prepares(d), "attention_prefill: only the kernel for heads of 128 prepares the queries itself, got head_dim %d", d);
@@ -1624,7 +1693,7 @@ LRS_API int lrs_attention_prefill(void* out, int out_stride, const void* q, int 
                                                               (const bf16*)k_pages, (const bf16*)v_pages, block_table, \
                                                               table_stride, token_request, positions, qblock_token0, \
                                                               qblock_count, n_blocks, chunk, nq, nkv, page_size, scale, window, \
-                                                              splits, slots, part_o, part_ml, own_sinks, softcap, own_gates, gate_stride)
+                                                              splits, slots, part_o, part_ml, own_sinks, softcap, own_gates, gate_stride, dv, distance)
 #define LAUNCH(D)                                \
   if (max_count <= 16) LAUNCH2(D, 1);            \
   else LAUNCH2(D, 2)
@@ -1641,13 +1710,15 @@ LRS_API int lrs_attention_prefill(void* out, int out_stride, const void* q, int 
         const bool many = nq / nkv > 4 && (int64_t)n_blocks * nkv * splits <= 2 * compute_units();
         if (many) block = dim3((nq / nkv < 8 ? nq / nkv : 8) * WAVE);
 #define D128(QB, MANY, IDLE)                                                                                                      \
-        if (softcap > 0.f) D128C(QB, MANY, IDLE, true);                                                                               \
-        else D128C(QB, MANY, IDLE, false)
-#define D128C(QB, MANY, IDLE, CAPPED)                                                                                             \
-        attention_prefill_d128_bf16_kernel<QB, MANY, IDLE, CAPPED><<<grid, block, 0, s>>>(                                            \
+        if (softcap > 0.f && distance) D128C(QB, MANY, IDLE, SCORES_BOTH);                                                            \
+        else if (softcap > 0.f) D128C(QB, MANY, IDLE, SCORES_CAPPED);                                                                 \
+        else if (distance) D128C(QB, MANY, IDLE, SCORES_DISTANCE);                                                                    \
+        else D128C(QB, MANY, IDLE, SCORES_PLAIN)
+#define D128C(QB, MANY, IDLE, SCORES)                                                                                             \
+        attention_prefill_d128_bf16_kernel<QB, MANY, IDLE, SCORES><<<grid, block, 0, s>>>(                                            \
             (bf16*)out, out_stride, (const bf16*)q, q_stride, (const bf16*)k_pages, (const bf16*)v_pages, block_table, table_stride, \
             token_request, positions, qblock_token0, qblock_count, n_blocks, chunk, nq, nkv, page_size, scale, window, splits, slots, part_o, part_ml, \
-            prepare, prep, own_sinks, softcap, own_gates, gate_stride)
+            prepare, prep, own_sinks, softcap, own_gates, gate_stride, dv, distance)
 #define D128_OF(QB)                                        \
         if (many && idle) { D128(QB, true, true); }        \
         else if (many) { D128(QB, true, false); }          \
@@ -1669,11 +1740,11 @@ LRS_API int lrs_attention_prefill(void* out, int out_stride, const void* q, int 
   if (lrs_check_launch("attention_prefill")) return 1;
   if (keep_first > 0) {
     launch_attention_kept((const bf16*)q, q_stride, (const bf16*)k_pages, (const bf16*)v_pages, block_table, table_stride, token_request,
-                          positions, tokens, nq, nkv, d, page_size, scale, window, keep_first, slots, part_o, part_ml, softcap, s);
+                          positions, tokens, nq, nkv, d, page_size, scale, window, keep_first, slots, part_o, part_ml, softcap, dv, distance, s);
     if (lrs_check_launch("attention_kept")) return 1;
   }
   if (slots > 1) {
-    launch_attention_merge((bf16*)out, out_stride, part_o, part_ml, tokens, nq, d, slots, sinks, (const bf16*)gates, gate_stride, s);
+    launch_attention_merge((bf16*)out, out_stride, part_o, part_ml, tokens, nq, dv, slots, sinks, (const bf16*)gates, gate_stride, s);
     return lrs_check_launch("attention_merge");
   }
   return 0;
@@ -1687,7 +1758,7 @@ LRS_API int lrs_attention(void* out, int out_stride, const void* q, int q_stride
                           const void* v_pages, const int* block_table, int table_stride,
                           const int* token_request, const int* positions, int dtype, int tokens,
                           int nq, int nkv, int d, int dv, int page_size, float scale, int window, int keep_first,
-                          const float* sinks, float softcap, const void* gates, int gate_stride, void* stream) {
+                          const float* sinks, float softcap, const void* gates, int gate_stride, const float* distance, void* stream) {
   // value pages [P, nkv, dv, page]; out rows hold nq heads of dv values
   LRS_REQUIRE(tokens > 0 && nq > 0 && nkv > 0 && d > 0 && dv > 0 && page_size > 0, "attention: bad sizes tokens=%d nq=%d nkv=%d d=%d dv=%d page=%d", tokens, nq, nkv, d, dv, page_size);
   LRS_REQUIRE(nq % nkv == 0, "attention: %d query heads do not divide into %d kv heads", nq, nkv);
@@ -1701,11 +1772,11 @@ LRS_API int lrs_attention(void* out, int out_stride, const void* q, int q_stride
   if (dtype == LRS_F32)
     attention_generic_kernel<float, THREADS><<<grid, THREADS, lds, s>>>(
         (float*)out, out_stride, (const float*)q, q_stride, (const float*)k_pages, (const float*)v_pages,
-        block_table, table_stride, token_request, positions, nq, nkv, d, dv, page_size, scale, window, keep_first, sinks, softcap, (const float*)gates, gate_stride);
+        block_table, table_stride, token_request, positions, nq, nkv, d, dv, page_size, scale, window, keep_first, sinks, softcap, (const float*)gates, gate_stride, distance);
   else if (dtype == LRS_BF16)
     attention_generic_kernel<bf16, THREADS><<<grid, THREADS, lds, s>>>(
         (bf16*)out, out_stride, (const bf16*)q, q_stride, (const bf16*)k_pages, (const bf16*)v_pages,
-        block_table, table_stride, token_request, positions, nq, nkv, d, dv, page_size, scale, window, keep_first, sinks, softcap, (const bf16*)gates, gate_stride);
+        block_table, table_stride, token_request, positions, nq, nkv, d, dv, page_size, scale, window, keep_first, sinks, softcap, (const bf16*)gates, gate_stride, distance);
   else
     return lrs_fail("attention: unknown dtype %d", dtype);
   return lrs_check_launch("attention");

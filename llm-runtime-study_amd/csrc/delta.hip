@@ -1,5 +1,6 @@
 // Linear-recurrent mixers whose state per head is a matrix S [dim, vdim] in float32: the gated delta rule (with one
-// decay a head, or one a head and key channel) and the selective state space recurrence (at the end of this file).
+// decay a head, or one a head and key channel), the selective state space recurrence and the matrix memory with exponential
+// gates (mLSTM; both at the end of this file).
 //
 // For every token, with q and k unit vectors of the head's key group, v the head's value, beta in (0, 1) the
 // step size and g in (0, 1) the decay:
@@ -129,20 +130,28 @@ __device__ __forceinline__ float row_sum16(float v) {
 //
 // RULE says which recurrence: RULE_DELTA as above; RULE_PLAIN without the correction (u = v: S <- g S + k v^T, what a
 // state space layer does with k = B, q = C, v = dt x); RULE_DELTA_CHANNELS with a decay per key channel (decays
-// [tokens, H * d]: row i of S is multiplied by its own decay first, then the rule runs with g = 1).
-enum { RULE_DELTA = 0, RULE_PLAIN = 1, RULE_DELTA_CHANNELS = 2 };
+// [tokens, H * d]: row i of S is multiplied by its own decay first, then the rule runs with g = 1); RULE_WEIGHTED without the
+// correction and with a weight on what is written (u = beta v), S having one column more than the values: its value is always
+// one, so that column is the running sum of the weighted keys and its read-out n . q.
+enum { RULE_DELTA = 0, RULE_PLAIN = 1, RULE_DELTA_CHANNELS = 2, RULE_WEIGHTED = 3 };
+
+// Where a token's queries, keys and values lie: rows of `ld` floats, the parts' first columns (each head after head).
+struct ScanRows {
+  int ld, q_at, k_at, v_at;
+};
 
 template <int ROWS, int CHUNK, int RULE>
 __global__ __launch_bounds__(256) void delta_scan_kernel(const float* __restrict__ qkv, const float* __restrict__ gates,
                                                          const int* __restrict__ cu, const int* __restrict__ slot_ids,
                                                          float* __restrict__ state, int64_t state_stride, int G, int H, int d,
-                                                         int dv, float* __restrict__ raw_out, const float* __restrict__ decays) {
+                                                         int dv, float* __restrict__ raw_out, const float* __restrict__ decays, ScanRows at) {
   constexpr int VECTORS = RULE == RULE_DELTA_CHANNELS ? 3 : 2;    // arrays of CHUNK x dpad values a buffer holds: k, q (, decays)
   constexpr int K4 = ROWS / 4;                 // float4 pieces of a thread's slice of a key
   constexpr int rows = ROWS;
   extern __shared__ __attribute__((aligned(16))) float lds[];
   const int r = blockIdx.x, h = blockIdx.y, block = blockIdx.z, tid = threadIdx.x;
-  const int dpad = rows * SPLIT, channels = 2 * G * d + H * dv, hk = h / (H / G);
+  const int dpad = rows * SPLIT, hk = h / (H / G);
+  const int values = RULE == RULE_WEIGHTED ? dv - 1 : dv;       // columns of S that have values of their own
   const int per_buffer = CHUNK * (VECTORS * dpad + COLUMNS + 4);
   const int c = tid / SPLIT, s = tid % SPLIT, column = block * COLUMNS + c;
   const bool mine = column < dv;
@@ -158,7 +167,7 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(const float* __restrict
   float4 k_reg[KQ], q_reg[KQ], g_reg[RULE == RULE_DELTA_CHANNELS ? KQ : 1];
   float v_reg = 0.f, scalar_reg = 0.f;
   const int pieces = CHUNK * dpad / 4, row_pieces = dpad / 4;
-  const bool d_whole = d % 4 == 0 && channels % 4 == 0;     // every piece of four is 16 bytes aligned
+  const bool d_whole = d % 4 == 0 && at.ld % 4 == 0 && at.q_at % 4 == 0 && at.k_at % 4 == 0;     // every piece of four is 16 bytes aligned
   auto fetch = [&](int c0) {
     const int count = min(CHUNK, n - c0);
 #pragma unroll
@@ -180,16 +189,16 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(const float* __restrict
         }
       }
       if (e < pieces && tt < count) {
-        const float* row = qkv + (int64_t)(start + c0 + tt) * channels + hk * d + i;
+        const float* row = qkv + (int64_t)(start + c0 + tt) * at.ld + hk * d + i;
         if (d_whole && i + 4 <= d) {
-          q_reg[p] = *(const float4*)row;
-          k_reg[p] = *(const float4*)(row + G * d);
+          q_reg[p] = *(const float4*)(row + at.q_at);
+          k_reg[p] = *(const float4*)(row + at.k_at);
         } else {
           float kq[8] = {};
           for (int x = 0; x < 4; ++x)
             if (i + x < d) {
-              kq[x] = row[x];
-              kq[4 + x] = row[G * d + x];
+              kq[x] = row[at.q_at + x];
+              kq[4 + x] = row[at.k_at + x];
             }
           q_reg[p] = make_float4(kq[0], kq[1], kq[2], kq[3]);
           k_reg[p] = make_float4(kq[4], kq[5], kq[6], kq[7]);
@@ -197,7 +206,8 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(const float* __restrict
       }
     }
     const int tt = tid / COLUMNS, cc = tid % COLUMNS;
-    v_reg = (tt < CHUNK && tt < count && block * COLUMNS + cc < dv) ? qkv[(int64_t)(start + c0 + tt) * channels + 2 * G * d + h * dv + block * COLUMNS + cc] : 0.f;
+    v_reg = (tt < CHUNK && tt < count && block * COLUMNS + cc < values) ? qkv[(int64_t)(start + c0 + tt) * at.ld + at.v_at + h * values + block * COLUMNS + cc] : 0.f;
+    if (RULE == RULE_WEIGHTED && block * COLUMNS + cc == values) v_reg = 1.f;
     scalar_reg = 0.f;
     if (tid < 2 * CHUNK && tid / 2 < count) scalar_reg = gates[(int64_t)(start + c0 + tid / 2) * 2 * H + (tid % 2) * H + h];
   };
@@ -248,11 +258,11 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(const float* __restrict
         dq = fmaf(S[i], qq[i], dq);
         kq = fmaf(kk[i], qq[i], kq);
       }
-      if constexpr (RULE != RULE_PLAIN) dk = row_sum16(dk);
+      if constexpr (RULE != RULE_PLAIN && RULE != RULE_WEIGHTED) dk = row_sum16(dk);
       dq = row_sum16(dq);
       kq = row_sum16(kq);
       const float beta = g_l[4 * tt], g = RULE == RULE_DELTA_CHANNELS ? 1.f : g_l[4 * tt + 1];
-      const float u = RULE == RULE_PLAIN ? v_l[tt * COLUMNS + c] : beta * (v_l[tt * COLUMNS + c] - g * dk);
+      const float u = RULE == RULE_PLAIN ? v_l[tt * COLUMNS + c] : RULE == RULE_WEIGHTED ? beta * v_l[tt * COLUMNS + c] : beta * (v_l[tt * COLUMNS + c] - g * dk);
 #pragma unroll
       for (int i = 0; i < ROWS; ++i) S[i] = fmaf(kk[i], u, g * S[i]);
       if (s == 0 && mine) raw_out[(int64_t)(start + c0 + tt) * H * dv + h * dv + column] = fmaf(u, kq, g * dq);
@@ -463,15 +473,16 @@ __global__ __launch_bounds__(256) void ssm_gate_kernel(const float* __restrict__
 template <int RULE>
 void launch_scan(int rows, bool single, dim3 grid, hipStream_t s, const float* qkv, const float* gates, const int* cu, const int* slot_ids,
                  float* state, int64_t state_stride, int G, int H, int d, int dv, float* raw, const float* decays) {
+  const ScanRows at{2 * G * d + H * dv, 0, G * d, 2 * G * d};
   const int chunk = rows == 16 ? 8 : 16, vectors = RULE == RULE_DELTA_CHANNELS ? 3 : 2;
   const size_t lds = (size_t)2 * chunk * (vectors * rows * SPLIT + COLUMNS + 4) * sizeof(float);
   if (single) {        // one token each: token r is request r's
     if (rows == 4) delta_scan_single_kernel<4, RULE><<<grid, 256, 0, s>>>(qkv, gates, slot_ids, state, state_stride, G, H, d, dv, raw, decays);
     else if (rows == 8) delta_scan_single_kernel<8, RULE><<<grid, 256, 0, s>>>(qkv, gates, slot_ids, state, state_stride, G, H, d, dv, raw, decays);
     else delta_scan_single_kernel<16, RULE><<<grid, 256, 0, s>>>(qkv, gates, slot_ids, state, state_stride, G, H, d, dv, raw, decays);
-  } else if (rows == 4) delta_scan_kernel<4, 16, RULE><<<grid, 256, lds, s>>>(qkv, gates, cu, slot_ids, state, state_stride, G, H, d, dv, raw, decays);
-  else if (rows == 8) delta_scan_kernel<8, 16, RULE><<<grid, 256, lds, s>>>(qkv, gates, cu, slot_ids, state, state_stride, G, H, d, dv, raw, decays);
-  else delta_scan_kernel<16, 8, RULE><<<grid, 256, lds, s>>>(qkv, gates, cu, slot_ids, state, state_stride, G, H, d, dv, raw, decays);
+  } else if (rows == 4) delta_scan_kernel<4, 16, RULE><<<grid, 256, lds, s>>>(qkv, gates, cu, slot_ids, state, state_stride, G, H, d, dv, raw, decays, at);
+  else if (rows == 8) delta_scan_kernel<8, 16, RULE><<<grid, 256, lds, s>>>(qkv, gates, cu, slot_ids, state, state_stride, G, H, d, dv, raw, decays, at);
+  else delta_scan_kernel<16, 8, RULE><<<grid, 256, lds, s>>>(qkv, gates, cu, slot_ids, state, state_stride, G, H, d, dv, raw, decays, at);
 }
 
 }  // namespace
@@ -601,4 +612,216 @@ LRS_API int lrs_ssm(void* out, int out_dtype, const void* proj, int proj_dtype, 
   else return lrs_fail("ssm: projections in dtype %d with outputs in dtype %d are not served", proj_dtype, out_dtype);
 #undef ALL
   return lrs_check_launch("ssm");
+}
+
+// ------------------------------------------------------------------ matrix memory with exponential gates (mLSTM)
+// Per head, with log gates i = cap tanh((i_in + i_bias) / cap) and f = log(sigmoid(cap tanh((f_in + f_bias) / cap))) and a running
+// maximum m (0 at a sequence's start):
+//     m' = max(f + m, i);   S <- exp(f + m - m') S + exp(i - m') k v^T;   n <- exp(f + m - m') n + exp(i - m') k
+//     o = S^T q / (max(|n . q|, exp(-m')) + 1e-6)
+// n is kept as one more column of S (RULE_WEIGHTED), q comes without its factor 1 / sqrt(d), which the read-out applies.
+//   mlstm_gates  per (request, head): walks the request's tokens for m; the two factors of every token, and exp(-m);
+//   delta_scan   as above, straight from the projection rows;
+//   mlstm_single steps of one token a request: gates and recurrence in one kernel, a workgroup 16 columns of a head's matrix;
+//   mlstm_read   per (token, head): the read-out over its normaliser, divided by its root mean square, times the norm's weight,
+//                times the sigmoid of the output gate.
+// A request's state row: S of every head (d padded to 16 lanes of rows, vdim + 1 columns), then m of every head.
+namespace {
+
+struct LogGates {
+  float input, forget;
+};
+__device__ __forceinline__ LogGates log_gates(float i_in, float f_in, float cap) {
+  const float y = cap * tanhf(f_in / cap);
+  return {cap * tanhf(i_in / cap), fminf(y, 0.f) - log1pf(expf(-fabsf(y)))};
+}
+
+// gates [tokens, 2 * H]: exp(i - m'), then exp(f + m - m') of every head (the order of the scan's scalars); floors [tokens, H].
+__global__ __launch_bounds__(WAVE) void mlstm_gates_kernel(const float* __restrict__ proj, int ld, int i_at, int f_at, const int* __restrict__ cu,
+                                                           const int* __restrict__ slot_ids, float* __restrict__ state, int64_t state_stride,
+                                                           int64_t m_offset, int H, const float* __restrict__ i_bias,
+                                                           const float* __restrict__ f_bias, float cap, float* __restrict__ gates,
+                                                           float* __restrict__ floors) {
+  const int r = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
+  const int start = cu[r], n = cu[r + 1] - start;
+  float* kept = state + (int64_t)slot_ids[r] * state_stride + m_offset + h;
+  const float ib = i_bias[h], fb = f_bias[h];
+  float m = *kept;
+  for (int c0 = 0; c0 < n; c0 += WAVE) {
+    const int count = min(WAVE, n - c0);
+    const int64_t token = start + c0 + min(lane, count - 1);
+    const LogGates log_gate = log_gates(proj[token * ld + i_at + h] + ib, proj[token * ld + f_at + h] + fb, cap);
+    // the maximum goes from token to token: the lanes' gates in turn, each lane keeping the value before and after its own token
+    float before = 0.f, after = 0.f;
+    for (int t = 0; t < count; ++t) {
+      const float f = __int_as_float(__builtin_amdgcn_readlane(__float_as_int(log_gate.forget), t));
+      const float i = __int_as_float(__builtin_amdgcn_readlane(__float_as_int(log_gate.input), t));
+      const float next = fmaxf(f + m, i);
+      before = lane == t ? m : before;
+      after = lane == t ? next : after;
+      m = next;
+    }
+    if (lane < count) {
+      gates[token * 2 * H + h] = expf(log_gate.input - after);
+      gates[token * 2 * H + H + h] = expf(log_gate.forget + before - after);
+      floors[token * H + h] = expf(-after);
+    }
+  }
+  if (lane == 0) *kept = m;
+}
+
+template <int ROWS>
+__global__ __launch_bounds__(256) void mlstm_single_kernel(const float* __restrict__ proj, ScanRows at, int i_at, int f_at,
+                                                           const int* __restrict__ slot_ids, float* __restrict__ state, int64_t state_stride,
+                                                           int64_t m_offset, int H, int d, int dv, const float* __restrict__ i_bias,
+                                                           const float* __restrict__ f_bias, float cap, float* __restrict__ raw_out,
+                                                           float* __restrict__ floors, float* __restrict__ maxima) {
+  // dv: columns of S, the values' and the one of the normaliser; the new m goes to `maxima` [requests, H] (every workgroup of the
+  // head reads the old one from the state row) and from there into the row by the read-out
+  const int r = blockIdx.x, h = blockIdx.y, block = blockIdx.z, tid = threadIdx.x;
+  const int c = tid / SPLIT, s = tid % SPLIT, column = block * COLUMNS + c;
+  if (column >= dv) return;
+  float* own = state + (int64_t)slot_ids[r] * state_stride;
+  float* st = own + (int64_t)h * ROWS * dv * SPLIT + (int64_t)block * COLUMNS * SPLIT;
+  const float* row = proj + (int64_t)r * at.ld;
+  float S[ROWS], kk[ROWS], qq[ROWS];
+#pragma unroll
+  for (int i = 0; i < ROWS; ++i) S[i] = st[(int64_t)i * dv * SPLIT + tid];
+  const float before = own[m_offset + h];
+  const float* q = row + at.q_at + h * d;
+  const float* k = row + at.k_at + h * d;
+  if (d % 4 == 0 && at.ld % 4 == 0 && at.q_at % 4 == 0 && at.k_at % 4 == 0) {
+#pragma unroll
+    for (int p = 0; p < ROWS / 4; ++p) {
+      const int i = s * ROWS + 4 * p;
+      const float4 zero = make_float4(0.f, 0.f, 0.f, 0.f);
+      const float4 a = i < d ? *(const float4*)(q + i) : zero, b = i < d ? *(const float4*)(k + i) : zero;
+      qq[4 * p] = a.x, qq[4 * p + 1] = a.y, qq[4 * p + 2] = a.z, qq[4 * p + 3] = a.w;
+      kk[4 * p] = b.x, kk[4 * p + 1] = b.y, kk[4 * p + 2] = b.z, kk[4 * p + 3] = b.w;
+    }
+  } else {
+#pragma unroll
+    for (int p = 0; p < ROWS; ++p) {
+      const int i = s * ROWS + p;
+      qq[p] = i < d ? q[i] : 0.f;
+      kk[p] = i < d ? k[i] : 0.f;
+    }
+  }
+  const float v = column < dv - 1 ? row[at.v_at + h * (dv - 1) + column] : 1.f;
+  const LogGates log_gate = log_gates(row[i_at + h] + i_bias[h], row[f_at + h] + f_bias[h], cap);
+  const float m = fmaxf(log_gate.forget + before, log_gate.input);
+  const float g = expf(log_gate.forget + before - m), u = expf(log_gate.input - m) * v;
+  float dq = 0.f, kq = 0.f;
+#pragma unroll
+  for (int i = 0; i < ROWS; ++i) {
+    dq = fmaf(S[i], qq[i], dq);
+    kq = fmaf(kk[i], qq[i], kq);
+  }
+  dq = row_sum16(dq);
+  kq = row_sum16(kq);
+#pragma unroll
+  for (int i = 0; i < ROWS; ++i) st[(int64_t)i * dv * SPLIT + tid] = fmaf(kk[i], u, g * S[i]);
+  if (s == 0) raw_out[((int64_t)r * H + h) * dv + column] = fmaf(u, kq, g * dq);
+  if (tid == 0 && block == 0) {
+    floors[(int64_t)r * H + h] = expf(-m);
+    maxima[(int64_t)r * H + h] = m;
+  }
+}
+
+// A wave a (token, head).  raw [tokens, H, dv + 1]: the read-out and, last, n . q (both without q's factor).  maxima given (steps
+// of one token a request): the request's new m, moved into its state row here.
+template <typename TO>
+__global__ __launch_bounds__(256) void mlstm_read_kernel(const float* __restrict__ raw, const float* __restrict__ floors,
+                                                         const float* __restrict__ proj, int ld, int g_at, const float* __restrict__ norm_w,
+                                                         float q_factor, float eps, int tokens, int H, int dv, TO* __restrict__ out,
+                                                         const float* __restrict__ maxima, const int* __restrict__ slot_ids,
+                                                         float* __restrict__ state, int64_t state_stride, int64_t m_offset) {
+  const int64_t pair = (int64_t)blockIdx.x * (blockDim.x / WAVE) + threadIdx.x / WAVE;
+  const int lane = threadIdx.x % WAVE;
+  if (pair >= (int64_t)tokens * H) return;
+  const int64_t token = pair / H;
+  const int h = (int)(pair % H);
+  const float* o = raw + pair * (dv + 1);
+  const float* gate = proj + token * ld + g_at + (int64_t)h * dv;
+  const float scale = q_factor / (fmaxf(fabsf(o[dv] * q_factor), floors[pair]) + 1e-6f);
+  constexpr int HELD = 8;                 // heads of up to 512 values stay in registers between the sum and the norm
+  float x[HELD], z[HELD];
+  float ss = 0.f;
+#pragma unroll
+  for (int n = 0; n < HELD; ++n) {        // every load is on its way before the first is used
+    const int i = lane + n * WAVE;
+    x[n] = i < dv ? o[i] * scale : 0.f;
+    z[n] = i < dv ? gate[i] : 0.f;
+    ss = fmaf(x[n], x[n], ss);
+  }
+  for (int i = lane + HELD * WAVE; i < dv; i += WAVE) ss = fmaf(o[i] * scale, o[i] * scale, ss);
+  ss = wave_sum(ss);
+  const float inv = 1.0f / sqrtf(ss / (float)dv + eps);
+  const float* w = norm_w + (int64_t)h * dv;
+  TO* dst = out + pair * dv;
+#pragma unroll
+  for (int n = 0; n < HELD; ++n) {
+    const int i = lane + n * WAVE;
+    if (i < dv) dst[i] = from_float<TO>(x[n] * inv * w[i] / (1.f + expf(-z[n])));
+  }
+  for (int i = lane + HELD * WAVE; i < dv; i += WAVE) dst[i] = from_float<TO>(o[i] * scale * inv * w[i] / (1.f + expf(-gate[i])));
+  if (maxima && lane == 0) state[(int64_t)slot_ids[token] * state_stride + m_offset + h] = maxima[pair];
+}
+
+}  // namespace
+
+// One step for a ragged batch.  proj [tokens, ld] float32: q (H*d) | k (H*d) | v (H*dv) | output gate (H*dv) | input gate (H) |
+// forget gate (H) | anything.  State rows: H * rows * 16 * (dv + 1) floats, then H.  gates [tokens, 2*H], floors [tokens, H] and raw
+// [tokens, H*(dv+1)] are float32 scratch; norm_w [H*dv]; out [tokens, H*dv] in out_dtype.
+LRS_API int lrs_mlstm(void* out, int out_dtype, const float* proj, int ld, int tokens, int requests, const int* cu, const int* slot_ids,
+                      float* state, int64_t state_stride, int H, int d, int dv, const float* i_bias, const float* f_bias, float cap,
+                      const float* norm_w, float eps, float* gates, float* floors, float* raw, void* stream) {
+  LRS_REQUIRE(tokens > 0 && requests > 0 && requests <= tokens, "mlstm: bad sizes tokens=%d requests=%d", tokens, requests);
+  LRS_REQUIRE(H > 0 && d > 0 && dv > 0, "mlstm: bad sizes H=%d d=%d dv=%d", H, d, dv);
+  LRS_REQUIRE(d <= 256, "mlstm: takes keys of up to 256 values, got %d", d);
+  LRS_REQUIRE(cap > 0.f && eps > 0.f, "mlstm: the gates' cap and eps must be positive");
+  const int rows = lrs_delta_state_rows(d), columns = dv + 1;
+  const ScanRows at{ld, 0, H * d, 2 * H * d};
+  const int g_at = 2 * H * d + H * dv, i_at = g_at + H * dv, f_at = i_at + H;
+  LRS_REQUIRE(ld >= f_at + H, "mlstm: projection rows of %d hold fewer than the %d columns needed", ld, f_at + H);
+  const int64_t m_offset = (int64_t)H * rows * SPLIT * columns;
+  LRS_REQUIRE(state_stride >= m_offset + H, "mlstm: a state row of %lld floats is too short", (long long)state_stride);
+  LRS_REQUIRE(((uintptr_t)proj % 16) == 0, "mlstm: the projection rows must be 16 bytes aligned");
+  LRS_REQUIRE(out_dtype == LRS_F32 || out_dtype == LRS_BF16, "mlstm: unknown dtype %d", out_dtype);
+  hipStream_t s = (hipStream_t)stream;
+  const dim3 sgrid(requests, H, (columns + COLUMNS - 1) / COLUMNS);
+  const bool single = tokens == requests;
+  float* maxima = single ? gates : nullptr;      // (the factors of single tokens never leave their kernel)
+  if (single) {
+#define SINGLE(ROWS)                                                                                                                    \
+  mlstm_single_kernel<ROWS><<<sgrid, 256, 0, s>>>(proj, at, i_at, f_at, slot_ids, state, state_stride, m_offset, H, d, columns, i_bias, \
+                                                  f_bias, cap, raw, floors, maxima)
+    if (rows == 4) SINGLE(4);
+    else if (rows == 8) SINGLE(8);
+    else SINGLE(16);
+#undef SINGLE
+  } else {
+    mlstm_gates_kernel<<<dim3(requests, H), WAVE, 0, s>>>(proj, ld, i_at, f_at, cu, slot_ids, state, state_stride, m_offset, H, i_bias, f_bias,
+                                                          cap, gates, floors);
+    const int chunk = rows == 16 ? 8 : 16;
+    const size_t lds = (size_t)2 * chunk * (2 * rows * SPLIT + COLUMNS + 4) * sizeof(float);
+#define SCAN(ROWS, CHUNK)                                                                                                                    \
+  delta_scan_kernel<ROWS, CHUNK, RULE_WEIGHTED><<<sgrid, 256, lds, s>>>(proj, gates, cu, slot_ids, state, state_stride, H, H, d, columns, raw, \
+                                                                        nullptr, at)
+    if (rows == 4) SCAN(4, 16);
+    else if (rows == 8) SCAN(8, 16);
+    else SCAN(16, 8);
+#undef SCAN
+  }
+  if (lrs_check_launch("mlstm")) return 1;
+  const int64_t pairs = (int64_t)tokens * H;
+  const unsigned blocks = (unsigned)((pairs + 3) / 4);
+  const float q_factor = 1.0f / sqrtf((float)d);
+  if (out_dtype == LRS_F32)
+    mlstm_read_kernel<float><<<blocks, 256, 0, s>>>(raw, floors, proj, ld, g_at, norm_w, q_factor, eps, tokens, H, dv, (float*)out, maxima, slot_ids,
+                                                    state, state_stride, m_offset);
+  else
+    mlstm_read_kernel<bf16><<<blocks, 256, 0, s>>>(raw, floors, proj, ld, g_at, norm_w, q_factor, eps, tokens, H, dv, (bf16*)out, maxima, slot_ids,
+                                                   state, state_stride, m_offset);
+  return lrs_check_launch("mlstm_read");
 }

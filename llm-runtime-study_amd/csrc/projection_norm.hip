@@ -4,37 +4,50 @@
 //   qkv_norm_prep   per token of the fused projection row [q: nq*d | k: nkv*d | v: nkv*dv | ...]: the RMS norm of the
 //                   whole q part and of the whole k part (one sum of squares each, a weight per column), the half-split
 //                   rotation of the first 2*rot_half dims of every q and k head, q written back in place, k into the
-//                   key pages [page, kv_head, slot, d], v into the value pages [page, kv_head, dv, slot];
+//                   key pages [page, kv_head, slot, d], v into the value pages [page, kv_head, dv, slot].  On the way, where
+//                   asked for: a bias per column added before anything else, the queries multiplied by a temperature that
+//                   grows with the position, the values mixed with those of an earlier layer (value_pages.h);
 //   sigmoid_gate    out[t, c] *= sigmoid(gate[t, c / group]): the output gate of the heads, a value a column or one a head;
 //   axpby           out = alpha * a + beta * b over float32 rows: sums of sublayer outputs and the scaled residual add,
 //                   optionally followed by the RMS norm of the new rows (the next layer's input) in the same pass;
 //   activation      out = act(x) elementwise: exact (erf) gelu, tanh gelu, silu, relu.
-#include "common.h"
+#include "value_pages.h"
 
 namespace {
+
+// A query at position p is multiplied by 1 + coef * ln(floor((p + 1) / every) + 1) (every 0: by one).
+struct QueryTemperature {
+  const int* positions;
+  float coef;
+  int every;
+};
+__device__ __forceinline__ float temperature_of(const QueryTemperature& t, int token) {
+  return t.every > 0 ? 1.f + t.coef * logf((float)((t.positions[token] + 1) / t.every) + 1.f) : 1.f;
+}
 
 template <typename T>
 __global__ __launch_bounds__(256) void qkv_norm_prep_kernel(T* __restrict__ qkv, int row_stride, int nq, int nkv, int d, int dv,
                                                             const float* __restrict__ q_weight, const float* __restrict__ k_weight,
                                                             float eps, const float* __restrict__ cosv, const float* __restrict__ sinv,
                                                             int rot_half, T* __restrict__ k_pages, T* __restrict__ v_pages,
-                                                            const int* __restrict__ slots, int page_size) {
+                                                            const int* __restrict__ slots, int page_size, const float* __restrict__ bias,
+                                                            QueryTemperature temperature, ValuePath<T> path) {
   __shared__ float scratch[16];
   const int token = blockIdx.x, tid = threadIdx.x;
   T* row = qkv + (int64_t)token * row_stride;
   const int qn = nq * d, kn = nkv * d, vn = nkv * dv;
   float ssq = 0.f, ssk = 0.f;
   for (int e = tid; e < qn; e += 256) {
-    const float x = to_float(row[e]);
+    const float x = to_float(row[e]) + (bias ? bias[e] : 0.f);
     ssq = fmaf(x, x, ssq);
   }
   for (int e = tid; e < kn; e += 256) {
-    const float x = to_float(row[qn + e]);
+    const float x = to_float(row[qn + e]) + (bias ? bias[qn + e] : 0.f);
     ssk = fmaf(x, x, ssk);
   }
   ssq = block_sum(ssq, scratch);
   ssk = block_sum(ssk, scratch);
-  const float inv_q = q_weight ? 1.0f / sqrtf(ssq / (float)qn + eps) : 1.f;
+  const float inv_q = (q_weight ? 1.0f / sqrtf(ssq / (float)qn + eps) : 1.f) * temperature_of(temperature, token);
   const float inv_k = k_weight ? 1.0f / sqrtf(ssk / (float)kn + eps) : 1.f;
   const int slot = slots ? slots[token] : -1;
   const int64_t page = slot >= 0 ? slot / page_size : 0, off = slot >= 0 ? slot % page_size : 0;
@@ -49,11 +62,12 @@ __global__ __launch_bounds__(256) void qkv_norm_prep_kernel(T* __restrict__ qkv,
     if (!is_q && slot < 0) continue;
     const T* src = row + (int64_t)head * d;
     const float* weight = is_q ? q_weight : k_weight;
+    const float* hb = bias ? bias + (int64_t)head * d : nullptr;
     const int wbase = (is_q ? head : head - nq) * d;
     const float inv = is_q ? inv_q : inv_k;
     T* dst = is_q ? row + (int64_t)head * d : k_pages + ((page * nkv + (head - nq)) * page_size + off) * d;
     if (j < rot_half) {
-      float a = to_float(src[j]) * inv, b = to_float(src[j + rot_half]) * inv;
+      float a = (to_float(src[j]) + (hb ? hb[j] : 0.f)) * inv, b = (to_float(src[j + rot_half]) + (hb ? hb[j + rot_half] : 0.f)) * inv;
       if (weight) {
         a *= weight[wbase + j];
         b *= weight[wbase + j + rot_half];
@@ -63,15 +77,15 @@ __global__ __launch_bounds__(256) void qkv_norm_prep_kernel(T* __restrict__ qkv,
       dst[j + rot_half] = from_float<T>(b * c + a * s);
     } else {
       const int i = j + rot_half;
-      float a = to_float(src[i]) * inv;
+      float a = (to_float(src[i]) + (hb ? hb[i] : 0.f)) * inv;
       if (weight) a *= weight[wbase + i];
       dst[i] = from_float<T>(a);
     }
   }
-  if (slot >= 0) {
+  if (slot >= 0 && v_pages) {           // (null: values_in_runs_kernel stores them)
     for (int e = tid; e < vn; e += 256) {
       const int kvh = e / dv, i = e % dv;
-      v_pages[((page * nkv + kvh) * dv + i) * page_size + off] = row[qn + kn + e];
+      v_pages[((page * nkv + kvh) * dv + i) * page_size + off] = value_on_its_way(path, row[qn + kn + e], qn + kn + e, token, vn, e);
     }
   }
 }
@@ -85,13 +99,21 @@ __global__ __launch_bounds__(256) void qkv_norm_prep_vec_kernel(bf16* __restrict
                                                                 const float* __restrict__ q_weight, const float* __restrict__ k_weight,
                                                                 float eps, const float* __restrict__ cosv, const float* __restrict__ sinv,
                                                                 int rot_half, bf16* __restrict__ k_pages, bf16* __restrict__ v_pages,
-                                                                const int* __restrict__ slots, int page_size) {
+                                                                const int* __restrict__ slots, int page_size, const float* __restrict__ bias,
+                                                                QueryTemperature temperature, ValuePath<bf16> path) {
   __shared__ float scratch[16];
   const int token = blockIdx.x, tid = threadIdx.x;
   bf16* row = qkv + (int64_t)token * row_stride;
   const int qn = nq * d, kn = nkv * d, vn = nkv * dv;
   const int rot8 = rot_half / 8, items = (d - rot_half) / 8, total = (nq + nkv) * items;
   bf16x8 lo[PREP_ITEMS], hi[PREP_ITEMS];
+  // eight values of a run with their biases added (asked for twice, for the sum of squares and for the write: the same bits)
+  auto biased = [&](const bf16x8& x, const float* b, float (&out)[8]) {
+    floatx4 b0 = {0.f, 0.f, 0.f, 0.f}, b1 = b0;
+    if (b) b0 = *(const floatx4*)b, b1 = *(const floatx4*)(b + 4);
+#pragma unroll
+    for (int i = 0; i < 8; ++i) out[i] = (float)x[i] + (i < 4 ? b0[i] : b1[i - 4]);
+  };
   float ssq = 0.f, ssk = 0.f;
 #pragma unroll
   for (int n = 0; n < PREP_ITEMS; ++n) {
@@ -99,15 +121,19 @@ __global__ __launch_bounds__(256) void qkv_norm_prep_vec_kernel(bf16* __restrict
     if (w < total) {
       const int head = w / items, j = w % items;
       const bf16* src = row + (int64_t)head * d;
+      const float* hb = bias ? bias + (int64_t)head * d : nullptr;
       const bool paired = j < rot8;
-      lo[n] = *(const bf16x8*)(src + (paired ? j * 8 : j * 8 + rot_half));
-      float ss = 0.f;
+      const int at = paired ? j * 8 : j * 8 + rot_half;
+      lo[n] = *(const bf16x8*)(src + at);
+      float ss = 0.f, x[8];
+      biased(lo[n], hb ? hb + at : nullptr, x);
 #pragma unroll
-      for (int i = 0; i < 8; ++i) ss = fmaf((float)lo[n][i], (float)lo[n][i], ss);
+      for (int i = 0; i < 8; ++i) ss = fmaf(x[i], x[i], ss);
       if (paired) {
         hi[n] = *(const bf16x8*)(src + j * 8 + rot_half);
+        biased(hi[n], hb ? hb + j * 8 + rot_half : nullptr, x);
 #pragma unroll
-        for (int i = 0; i < 8; ++i) ss = fmaf((float)hi[n][i], (float)hi[n][i], ss);
+        for (int i = 0; i < 8; ++i) ss = fmaf(x[i], x[i], ss);
       }
       if (head < nq) ssq += ss;
       else ssk += ss;
@@ -115,7 +141,7 @@ __global__ __launch_bounds__(256) void qkv_norm_prep_vec_kernel(bf16* __restrict
   }
   ssq = block_sum(ssq, scratch);
   ssk = block_sum(ssk, scratch);
-  const float inv_q = q_weight ? 1.0f / sqrtf(ssq / (float)qn + eps) : 1.f;
+  const float inv_q = (q_weight ? 1.0f / sqrtf(ssq / (float)qn + eps) : 1.f) * temperature_of(temperature, token);
   const float inv_k = k_weight ? 1.0f / sqrtf(ssk / (float)kn + eps) : 1.f;
   const int slot = slots ? slots[token] : -1;
   const int64_t page = slot >= 0 ? slot / page_size : 0, off = slot >= 0 ? slot % page_size : 0;
@@ -133,7 +159,11 @@ __global__ __launch_bounds__(256) void qkv_norm_prep_vec_kernel(bf16* __restrict
     const float inv = is_q ? inv_q : inv_k;
     bf16* dst = is_q ? row + (int64_t)head * d : k_pages + ((page * nkv + (head - nq)) * page_size + off) * d;
     const floatx4 one4 = {1.f, 1.f, 1.f, 1.f};
+    const float* hb = bias ? bias + (int64_t)head * d : nullptr;
+    float xl[8], xh[8];
+    biased(lo[n], hb ? hb + (j < rot8 ? j * 8 : j * 8 + rot_half) : nullptr, xl);
     if (j < rot8) {
+      biased(hi[n], hb ? hb + j * 8 + rot_half : nullptr, xh);
       // weights and angles of the eight pairs, 16 bytes a load, all asked for before any is used
       floatx4 wa[2], wb[2], c4[2], s4[2];
 #pragma unroll
@@ -146,7 +176,7 @@ __global__ __launch_bounds__(256) void qkv_norm_prep_vec_kernel(bf16* __restrict
       bf16x8 first, second;
 #pragma unroll
       for (int i = 0; i < 8; ++i) {
-        const float a = (float)lo[n][i] * inv * wa[i / 4][i % 4], b = (float)hi[n][i] * inv * wb[i / 4][i % 4];
+        const float a = xl[i] * inv * wa[i / 4][i % 4], b = xh[i] * inv * wb[i / 4][i % 4];
         const float c = c4[i / 4][i % 4], sn = s4[i / 4][i % 4];
         first[i] = (bf16)(a * c - b * sn);
         second[i] = (bf16)(b * c + a * sn);
@@ -160,14 +190,14 @@ __global__ __launch_bounds__(256) void qkv_norm_prep_vec_kernel(bf16* __restrict
       for (int half = 0; half < 2; ++half) wa[half] = weight ? *(const floatx4*)(weight + wbase + at + half * 4) : one4;
       bf16x8 only;
 #pragma unroll
-      for (int i = 0; i < 8; ++i) only[i] = (bf16)((float)lo[n][i] * inv * wa[i / 4][i % 4]);
+      for (int i = 0; i < 8; ++i) only[i] = (bf16)(xl[i] * inv * wa[i / 4][i % 4]);
       *(bf16x8*)(dst + at) = only;
     }
   }
-  if (slot >= 0) {
+  if (slot >= 0 && v_pages) {           // (null: values_in_runs_kernel stores them)
     for (int e = tid; e < vn; e += 256) {
       const int kvh = e / dv, i = e % dv;
-      v_pages[((page * nkv + kvh) * dv + i) * page_size + off] = row[qn + kn + e];
+      v_pages[((page * nkv + kvh) * dv + i) * page_size + off] = value_on_its_way(path, row[qn + kn + e], qn + kn + e, token, vn, e);
     }
   }
 }
@@ -276,10 +306,14 @@ __global__ void activation_kernel(T* __restrict__ out, const T* __restrict__ x, 
 
 // qkv [tokens, row_stride] in dtype: q (nq*d) | k (nkv*d) | v (nkv*dv) | anything else.  q_weight [nq*d], k_weight [nkv*d]
 // float32 (both null: no norm).  cos, sin [tokens, rot_half] float32.  slots[t] = page * page_size + offset (negative: the
-// token's key and value are not stored).
+// token's key and value are not stored).  bias (float32 [nq*d + nkv*d + nkv*dv], or null) is added to q, k and v as they are read.
+// every > 0: queries are multiplied by 1 + coef * ln(floor((positions[t] + 1) / every) + 1).  first_values [tokens, nkv*dv] in
+// dtype, or null: value_mix null leaves the step's values there, value_mix given (one float32 on the device) mixes
+// v <- (1 - value_mix) v + value_mix first_values.
 LRS_API int lrs_qkv_norm_prep(void* qkv, int dtype, int tokens, int row_stride, int nq, int nkv, int d, int dv, const float* q_weight,
                               const float* k_weight, float eps, const float* cosv, const float* sinv, int rot_half, void* k_pages,
-                              void* v_pages, const int* slots, int page_size, void* stream) {
+                              void* v_pages, const int* slots, int page_size, const float* bias, const int* positions, float coef, int every,
+                              void* first_values, const float* value_mix, void* stream) {
   LRS_REQUIRE(tokens > 0 && nq > 0 && nkv > 0 && d > 0 && dv > 0, "qkv_norm_prep: bad sizes tokens=%d nq=%d nkv=%d d=%d dv=%d", tokens, nq, nkv, d, dv);
   LRS_REQUIRE(row_stride >= nq * d + nkv * d + nkv * dv, "qkv_norm_prep: rows of %d hold fewer than q, k and v", row_stride);
   LRS_REQUIRE(rot_half >= 0 && 2 * rot_half <= d, "qkv_norm_prep: rotary width %d exceeds head_dim %d", 2 * rot_half, d);
@@ -287,18 +321,38 @@ LRS_API int lrs_qkv_norm_prep(void* qkv, int dtype, int tokens, int row_stride, 
   LRS_REQUIRE((q_weight == nullptr) == (k_weight == nullptr), "qkv_norm_prep: q and k norm weights must come together");
   LRS_REQUIRE(!q_weight || eps > 0.f, "qkv_norm_prep: eps must be positive");
   LRS_REQUIRE(k_pages && v_pages && slots && page_size > 0, "qkv_norm_prep: cache write needs pages, slots and a page size");
+  LRS_REQUIRE(every >= 0 && (every == 0 || positions), "qkv_norm_prep: a temperature needs a positive step and the positions");
+  LRS_REQUIRE(!value_mix || first_values, "qkv_norm_prep: nothing to mix the values with");
   hipStream_t s = (hipStream_t)stream;
+  const QueryTemperature temperature{positions, coef, every};
+  // steps of many tokens: the values as runs of slots, 16 bytes a store, by workgroups of their own (token by token they are
+  // 2-byte writes a page row apart)
+  if (tokens >= 64 && page_size % (dtype == LRS_F32 ? 4 : 8) == 0 && (uintptr_t)v_pages % 16 == 0) {
+    const dim3 vgrid((tokens + 15) / 16, nkv);
+    if (dtype == LRS_F32)
+      values_in_runs_kernel<float><<<vgrid, 256, 0, s>>>((const float*)qkv, row_stride, (nq + nkv) * d, tokens, nkv, dv, (float*)v_pages, slots, page_size,
+                                                         ValuePath<float>{bias, (float*)first_values, value_mix});
+    else if (dtype == LRS_BF16)
+      values_in_runs_kernel<bf16><<<vgrid, 256, 0, s>>>((const bf16*)qkv, row_stride, (nq + nkv) * d, tokens, nkv, dv, (bf16*)v_pages, slots, page_size,
+                                                        ValuePath<bf16>{bias, (bf16*)first_values, value_mix});
+    else return lrs_fail("qkv_norm_prep: unknown dtype %d", dtype);
+    if (lrs_check_launch("values_in_runs")) return 1;
+    v_pages = nullptr;
+  }
   if (dtype == LRS_F32)
     qkv_norm_prep_kernel<float><<<tokens, 256, 0, s>>>((float*)qkv, row_stride, nq, nkv, d, dv, q_weight, k_weight, eps, cosv, sinv, rot_half,
-                                                       (float*)k_pages, (float*)v_pages, slots, page_size);
+                                                       (float*)k_pages, (float*)v_pages, slots, page_size, bias, temperature,
+                                                       ValuePath<float>{bias, (float*)first_values, value_mix});
   else if (dtype == LRS_BF16 && d % 8 == 0 && rot_half % 8 == 0 && row_stride % 8 == 0 &&
-           ((uintptr_t)qkv | (uintptr_t)q_weight | (uintptr_t)k_weight | (uintptr_t)cosv | (uintptr_t)sinv) % 16 == 0 &&
+           ((uintptr_t)qkv | (uintptr_t)q_weight | (uintptr_t)k_weight | (uintptr_t)cosv | (uintptr_t)sinv | (uintptr_t)bias | (uintptr_t)k_pages) % 16 == 0 &&
            (nq + nkv) * (d - rot_half) / 8 <= 256 * PREP_ITEMS)
     qkv_norm_prep_vec_kernel<<<tokens, 256, 0, s>>>((bf16*)qkv, row_stride, nq, nkv, d, dv, q_weight, k_weight, eps, cosv, sinv, rot_half,
-                                                    (bf16*)k_pages, (bf16*)v_pages, slots, page_size);
+                                                    (bf16*)k_pages, (bf16*)v_pages, slots, page_size, bias, temperature,
+                                                    ValuePath<bf16>{bias, (bf16*)first_values, value_mix});
   else if (dtype == LRS_BF16)
     qkv_norm_prep_kernel<bf16><<<tokens, 256, 0, s>>>((bf16*)qkv, row_stride, nq, nkv, d, dv, q_weight, k_weight, eps, cosv, sinv, rot_half,
-                                                      (bf16*)k_pages, (bf16*)v_pages, slots, page_size);
+                                                      (bf16*)k_pages, (bf16*)v_pages, slots, page_size, bias, temperature,
+                                                      ValuePath<bf16>{bias, (bf16*)first_values, value_mix});
   else return lrs_fail("qkv_norm_prep: unknown dtype %d", dtype);
   return lrs_check_launch("qkv_norm_prep");
 }

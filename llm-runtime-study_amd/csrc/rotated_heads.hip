@@ -10,7 +10,7 @@
 //                      for rows [gate: inter | up: inter];
 //   add_gathered       out[t, :] += table[ids[t], :] over float32 rows (a learned position vector added to the stream);
 //   scale_values       x *= factor over float32 values (logits times a constant).
-#include "common.h"
+#include "value_pages.h"
 
 namespace {
 
@@ -207,47 +207,6 @@ __global__ __launch_bounds__(256) void rotate_unit_prep_vec_kernel(bf16* __restr
   }
 }
 
-// The values of 16 consecutive tokens of the step and one kv head into the value pages [page, kv_head, dv, slot], for steps of
-// many tokens: tokens that follow each other inside a page lie side by side there, so a thread gathers one dim of 16 / sizeof(T)
-// such tokens (neighbouring lanes read neighbouring dims of one token), adds the dim's bias and writes one 16-byte store; where
-// a run is broken (a page's edge, another request, a slot that is not stored) it stores one by one.
-template <typename T>
-__global__ __launch_bounds__(256) void values_in_runs_kernel(const T* __restrict__ qkv, int row_stride, int v_offset, int tokens, int nkv, int dv,
-                                                             T* __restrict__ v_pages, const int* __restrict__ slots, int page_size,
-                                                             const float* __restrict__ bias) {
-  constexpr int RUN = 16 / sizeof(T);
-  typedef T vec __attribute__((ext_vector_type(RUN)));
-  __shared__ int slot_of[16];
-  const int tid = threadIdx.x, token0 = blockIdx.x * 16, kvh = blockIdx.y;
-  if (tid < 16) slot_of[tid] = token0 + tid < tokens ? slots[token0 + tid] : -1;
-  __syncthreads();
-  for (int e = tid; e < dv * (16 / RUN); e += 256) {
-    const int dim = e % dv, first = (e / dv) * RUN;
-    const int slot0 = slot_of[first];
-    bool run = slot0 >= 0 && slot0 % RUN == 0 && slot0 % page_size + RUN <= page_size;
-#pragma unroll
-    for (int i = 1; i < RUN; ++i) run = run && slot_of[first + i] == slot0 + i;
-    const int column = v_offset + kvh * dv + dim;
-    const float b = bias ? bias[column] : 0.f;
-    const T* src = qkv + (int64_t)(token0 + first) * row_stride + column;
-    if (run) {
-      vec v;
-#pragma unroll
-      for (int i = 0; i < RUN; ++i) v[i] = from_float<T>(to_float(src[(int64_t)i * row_stride]) + b);
-      const int64_t page = slot0 / page_size, off = slot0 % page_size;
-      *(vec*)(v_pages + ((page * nkv + kvh) * dv + dim) * page_size + off) = v;
-    } else {
-#pragma unroll
-      for (int i = 0; i < RUN; ++i) {
-        const int slot = slot_of[first + i];
-        if (slot < 0) continue;
-        const int64_t page = slot / page_size, off = slot % page_size;
-        v_pages[((page * nkv + kvh) * dv + dim) * page_size + off] = from_float<T>(to_float(src[(int64_t)i * row_stride]) + b);
-      }
-    }
-  }
-}
-
 template <typename T>
 __global__ void gated_clamped_kernel(T* __restrict__ out, const T* __restrict__ gu, int64_t count, int inter, float alpha, float limit) {
   const int64_t e = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
@@ -293,9 +252,9 @@ LRS_API int lrs_rotate_unit_prep(void* qkv, int dtype, int tokens, int row_strid
   if (tokens >= 64 && page_size % (dtype == LRS_F32 ? 4 : 8) == 0 && (uintptr_t)v_pages % 16 == 0) {
     const dim3 vgrid((tokens + 15) / 16, nkv);
     if (dtype == LRS_F32)
-      values_in_runs_kernel<float><<<vgrid, 256, 0, s>>>((const float*)qkv, row_stride, (nq + nkv) * d, tokens, nkv, dv, (float*)v_pages, slots, page_size, bias);
+      values_in_runs_kernel<float><<<vgrid, 256, 0, s>>>((const float*)qkv, row_stride, (nq + nkv) * d, tokens, nkv, dv, (float*)v_pages, slots, page_size, ValuePath<float>{bias, nullptr, nullptr});
     else if (dtype == LRS_BF16)
-      values_in_runs_kernel<bf16><<<vgrid, 256, 0, s>>>((const bf16*)qkv, row_stride, (nq + nkv) * d, tokens, nkv, dv, (bf16*)v_pages, slots, page_size, bias);
+      values_in_runs_kernel<bf16><<<vgrid, 256, 0, s>>>((const bf16*)qkv, row_stride, (nq + nkv) * d, tokens, nkv, dv, (bf16*)v_pages, slots, page_size, ValuePath<bf16>{bias, nullptr, nullptr});
     else return lrs_fail("rotate_unit_prep: unknown dtype %d", dtype);
     if (lrs_check_launch("values_in_runs")) return 1;
     v_pages = nullptr;

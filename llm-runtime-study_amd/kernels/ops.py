@@ -124,9 +124,14 @@ _SIGNATURES = {
                                             c_void_p, c_int64, c_void_p]),
     "lrs_norm_begin_parts": (c_int, [c_int]),
     "lrs_attention": (c_int, [c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p,
-                              c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_int, c_void_p, c_float, c_void_p, c_int, c_void_p]),
+                              c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_int, c_void_p, c_float, c_void_p, c_int, c_void_p, c_void_p]),
     "lrs_qkv_norm_prep": (c_int, [c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_float, c_void_p, c_void_p,
-                                  c_int, c_void_p, c_void_p, c_void_p, c_int, c_void_p]),
+                                  c_int, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_float, c_int, c_void_p, c_void_p, c_void_p]),
+    "lrs_gated_norm_add": (c_int, [c_void_p, c_void_p, c_void_p, c_int, c_int, c_void_p, c_void_p, c_float, c_int, c_int, c_void_p, c_float,
+                                   c_void_p, c_int, c_void_p]),
+    "lrs_xielu": (c_int, [c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_int, c_void_p, c_void_p]),
+    "lrs_mlstm": (c_int, [c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p, c_int64, c_int, c_int, c_int,
+                          c_void_p, c_void_p, c_float, c_void_p, c_float, c_void_p, c_void_p, c_void_p, c_void_p]),
     "lrs_sigmoid_gate": (c_int, [c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p]),
     "lrs_rotate_unit_prep": (c_int, [c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_void_p, c_void_p, c_int, c_int,
                                      c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p]),
@@ -143,10 +148,10 @@ _SIGNATURES = {
                         c_void_p, c_void_p, c_void_p, c_void_p, c_void_p]),
     "lrs_attention_decode": (c_int, [c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_void_p,
                                      c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_int, c_int, c_int, c_int,
-                                     c_void_p, c_void_p, c_int, c_float, c_void_p, c_void_p, c_int, c_void_p, c_float, c_void_p, c_int, c_void_p]),
+                                     c_void_p, c_void_p, c_int, c_float, c_void_p, c_void_p, c_int, c_void_p, c_float, c_void_p, c_int, c_int, c_void_p, c_void_p]),
     "lrs_attention_prefill": (c_int, [c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p,
                                       c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_int,
-                                      c_int, c_int, c_void_p, c_void_p, c_int, c_void_p, c_int, c_float, c_void_p, c_void_p, c_void_p, c_float, c_void_p, c_int, c_void_p]),
+                                      c_int, c_int, c_void_p, c_void_p, c_int, c_void_p, c_int, c_float, c_void_p, c_void_p, c_void_p, c_float, c_void_p, c_int, c_int, c_void_p, c_void_p]),
     "lrs_attention_prefill_prepares": (c_int, [c_int]),
     "lrs_compute_units": (c_int, []),
     "lrs_gemm_lines_width": (c_int, [c_int, c_int, c_int]),
@@ -223,9 +228,9 @@ def library():
 # and _SIGNATURES by kernels/plan_codegen.py, is the other side (a test keeps the two in step).
 PLAN_OPS = ("lrs_activation", "lrs_add_gathered", "lrs_add_into", "lrs_add_rmsnorm", "lrs_advance_decode", "lrs_advance_slots", "lrs_attention", "lrs_attention_decode",
             "lrs_attention_prefill", "lrs_axpby", "lrs_choose_tokens", "lrs_choose_tokens_split", "lrs_copy_to_pinned", "lrs_delta_rule", "lrs_delta_rule_channels", "lrs_embed", "lrs_fill_i32",
-            "lrs_filter_logits", "lrs_gated_clamped", "lrs_gather_rows", "lrs_gemm", "lrs_gemm_lines_add_rmsnorm", "lrs_gemm_mid_add_norm_begin", "lrs_gemm_mid_qk_prep", "lrs_gemm_mid_scaled",
-            "lrs_gemm_norm_chain", "lrs_head_gemm", "lrs_latent_attention", "lrs_latent_attention_groups", "lrs_latent_prep", "lrs_layernorm", "lrs_library_gemm", "lrs_moe_align", "lrs_moe_combine", "lrs_moe_experts", "lrs_moe_route", "lrs_moe_route_align", "lrs_norm_add",
-            "lrs_qk_prep", "lrs_qkv_norm_prep", "lrs_rmsnorm", "lrs_rope_table", "lrs_rotate_unit_prep", "lrs_round_rows", "lrs_scale_add_layernorm", "lrs_scale_rows", "lrs_scale_values", "lrs_sigmoid_gate", "lrs_silu_mul", "lrs_soft_cap", "lrs_ssm")
+            "lrs_filter_logits", "lrs_gated_clamped", "lrs_gated_norm_add", "lrs_gather_rows", "lrs_gemm", "lrs_gemm_lines_add_rmsnorm", "lrs_gemm_mid_add_norm_begin", "lrs_gemm_mid_qk_prep", "lrs_gemm_mid_scaled",
+            "lrs_gemm_norm_chain", "lrs_head_gemm", "lrs_latent_attention", "lrs_latent_attention_groups", "lrs_latent_prep", "lrs_layernorm", "lrs_library_gemm", "lrs_mlstm", "lrs_moe_align", "lrs_moe_combine", "lrs_moe_experts", "lrs_moe_route", "lrs_moe_route_align", "lrs_norm_add",
+            "lrs_qk_prep", "lrs_qkv_norm_prep", "lrs_rmsnorm", "lrs_rope_table", "lrs_rotate_unit_prep", "lrs_round_rows", "lrs_scale_add_layernorm", "lrs_scale_rows", "lrs_scale_values", "lrs_sigmoid_gate", "lrs_silu_mul", "lrs_soft_cap", "lrs_ssm", "lrs_xielu")
 _PLAN_INDEX = {name: index for index, name in enumerate(PLAN_OPS)}
 
 
@@ -980,14 +985,25 @@ def _sinks(sinks: torch.Tensor | None, nq: int, who: str):
     return _dev(sinks, "sinks")
 
 
+def _distance(distance: torch.Tensor | None, nq: int, who: str):
+    """Address of a bias by distance, float32 [2, nq]: the heads' rates, then their reaches (a score at distance x loses
+    rate * ln(1 + reach * x)); None: no bias."""
+    if distance is None:
+        return None
+    _need(distance.dtype == torch.float32 and distance.shape == (2, nq) and distance.is_contiguous(), f"{who}: distance must be float32 [2, {nq}]")
+    return _dev(distance, "distance")
+
+
 def attention(out: torch.Tensor, q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor, block_table: torch.Tensor,
               token_request: torch.Tensor, positions: torch.Tensor, nq: int, scale: float, window: int = 0, keep_first: int = 0,
-              sinks: torch.Tensor | None = None, softcap: float = 0.0, gates: torch.Tensor | None = None) -> None:
+              sinks: torch.Tensor | None = None, softcap: float = 0.0, gates: torch.Tensor | None = None,
+              distance: torch.Tensor | None = None) -> None:
     """out [T, nq*dv]; q [T, >= nq*d] (leading nq*d columns of each row); key pages [P, nkv, page, d],
     value pages [P, nkv, dv, page].  window: a token at p sees keys above p - window; keep_first: and those below keep_first.
     sinks (float32 [nq]): the softmax's denominator of head h has one more term exp(sinks[h]), without key or value.
     softcap > 0: the scaled scores pass softcap * tanh(score / softcap) before the softmax.
-    gates ([T, nq], rows of any stride): head h's output is multiplied by sigmoid(gates[t, h])."""
+    gates ([T, nq], rows of any stride): head h's output is multiplied by sigmoid(gates[t, h]).
+    distance (float32 [2, nq]): head h's score of a key x positions back loses distance[0, h] * ln(1 + distance[1, h] * x)."""
     tokens = out.shape[0]
     _need(k_pages.dim() == 4 and v_pages.dim() == 4 and k_pages.is_contiguous() and v_pages.is_contiguous(), "attention: pages must be contiguous")
     _, nkv, page_size, d = k_pages.shape
@@ -1002,14 +1018,19 @@ def attention(out: torch.Tensor, q: torch.Tensor, k_pages: torch.Tensor, v_pages
         _dev(out, "out"), _rows(out, "out"), _dev(q, "q"), _rows(q, "q"), _dev(k_pages, "k_pages"), _dev(v_pages, "v_pages"),
         _dev(block_table, "block_table"), block_table.stride(0), _dev(token_request, "token_request"), _dev(positions, "positions"),
         dtype_code(q.dtype), tokens, nq, nkv, d, dv, page_size, scale, window, keep_first, _sinks(sinks, nq, "attention"), float(softcap),
-        *_gates(gates, tokens, nq, q.dtype, "attention"), _stream())
+        *_gates(gates, tokens, nq, q.dtype, "attention"), _distance(distance, nq, "attention"), _stream())
 
 
 def qkv_norm_prep(qkv: torch.Tensor, nq: int, nkv: int, d: int, dv: int, q_weight, k_weight, eps: float, cos, sin,
-                  k_pages: torch.Tensor, v_pages: torch.Tensor, slots: torch.Tensor, page_size: int) -> None:
+                  k_pages: torch.Tensor, v_pages: torch.Tensor, slots: torch.Tensor, page_size: int, bias: torch.Tensor | None = None,
+                  temperature: tuple | None = None, positions: torch.Tensor | None = None, first_values: torch.Tensor | None = None,
+                  value_mix: torch.Tensor | None = None) -> None:
     """The rows of `qkv` [T, >= nq*d + nkv*d + nkv*dv] (q | k | v | whatever follows): q and k each divided by the root mean
     square of the whole part (all heads at once) and multiplied by a weight per column (float32 [nq*d], [nkv*d]; None: no
-    norm), the first 2 * cos.shape[1] dims of every head rotated; q in place, k and v into the pages."""
+    norm), the first 2 * cos.shape[1] dims of every head rotated; q in place, k and v into the pages.  On the way: `bias` (float32,
+    a value per column of q, k and v) is added first; `temperature` (coef, every) multiplies the queries of a token at position p
+    by 1 + coef * ln(floor((p + 1) / every) + 1); `first_values` [T, nkv*dv] receives the step's values, or, with `value_mix`
+    (float32 [1] on the device), is what they are mixed with: v <- (1 - value_mix) v + value_mix first_values."""
     tokens = qkv.shape[0]
     stride = _rows(qkv, "qkv")
     _need(qkv.shape[1] >= (nq + nkv) * d + nkv * dv, "qkv_norm_prep: the rows hold fewer than q, k and v")
@@ -1026,10 +1047,52 @@ def qkv_norm_prep(qkv: torch.Tensor, nq: int, nkv: int, d: int, dv: int, q_weigh
     _need(k_pages.is_contiguous() and v_pages.is_contiguous() and k_pages.dtype == qkv.dtype and v_pages.dtype == qkv.dtype,
           "qkv_norm_prep: pages must be contiguous and of the activation dtype")
     _need(slots.dtype == torch.int32 and slots.numel() >= tokens and slots.is_contiguous(), "qkv_norm_prep: slots must be int32 [T]")
+    if bias is not None:
+        _need(bias.dtype == torch.float32 and bias.is_contiguous() and bias.numel() >= (nq + nkv) * d + nkv * dv, "qkv_norm_prep: bias must hold a float32 value per column")
+    coef, every = temperature if temperature is not None else (0.0, 0)
+    if every:
+        _need(every > 0 and positions is not None and positions.dtype == torch.int32 and positions.numel() >= tokens and positions.is_contiguous(),
+              "qkv_norm_prep: a temperature needs a positive step and int32 positions [T]")
+    if first_values is not None:
+        _need(first_values.shape == (tokens, nkv * dv) and first_values.dtype == qkv.dtype and first_values.is_contiguous(),
+              f"qkv_norm_prep: first_values must be contiguous [{tokens}, {nkv * dv}] of the activation dtype")
+    if value_mix is not None:
+        _need(first_values is not None and value_mix.dtype == torch.float32 and value_mix.numel() == 1, "qkv_norm_prep: value_mix is one float32 and needs first_values")
     _launch("lrs_qkv_norm_prep", _dev(qkv, "qkv"), dtype_code(qkv.dtype), tokens, stride, nq, nkv, d, dv,
             None if q_weight is None else _dev(q_weight, "q_weight"), None if k_weight is None else _dev(k_weight, "k_weight"), eps,
             None if cos is None else cos.data_ptr(), None if sin is None else sin.data_ptr(), rot_half, _dev(k_pages, "k_pages"),
-            _dev(v_pages, "v_pages"), _dev(slots, "slots"), page_size, _stream())
+            _dev(v_pages, "v_pages"), _dev(slots, "slots"), page_size, None if bias is None else _dev(bias, "bias"),
+            _dev(positions, "positions") if every else None, float(coef), every, None if first_values is None else _dev(first_values, "first_values"),
+            None if value_mix is None else _dev(value_mix, "value_mix"), _stream())
+
+
+def gated_norm_add(stream: torch.Tensor, y: torch.Tensor, gate: torch.Tensor | None, gate_bias: torch.Tensor | None, weight: torch.Tensor, eps: float,
+                   next_weight: torch.Tensor | None = None, next_eps: float = 0.0, normed: torch.Tensor | None = None) -> None:
+    """stream += weight * g / sqrt(mean(g^2) + eps) per row, g = y * sigmoid(gate + gate_bias); stream and y contiguous float32
+    [T, C], gate [T, C] of either dtype with rows of any stride (None: g = y), gate_bias, weight float32 [C].  normed [T, C]:
+    receives the RMS norm of the new rows times next_weight (float32 [C])."""
+    rows, cols = stream.shape
+    for name, t in (("stream", stream), ("y", y)):
+        _need(t.dtype == torch.float32 and t.is_contiguous() and t.shape == (rows, cols), f"gated_norm_add: {name} must be contiguous float32 [T, C]")
+    for name, t in (("gate_bias", gate_bias), ("weight", weight), ("next_weight", next_weight)):
+        _need(t is None or (t.dtype == torch.float32 and t.numel() == cols and t.is_contiguous()), f"gated_norm_add: {name} must be float32 [{cols}]")
+    _need(gate is None or (gate.shape == (rows, cols) and gate.stride(1) == 1), "gated_norm_add: gate must be [T, C]")
+    _need(normed is None or (next_weight is not None and normed.shape == stream.shape and normed.is_contiguous()),
+          "gated_norm_add: the normalised rows need a contiguous [T, C] buffer and the norm's weight")
+    _launch("lrs_gated_norm_add", _dev(stream, "stream"), _dev(y, "y"), None if gate is None else _dev(gate, "gate"),
+            0 if gate is None else dtype_code(gate.dtype), 0 if gate is None else _rows(gate, "gate"),
+            None if gate is None or gate_bias is None else _dev(gate_bias, "gate_bias"), _dev(weight, "weight"), eps, rows, cols,
+            None if normed is None else _dev(next_weight, "next_weight"), next_eps, None if normed is None else _dev(normed, "normed"),
+            0 if normed is None else dtype_code(normed.dtype), _stream())
+
+
+def xielu(out: torch.Tensor, x: torch.Tensor, numbers: torch.Tensor) -> None:
+    """out = a x^2 + x / 2 where x > 0, b (exp(x) - 1 - x) + x / 2 elsewhere; numbers: float32 [2] on the device, a and b.  out and
+    x [T, C], rows of any stride (out may be x)."""
+    _need(out.dim() == 2 and out.shape == x.shape and out.dtype == x.dtype and x.numel() > 0, "xielu: out and x must be [T, C] of one dtype")
+    _need(numbers.dtype == torch.float32 and numbers.numel() == 2 and numbers.is_contiguous(), "xielu: numbers must be float32 [2]")
+    _launch("lrs_xielu", _dev(out, "out"), _rows(out, "out"), _dev(x, "x"), _rows(x, "x"), dtype_code(x.dtype), x.shape[0], x.shape[1],
+            _dev(numbers, "numbers"), _stream())
 
 
 def sigmoid_gate(out: torch.Tensor, gate: torch.Tensor) -> None:
@@ -1120,9 +1183,10 @@ def activation(out: torch.Tensor, x: torch.Tensor, kind: str) -> None:
 DECODE_HEAD_DIMS = (32, 64, 96, 128, 192)
 
 
-def attention_decode_supported(dtype: torch.dtype, nq: int, nkv: int, d: int, page_size: int) -> bool:
-    """Whether the matrix-core decode kernel takes this shape (else use attention())."""
-    return dtype == torch.bfloat16 and d in DECODE_HEAD_DIMS and page_size % 16 == 0 and nq // nkv <= 16
+def attention_decode_supported(dtype: torch.dtype, nq: int, nkv: int, d: int, page_size: int, dv: int | None = None) -> bool:
+    """Whether the matrix-core kernels take this shape (else use attention()); dv: the values' size, if it is not d."""
+    narrower = dv is None or dv == d or (0 < dv < d and dv % 16 == 0)
+    return dtype == torch.bfloat16 and d in DECODE_HEAD_DIMS and page_size % 16 == 0 and nq // nkv <= 16 and narrower
 
 
 @dataclass
@@ -1149,7 +1213,7 @@ def attention_decode(out: torch.Tensor, q: torch.Tensor, k_pages: torch.Tensor, 
                      token_request: torch.Tensor, positions: torch.Tensor, nq: int, scale: float, window: int = 0, splits: int = 1,
                      part_o: torch.Tensor | None = None, part_ml: torch.Tensor | None = None, max_context: int | None = None,
                      prepare: "DecodePrepare | None" = None, form: int = 0, keep_first: int = 0, sinks: torch.Tensor | None = None,
-                     softcap: float = 0.0, gates: torch.Tensor | None = None) -> None:
+                     softcap: float = 0.0, gates: torch.Tensor | None = None, distance: torch.Tensor | None = None) -> None:
     """attention() for a step with one query token per request, bfloat16 only; the keys of a token
     are divided between `splits` workgroups whose partial results meet in part_o / part_ml.
     keep_first (with a window and prepared heads): the first positions of a sequence stay visible behind the window; their
@@ -1160,9 +1224,10 @@ def attention_decode(out: torch.Tensor, q: torch.Tensor, k_pages: torch.Tensor, 
     tokens = out.shape[0]
     _need(k_pages.dim() == 4 and k_pages.is_contiguous() and v_pages.is_contiguous(), "attention_decode: pages must be contiguous")
     _, nkv, page_size, d = k_pages.shape
-    _need(v_pages.shape == (k_pages.shape[0], nkv, d, page_size), "attention_decode: key pages must be [P, nkv, page, d] and value pages [P, nkv, d, page]")
-    _need(attention_decode_supported(q.dtype, nq, nkv, d, page_size), f"attention_decode: unsupported shape nq={nq} nkv={nkv} d={d} page={page_size} {q.dtype}")
-    _need(out.shape[1] == nq * d and q.shape[0] == tokens and q.shape[1] >= nq * d, "attention_decode: q/out widths do not match nq*d")
+    dv = v_pages.shape[2]                  # values may be narrower than keys
+    _need(v_pages.shape == (k_pages.shape[0], nkv, dv, page_size), "attention_decode: key pages must be [P, nkv, page, d] and value pages [P, nkv, dv, page]")
+    _need(attention_decode_supported(q.dtype, nq, nkv, d, page_size, dv), f"attention_decode: unsupported shape nq={nq} nkv={nkv} d={d} dv={dv} page={page_size} {q.dtype}")
+    _need(out.shape[1] == nq * dv and q.shape[0] == tokens and q.shape[1] >= nq * d, "attention_decode: q/out widths do not match nq*d and nq*dv")
     _need(q.dtype == k_pages.dtype == v_pages.dtype == out.dtype, "attention_decode: q, pages and out must share a dtype")
     _need(block_table.dim() == 2 and block_table.dtype == torch.int32 and block_table.stride(1) == 1, "attention_decode: block_table must be int32 [R, blocks]")
     for name, t in (("token_request", token_request), ("positions", positions)):
@@ -1170,10 +1235,11 @@ def attention_decode(out: torch.Tensor, q: torch.Tensor, k_pages: torch.Tensor, 
     _need(keep_first >= 0 and (keep_first == 0 or (window > 0 and prepare is None)), "attention_decode: kept first positions need a window and prepared heads")
     slots = splits + (1 if keep_first else 0)
     if slots > 1:
-        _need(part_o is not None and part_o.dtype == torch.float32 and part_o.is_contiguous() and part_o.numel() >= tokens * nq * slots * d, "attention_decode: part_o too small")
+        _need(part_o is not None and part_o.dtype == torch.float32 and part_o.is_contiguous() and part_o.numel() >= tokens * nq * slots * dv, "attention_decode: part_o too small")
         _need(part_ml is not None and part_ml.dtype == torch.float32 and part_ml.is_contiguous() and part_ml.numel() >= tokens * nq * slots * 2, "attention_decode: part_ml too small")
     fused = [0, None, None, 0, 0.0, None, None, 0]
     if prepare is not None:
+        _need(dv == d, "attention_decode: heads whose values are narrower than their keys must come prepared")
         _need(decode_prepare_supported(d, prepare.cos is not None), f"attention_decode: cannot rotate heads of {d} dims itself")
         _need((prepare.q_weight is None) == (prepare.k_weight is None), "attention_decode: q and k norm weights must come together")
         _need(prepare.kv_heads in (0, nkv) and q.shape[1] >= (nq + 2 * prepare.kv_heads) * d, "attention_decode: q rows must hold the q heads and kv_heads (0 or all) k and v heads")
@@ -1192,7 +1258,8 @@ def attention_decode(out: torch.Tensor, q: torch.Tensor, k_pages: torch.Tensor, 
         _dev(q, "q"), _rows(q, "q"), _dev(k_pages, "k_pages"), _dev(v_pages, "v_pages"), _dev(block_table, "block_table"), block_table.stride(0),
         _dev(token_request, "token_request"), _dev(positions, "positions"), tokens,
         block_table.shape[1] * page_size if max_context is None else max_context, nq, nkv, d, page_size, scale, window, keep_first, splits,
-        form, *fused, _sinks(sinks, nq, "attention_decode"), float(softcap), *_gates(gates, tokens, nq, q.dtype, "attention_decode"), _stream())
+        form, *fused, _sinks(sinks, nq, "attention_decode"), float(softcap), *_gates(gates, tokens, nq, q.dtype, "attention_decode"), dv,
+        _distance(distance, nq, "attention_decode"), _stream())
 
 
 def attention_prefill(out: torch.Tensor, q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor, block_table: torch.Tensor,
@@ -1200,7 +1267,7 @@ def attention_prefill(out: torch.Tensor, q: torch.Tensor, k_pages: torch.Tensor,
                       nq: int, scale: float, window: int = 0, max_count: int | None = None, max_context: int | None = None,
                       splits: int = 1, part_o: torch.Tensor | None = None, part_ml: torch.Tensor | None = None,
                       prepare: "DecodePrepare | None" = None, keep_first: int = 0, sinks: torch.Tensor | None = None,
-                      softcap: float = 0.0, gates: torch.Tensor | None = None) -> None:
+                      softcap: float = 0.0, gates: torch.Tensor | None = None, distance: torch.Tensor | None = None) -> None:
     """attention() on matrix cores for any bfloat16 step.  qblock_token0 / qblock_count list groups of at
     most attention_prefill_group() consecutive tokens of one request that together cover every token of
     the step once; `max_count` is the largest count among them (the group limit if not given) and
@@ -1215,9 +1282,10 @@ def attention_prefill(out: torch.Tensor, q: torch.Tensor, k_pages: torch.Tensor,
     tokens = out.shape[0]
     _need(k_pages.dim() == 4 and k_pages.is_contiguous() and v_pages.is_contiguous(), "attention_prefill: pages must be contiguous")
     _, nkv, page_size, d = k_pages.shape
-    _need(v_pages.shape == (k_pages.shape[0], nkv, d, page_size), "attention_prefill: key pages must be [P, nkv, page, d] and value pages [P, nkv, d, page]")
-    _need(attention_decode_supported(q.dtype, nq, nkv, d, page_size), f"attention_prefill: unsupported shape nq={nq} nkv={nkv} d={d} page={page_size} {q.dtype}")
-    _need(out.shape[1] == nq * d and q.shape[0] == tokens and q.shape[1] >= nq * d, "attention_prefill: q/out widths do not match nq*d")
+    dv = v_pages.shape[2]                  # values may be narrower than keys
+    _need(v_pages.shape == (k_pages.shape[0], nkv, dv, page_size), "attention_prefill: key pages must be [P, nkv, page, d] and value pages [P, nkv, dv, page]")
+    _need(attention_decode_supported(q.dtype, nq, nkv, d, page_size, dv), f"attention_prefill: unsupported shape nq={nq} nkv={nkv} d={d} dv={dv} page={page_size} {q.dtype}")
+    _need(out.shape[1] == nq * dv and q.shape[0] == tokens and q.shape[1] >= nq * d, "attention_prefill: q/out widths do not match nq*d and nq*dv")
     _need(q.dtype == k_pages.dtype == v_pages.dtype == out.dtype, "attention_prefill: q, pages and out must share a dtype")
     _need(block_table.dim() == 2 and block_table.dtype == torch.int32 and block_table.stride(1) == 1, "attention_prefill: block_table must be int32 [R, blocks]")
     for name, t in (("token_request", token_request), ("positions", positions)):
@@ -1229,7 +1297,7 @@ def attention_prefill(out: torch.Tensor, q: torch.Tensor, k_pages: torch.Tensor,
     _need(keep_first >= 0 and (keep_first == 0 or (window > 0 and prepare is None)), "attention_prefill: kept first positions need a window and prepared heads")
     slots = splits + (1 if keep_first else 0)
     if slots > 1:
-        _need(part_o is not None and part_o.dtype == torch.float32 and part_o.is_contiguous() and part_o.numel() >= tokens * nq * slots * d, "attention_prefill: part_o too small")
+        _need(part_o is not None and part_o.dtype == torch.float32 and part_o.is_contiguous() and part_o.numel() >= tokens * nq * slots * dv, "attention_prefill: part_o too small")
         _need(part_ml is not None and part_ml.dtype == torch.float32 and part_ml.is_contiguous() and part_ml.numel() >= tokens * nq * slots * 2, "attention_prefill: part_ml too small")
     fused = [0, None, 0, 0.0, None, None]
     if prepare is not None:
@@ -1250,7 +1318,8 @@ def attention_prefill(out: torch.Tensor, q: torch.Tensor, k_pages: torch.Tensor,
         attention_prefill_group() if max_count is None else max_count,
         block_table.shape[1] * page_size if max_context is None else max_context, nq, nkv, d, page_size, scale, window, keep_first,
         tokens, splits, None if slots == 1 else _dev(part_o, "part_o"), None if slots == 1 else _dev(part_ml, "part_ml"), *fused,
-        _sinks(sinks, nq, "attention_prefill"), float(softcap), *_gates(gates, tokens, nq, q.dtype, "attention_prefill"), _stream())
+        _sinks(sinks, nq, "attention_prefill"), float(softcap), *_gates(gates, tokens, nq, q.dtype, "attention_prefill"), dv,
+        _distance(distance, nq, "attention_prefill"), _stream())
 
 
 def attention_prefill_prepares(d: int) -> bool:
@@ -1454,6 +1523,35 @@ def state_space(out: torch.Tensor, proj: torch.Tensor, state: torch.Tensor, toke
             state.stride(0), _dev(conv_weight, "conv_weight"), None if conv_bias is None else _dev(conv_bias, "conv_bias"), taps, groups, heads,
             state_size, vdim, _dev(a_log, "a_log"), _dev(dt_bias, "dt_bias"), _dev(skip, "skip"), _dev(norm_weight, "norm_weight"), norm_parts,
             eps, _dev(qkv, "qkv"), _dev(gates, "gates"), _dev(raw, "raw"), _dev(skipped, "skipped"), _stream())
+
+
+def mlstm_state_floats(heads: int, dim: int, vdim: int) -> int:
+    """Floats of one request's state row of a matrix memory with exponential gates: the matrix of every head with the normaliser
+    as its last column (dim padded to 16 lanes of 4, 8 or 16 rows), then the running maximum of every head."""
+    return heads * library().lrs_delta_state_rows(dim) * 16 * (vdim + 1) + heads
+
+
+def mlstm(out: torch.Tensor, proj: torch.Tensor, state: torch.Tensor, cu_seqlens: torch.Tensor, slot_ids: torch.Tensor, requests: int, heads: int,
+          dim: int, vdim: int, i_bias: torch.Tensor, f_bias: torch.Tensor, cap: float, norm_weight: torch.Tensor, eps: float,
+          gates: torch.Tensor, floors: torch.Tensor, raw: torch.Tensor) -> None:
+    """One step of the matrix memory for a ragged batch.  proj float32 [T, >= C], columns q (heads*dim) | k (heads*dim) |
+    v (heads*vdim) | output gate (heads*vdim) | input gate (heads) | forget gate (heads); state [slots, floats] float32 is read and
+    written at the rows slot_ids names; i_bias, f_bias [heads], norm_weight [heads*vdim]; out [T, heads*vdim]."""
+    tokens = out.shape[0]
+    _need(out.is_contiguous() and out.shape[1] == heads * vdim, "mlstm: out must be contiguous [T, heads*vdim]")
+    _need(proj.dtype == torch.float32 and proj.shape[0] >= tokens and proj.shape[1] >= 2 * heads * (dim + vdim + 1), "mlstm: proj must be float32 and hold every column")
+    _need(state.dim() == 2 and state.dtype == torch.float32 and state.is_contiguous() and state.shape[1] >= mlstm_state_floats(heads, dim, vdim),
+          "mlstm: state rows are too short")
+    for name, t, count in (("i_bias", i_bias, heads), ("f_bias", f_bias, heads), ("norm_weight", norm_weight, heads * vdim)):
+        _need(t.dtype == torch.float32 and t.numel() == count and t.is_contiguous(), f"mlstm: {name} must hold {count} float32 values")
+    for name, t, count in (("cu_seqlens", cu_seqlens, requests + 1), ("slot_ids", slot_ids, requests)):
+        _need(t.dtype == torch.int32 and t.numel() >= count and t.is_contiguous(), f"mlstm: {name} must be int32 [{count}]")
+    for name, t, count in (("gates", gates, tokens * 2 * heads), ("floors", floors, tokens * heads), ("raw", raw, tokens * heads * (vdim + 1))):
+        _need(t.dtype == torch.float32 and t.is_contiguous() and t.numel() >= count, f"mlstm: {name} scratch too small")
+    _launch("lrs_mlstm", _dev(out, "out"), dtype_code(out.dtype), _dev(proj, "proj"), _rows(proj, "proj"), tokens, requests,
+            _dev(cu_seqlens, "cu_seqlens"), _dev(slot_ids, "slot_ids"), _dev(state, "state"), state.stride(0), heads, dim, vdim,
+            _dev(i_bias, "i_bias"), _dev(f_bias, "f_bias"), cap, _dev(norm_weight, "norm_weight"), eps, _dev(gates, "gates"),
+            _dev(floors, "floors"), _dev(raw, "raw"), _stream())
 
 
 # ------------------------------------------------------------------- routed experts

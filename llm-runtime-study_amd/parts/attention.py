@@ -31,6 +31,13 @@ softmax's denominator, which has no key and no value; `score_cap` passes the sca
 of its partial results, where `True` gates every value by a kernel of its own; `bias` with any of these
 adds the stacked biases to q, k and v: in the product's epilogue, or, where `rotate_unit_prep` prepares the heads, in that kernel
 as it reads the rows (in float32; the product then runs without a bias, through the vendor's library for many rows).
+
+And with the norm over the projection: `query_temperature` (coef, every) multiplies a query at position p by
+1 + coef * ln(floor((p + 1) / every) + 1); `value_mix` mixes a layer's values with those of an earlier layer of the same token,
+v <- (1 - lambda) v + lambda v_first with a learned lambda, before they are cached ("first": the layer whose values the others take,
+"later": a layer that takes them; they stay in a buffer of the step); `distance_bias` takes rate_h * ln(1 + reach_h * (i - j)) off
+head h's score of query i and key j; a number for `sink` is a sink of that score in every head instead of a learned one.  Values
+narrower than keys (a multiple of 16) run on the matrix cores too.
 """
 
 from __future__ import annotations
@@ -52,12 +59,17 @@ class GQAAttention(Part):
     wants_query_groups = True   # ragged steps go to a kernel that walks groups of a request's consecutive tokens
     can_overwrite = True        # forward(..., accumulate=False) stores its output
 
+    @property
+    def carries_rows(self) -> bool:
+        return self.whole_rows
+
     def __init__(self, hidden_size: int, num_heads: int, num_kv_heads: int, head_dim: int, *,
                  position: PartSpec = PartSpec("none"), qk_norm: bool = False, qk_norm_eps: float = 1e-6,
                  bias: bool = False, scale: float | None = None, window: int | None = None,
                  kv_shared: bool = False, values_from_keys: bool = False, norm_over: str = "head", value_dim: int | None = None,
-                 keep_first: int = 0, output_gate: bool | str = False, unit_norm_after_rotation: bool = False, sink: bool = False,
-                 score_cap: float | None = None):
+                 keep_first: int = 0, output_gate: bool | str = False, unit_norm_after_rotation: bool = False,
+                 sink: bool | float = False, score_cap: float | None = None, query_temperature: tuple | None = None,
+                 value_mix: str | None = None, distance_bias: bool = False):
         for name, value in (("hidden_size", hidden_size), ("num_heads", num_heads), ("num_kv_heads", num_kv_heads), ("head_dim", head_dim)):
             if value <= 0:
                 raise ValueError(f"{name} must be positive, got {value}")
@@ -91,11 +103,20 @@ class GQAAttention(Part):
         if unit_norm_after_rotation and qk_norm_eps <= 0:
             raise ValueError(f"qk_norm_eps must be positive, got {qk_norm_eps}")
         self.norm_over, self.value_dim, self.keep_first, self.output_gate = norm_over, value_dim or head_dim, keep_first, output_gate
-        self.unit_after, self.has_sink, self.score_cap = unit_norm_after_rotation, sink, score_cap
+        self.unit_after, self.has_sink, self.score_cap = unit_norm_after_rotation, sink is True, score_cap
+        self.sink_score = None if isinstance(sink, bool) else float(sink)        # a sink of one known score in every head
+        if query_temperature is not None and query_temperature[1] <= 0:
+            raise ValueError(f"the query temperature's step must be positive, got {query_temperature[1]}")
+        if value_mix not in (None, "first", "later"):
+            raise ValueError(f"value_mix must be None, 'first' or 'later', got {value_mix!r}")
+        self.query_temperature, self.value_mix, self.distance_bias = query_temperature, value_mix, distance_bias
         self.neighbours = getattr(self.position, "pairing", "halves") == "interleaved"
         # the forms that the kernels preparing whole rows serve (see the module's text)
         self.whole_rows = bool((qk_norm and norm_over == "projection") or self.value_dim != head_dim or keep_first > 0 or output_gate
-                               or unit_norm_after_rotation or sink or score_cap is not None or self.neighbours)
+                               or unit_norm_after_rotation or self.has_sink or self.sink_score is not None or score_cap is not None or self.neighbours
+                               or query_temperature is not None or value_mix is not None or distance_bias)
+        if (unit_norm_after_rotation or self.neighbours) and (query_temperature is not None or value_mix is not None):
+            raise ValueError("a query temperature and mixed values are made by the kernel that normalises over the projection")
         if self.whole_rows and (kv_shared or values_from_keys or (qk_norm and norm_over == "head")):
             raise ValueError("a norm over the projection or after the rotation, values of their own size, kept first positions, a sink, "
                              "capped scores and an output gate come without shared or key-made values and per-head norms before the rotation")
@@ -103,7 +124,7 @@ class GQAAttention(Part):
             raise ValueError("neighbouring pairs are rotated by the kernel that normalises after the rotation or not at all")
         self.b_late = None
         self.gate_width = 0 if not output_gate else num_heads if output_gate == "head" else num_heads * self.value_dim
-        self.sinks = None
+        self.sinks = self.distance = self.mix = None
         self.w_qkv = self.b_qkv = self.w_o = self.q_norm = self.k_norm = None
 
     # ------------------------------------------------------------------ weights
@@ -118,6 +139,11 @@ class GQAAttention(Part):
             specs["g_proj.weight"] = TensorSpec((self.gate_width, h))
         if self.has_sink:
             specs["sink"] = TensorSpec((self.num_heads,), role="bias")
+        if self.value_mix is not None:      # (the layer the others take their values from has no use for its own)
+            specs["value_mix"] = TensorSpec((), role="bias", optional=self.value_mix == "first")
+        if self.distance_bias:              # drawn around one at random: a reach must not be negative
+            specs["distance_rate"] = TensorSpec((self.num_heads,), role="norm")
+            specs["distance_reach"] = TensorSpec((self.num_heads,), role="norm")
         specs["o_proj.weight"] = TensorSpec((h, self.num_heads * self.value_dim))
         if self.qk_norm:
             over = d if self.norm_over == "head" else None
@@ -132,17 +158,18 @@ class GQAAttention(Part):
             names += ("g_proj",)
         stacked = [weights[f"{n}.weight"] for n in names]
         biases = [weights[f"{n}.bias"] if n != "g_proj" else weights["g_proj.weight"].new_zeros(self.gate_width) for n in names] if self.bias else None
-        pad = -sum(w.shape[0] for w in stacked) % 16 if self.whole_rows else 0     # rows of whole groups of 16 columns suit every product kernel
-        if pad:
-            stacked.append(stacked[0].new_zeros(pad, self.hidden_size))
-            if biases is not None:
-                biases.append(biases[0].new_zeros(pad))
-        self.w_qkv = torch.cat(stacked, 0).to(dtype).contiguous()
-        self.b_qkv = torch.cat(biases, 0).to(dtype).contiguous() if self.bias else None
-        # the kernel that rotates and then normalises the heads adds the biases itself, in float32, as it reads the rows
-        self.b_late = torch.cat(biases, 0).float().contiguous() if self.bias and (self.unit_after or self.neighbours) else None
+        self.w_qkv = self.stack_rows(stacked, dtype) if self.whole_rows else torch.cat(stacked, 0).to(dtype).contiguous()
+        self.b_qkv = torch.cat(biases, 0).to(dtype).contiguous() if self.bias and not self.whole_rows else None
+        # the kernels that prepare whole rows add the biases themselves, in float32, as they read the rows
+        self.b_late = torch.cat(biases, 0).float().contiguous() if self.bias and self.whole_rows else None
         if self.has_sink:
             self.sinks = weights["sink"].float().contiguous()
+        elif self.sink_score is not None:
+            self.sinks = torch.full((self.num_heads,), self.sink_score, dtype=torch.float32, device=self.w_qkv.device)
+        if self.value_mix == "later":
+            self.mix = weights["value_mix"].float().reshape(1).contiguous()
+        if self.distance_bias:
+            self.distance = torch.stack((weights["distance_rate"].float(), weights["distance_reach"].float())).contiguous()
         self.w_o = weights["o_proj.weight"].to(dtype).contiguous()
         if self.qk_norm:
             self.q_norm = weights["q_norm.weight"]
@@ -336,19 +363,22 @@ class GQAAttention(Part):
         t, d, dv, nq, nkv = rows_of(x), self.head_dim, self.value_dim, self.num_heads, self.num_kv_heads
         gate_at = (nq + nkv) * d + nkv * dv
         qkv = ctx.scratch("attn_qkvg", (t, self.w_qkv.shape[0]), ctx.dtype)
-        linear(ctx, qkv, x, self.w_qkv, None if self.b_late is not None else self.b_qkv)
+        linear(ctx, qkv, x, self.w_qkv)
+        self.hand_out_carried(ctx, qkv)
         if self.unit_after or self.neighbours:
             ops.rotate_unit_prep(qkv, nq, nkv, d, dv, self.qk_norm_eps, self.unit_after, cos, sin, self.neighbours, cache.k_pages, cache.v_pages,
                                  group.slots, group.page_size, bias=self.b_late)
         else:
+            first = None if self.value_mix is None else ctx.scratch("attn_first_values", (t, nkv * dv), ctx.dtype)
             ops.qkv_norm_prep(qkv, nq, nkv, d, dv, self.q_norm, self.k_norm, self.qk_norm_eps, cos, sin, cache.k_pages, cache.v_pages,
-                              group.slots, group.page_size)
-        more = {"sinks": self.sinks, "softcap": self.score_cap or 0.0}
+                              group.slots, group.page_size, bias=self.b_late, temperature=self.query_temperature, positions=ctx.positions,
+                              first_values=first, value_mix=self.mix)
+        more = {"sinks": self.sinks, "softcap": self.score_cap or 0.0, "distance": self.distance}
         # a gate a head is applied by the attention kernel that finishes a query (or by the merge of its partial results); a
         # gate a value by a kernel of its own behind them
         gates = qkv[:, gate_at:gate_at + nq] if self.output_gate == "head" else None
         out = ctx.scratch("attn_out", (t, nq * dv), ctx.dtype)
-        cores = dv == d and ops.attention_decode_supported(ctx.dtype, nq, nkv, d, group.page_size)
+        cores = ops.attention_decode_supported(ctx.dtype, nq, nkv, d, group.page_size, dv)
         extra = 1 if self.keep_first else 0      # the kept first positions' share is one more partial result for the merge
         if cores and ctx.all_decode:
             longest, bound = ctx.max_k, ctx.max_k_bound
@@ -357,7 +387,7 @@ class GQAAttention(Part):
             splits = self._decode_splits(t * nkv, longest, bound, group.page_size)
             part_o = part_ml = None
             if splits + extra > 1:
-                part_o = ctx.scratch("attn_part_o", (t, nq * (splits + extra) * d), torch.float32)
+                part_o = ctx.scratch("attn_part_o", (t, nq * (splits + extra) * dv), torch.float32)
                 part_ml = ctx.scratch("attn_part_ml", (t, nq * (splits + extra) * 2), torch.float32)
             ops.attention_decode(out, qkv, cache.k_pages, cache.v_pages, group.block_table, ctx.token_slot, ctx.positions,
                                  nq, self.scale, self.window or 0, splits, part_o, part_ml, ctx.max_k_bound, None, form=1,
@@ -369,7 +399,7 @@ class GQAAttention(Part):
                 splits = self._decode_splits(singles * nkv, longest, ctx.max_k_bound, group.page_size)
                 part_o = part_ml = None
                 if splits + extra > 1:
-                    part_o = ctx.scratch("attn_single_part_o", (singles, nq * (splits + extra) * d), torch.float32)
+                    part_o = ctx.scratch("attn_single_part_o", (singles, nq * (splits + extra) * dv), torch.float32)
                     part_ml = ctx.scratch("attn_single_part_ml", (singles, nq * (splits + extra) * 2), torch.float32)
                 ops.attention_decode(out[:singles], qkv[:singles], cache.k_pages, cache.v_pages, group.block_table, ctx.token_slot,
                                      ctx.positions, nq, self.scale, self.window or 0, splits, part_o, part_ml, ctx.max_k_bound, None, form=1,
@@ -377,10 +407,10 @@ class GQAAttention(Part):
             rest = ctx.memo.get("rows_after_singles")
             if rest is None:
                 rest = ctx.memo["rows_after_singles"] = (ctx.token_slot[singles:], ctx.positions[singles:])
-            splits = self._prefill_splits(ctx.num_qblocks * nkv, longest, (t - singles) * nq * d, nq // nkv, t - singles)
+            splits = self._prefill_splits(ctx.num_qblocks * nkv, longest, (t - singles) * nq * dv, nq // nkv, t - singles)
             part_o = part_ml = None
             if splits + extra > 1:
-                part_o = ctx.scratch("attn_part_o", (t - singles, nq * (splits + extra) * d), torch.float32)
+                part_o = ctx.scratch("attn_part_o", (t - singles, nq * (splits + extra) * dv), torch.float32)
                 part_ml = ctx.scratch("attn_part_ml", (t - singles, nq * (splits + extra) * 2), torch.float32)
             ops.attention_prefill(out[singles:], qkv[singles:], cache.k_pages, cache.v_pages, group.block_table, rest[0], rest[1],
                                   ctx.qblock_token0, ctx.qblock_count, nq, self.scale, self.window or 0, ctx.max_qblock, ctx.max_k_bound,

@@ -48,6 +48,12 @@ Optional, each announced by a class attribute (a part without it is simply given
                               gives them to its kernel for decode steps).  Without the attribute nothing is built and
                               ctx.num_qblocks is 0: a model of other mixers does not pay for it
 
+  carries_rows = True         mixer / feed_forward: another matrix that reads the part's own input can be stacked behind its first
+                              product (`carry(matrix)` before bind(); Part.stack_rows and Part.hand_out_carried do the work): after
+                              forward(), ctx.memo["carried_rows"] holds what the matrix made of the input, a view [T, rows] of
+                              the product's output (in that buffer's dtype).  A block whose residual is gated by a matrix of
+                              the sublayer's input saves a launch this way
+
 A part may also say how its steps can be run again without it (both default to no):
 
   graph_safe = True           it launches only kernels on preallocated buffers, and reads the step's data from
@@ -225,6 +231,38 @@ class Part:
 
     def bind(self, weights: Mapping[str, torch.Tensor], dtype: torch.dtype) -> None:
         """Take the device tensors named by tensors(); `dtype` is the activation dtype."""
+
+    # ---- a matrix of somebody else's behind the part's first product (carries_rows)
+    _carried: torch.Tensor | None = None
+    _carried_at = 0
+
+    def carry(self, matrix: torch.Tensor) -> None:
+        """Stack `matrix` [rows, in] behind the part's first product when the part is bound next."""
+        self._carried = matrix
+
+    def stack_rows(self, matrices: list, dtype: torch.dtype) -> torch.Tensor:
+        """`matrices` one under the other in `dtype`, zero rows up to a multiple of 16 (whole groups of 16 output columns suit every
+        product kernel), then the carried matrix and zero rows likewise."""
+        width = matrices[0].shape[1]
+
+        def padded(parts):
+            pad = -sum(m.shape[0] for m in parts) % 16
+            return parts + ([parts[0].new_zeros(pad, width)] if pad else [])
+
+        parts = padded([m.to(dtype) for m in matrices])
+        self._carried_rows = 0
+        if self._carried is not None:
+            self._carried_at, carried = sum(m.shape[0] for m in parts), self._carried.to(dtype)
+            self._carried_rows = carried.shape[0]
+            parts += padded([carried])
+            self._carried = None
+        return torch.cat(parts, 0).contiguous()
+
+    _carried_rows = 0
+
+    def hand_out_carried(self, ctx, product: torch.Tensor) -> None:
+        if self._carried_rows:
+            ctx.memo["carried_rows"] = product[:, self._carried_at:self._carried_at + self._carried_rows]
 
     def weight_bytes(self) -> int:
         """Bytes of weights that one step reads (for roofline accounting)."""

@@ -22,6 +22,14 @@ ParallelBlock: one norm, and both sublayers read its output; their sum, times a 
 The mixer stores its output into a float32 buffer of the step, the feed-forward adds into it, and one kernel adds the buffer
 into the stream and leaves the next block's norm of the new stream beside it (`axpby` with a norm), which the model hands
 to the block that runs next if that is one of this kind.
+
+SandwichBlock: a norm before and a norm after each sublayer, the sublayer's output gated by its own input before the second norm and
+scaled after it:
+    x = norm1(h);  h = h + scale1 * norm1b(mixer(x) * sigmoid(G1 x + g1)), then the feed-forward likewise (it may be absent)
+The gate's matrix is stacked behind the sublayer's first product where the sublayer can carry it, the scale is part of the second
+norm's weight, and one kernel (`gated_norm_add`) gates, normalises, adds into the stream and leaves the norm that comes next, in this
+layer or the next one, beside it.  Gate and scale are parameters of the block: with neither it is the plain arrangement of norms on
+both sides.
 """
 
 from __future__ import annotations
@@ -29,8 +37,8 @@ from __future__ import annotations
 import torch
 
 from ..kernels import ops
-from .base import Part, PartSpec, create, flops_of, register, under
-from .linear import materialize
+from .base import Part, PartSpec, TensorSpec, create, flops_of, register, under
+from .linear import linear, materialize
 
 
 class PreNormBlock(Part):
@@ -378,3 +386,112 @@ class ParallelBlock(Part):
 
 
 register("block", "parallel", ParallelBlock)
+
+
+class SandwichBlock(ParallelBlock):
+    """Norms on both sides of every sublayer, optionally a gate on the sublayer's output and a scale behind the second norm.  What is
+    handed to the next block, and what a block says of itself, are ParallelBlock's."""
+
+    def __init__(self, mixer: PartSpec, mixer_norm: PartSpec, mixer_out_norm: PartSpec, feed_forward: PartSpec | None = None,
+                 ff_norm: PartSpec | None = None, ff_out_norm: PartSpec | None = None, gated: bool = False, scaled: bool = False,
+                 names: dict | None = None):
+        if (feed_forward is None) != (ff_norm is None) or (feed_forward is None) != (ff_out_norm is None):
+            raise ValueError("a feed-forward and its two norms come together")
+        self.mixer = create("mixer", mixer)
+        self.feed_forward = None if feed_forward is None else create("feed_forward", feed_forward)
+        self.mixer_norm, self.mixer_out_norm = create("norm", mixer_norm), create("norm", mixer_out_norm)
+        self.ff_norm = None if ff_norm is None else create("norm", ff_norm)
+        self.ff_out_norm = None if ff_out_norm is None else create("norm", ff_out_norm)
+        for part in (self.mixer, self.feed_forward):
+            if part is not None and not getattr(part, "can_overwrite", False):
+                raise ValueError(f"a sublayer between two norms must store its output (accumulate=False): {type(part).__name__} cannot")
+        for norm in (self.mixer_norm, self.mixer_out_norm, self.ff_norm, self.ff_out_norm):
+            if norm is not None and not callable(getattr(norm, "rms_parameters", None)):
+                raise ValueError("the norms on both sides of a sublayer must be RMS norms (rms_parameters)")
+        self.gated, self.scaled = gated, scaled
+        self.names = {name: name for name in ("mixer", "feed_forward", "mixer_norm", "mixer_out_norm", "ff_norm", "ff_out_norm",
+                                              "mixer_gate", "ff_gate", "mixer_scale", "ff_scale")}
+        self.names.update(names or {})
+        self._bound: dict = {}
+
+    def _children(self):
+        return [(self.names[k], getattr(self, k)) for k in ("mixer_norm", "mixer", "mixer_out_norm", "ff_norm", "feed_forward", "ff_out_norm")
+                if getattr(self, k) is not None]
+
+    def _sublayers(self):
+        yield "mixer", self.mixer, self.mixer_out_norm
+        if self.feed_forward is not None:
+            yield "ff", self.feed_forward, self.ff_out_norm
+
+    def tensors(self):
+        out = super().tensors()
+        size = self.mixer_norm.size
+        for which, _, _ in self._sublayers():
+            if self.gated:
+                out[self.names[f"{which}_gate"] + ".weight"] = TensorSpec((size, size))
+                out[self.names[f"{which}_gate"] + ".bias"] = TensorSpec((size,), role="bias")
+            if self.scaled:
+                out[self.names[f"{which}_scale"] + ".weight"] = TensorSpec((size,), role="norm")
+        return out
+
+    def bind(self, weights, dtype):
+        matrices = {}
+        if self.gated:
+            for which, part, _ in self._sublayers():
+                matrix = weights[self.names[f"{which}_gate"] + ".weight"]
+                if getattr(part, "carries_rows", False):
+                    part.carry(matrix)
+                else:
+                    matrices[which] = matrix.to(dtype).contiguous()
+        super().bind(weights, dtype)
+        for which, _, norm in self._sublayers():
+            weight, eps = norm.rms_parameters()
+            weight = weight.float()
+            if self.scaled:
+                weight = weight * weights[self.names[f"{which}_scale"] + ".weight"].float()
+            bias = weights[self.names[f"{which}_gate"] + ".bias"].float().contiguous() if self.gated else None
+            self._bound[which] = (weight.contiguous(), eps, matrices.get(which), bias)
+
+    def weight_bytes(self):
+        return super().weight_bytes() + sum(m.numel() * m.element_size() for _, _, m, _ in self._bound.values() if m is not None)
+
+    def flops(self, tokens, pairs):
+        gates = 2.0 * tokens * self.mixer_norm.size ** 2 * sum(1 for _ in self._sublayers()) if self.gated else 0.0
+        return super().flops(tokens, pairs) + gates
+
+    @property
+    def first_norm(self):
+        return self.mixer_norm
+
+    def forward(self, ctx, h, cache, given=None, next_norm=None):
+        x = given[1] if given is not None and given[0] is self.mixer_norm else self.mixer_norm.forward(ctx, h)
+        x = self._update(ctx, "mixer", self.mixer, x, h, (cache,), self.ff_norm if self.feed_forward is not None else next_norm)
+        if self.feed_forward is not None:
+            x = self._update(ctx, "ff", self.feed_forward, x, h, (), next_norm)
+        return None if x is None else (next_norm, x)
+
+    def _update(self, ctx, which, part, x, h, more, following):
+        """h += scale * norm(part(x) * gate(x)); returns the following norm of the new stream, if that is one this kernel makes."""
+        weight, eps, matrix, bias = self._bound[which]
+        y = ctx.scratch("sublayer_out", tuple(h.shape), torch.float32)
+        gate = None
+        ctx.memo.pop("carried_rows", None)
+        part.forward(ctx, x, y, *more, accumulate=False)
+        if matrix is not None:
+            gate = ctx.scratch("sublayer_gate", tuple(h.shape), ctx.dtype)
+            linear(ctx, gate, materialize(ctx, x), matrix)
+        elif self.gated:
+            gate = ctx.memo.pop("carried_rows")
+        parameters = getattr(following, "rms_parameters", None)
+        if parameters is None:
+            ops.gated_norm_add(h, y, gate, bias, weight, eps)
+            return None
+        next_weight, next_eps = parameters()
+        turn = ctx.memo["normed_stream_turn"] = 1 - ctx.memo.get("normed_stream_turn", 0)     # not the buffer x lies in
+        normed = ctx.scratch(f"stream_normed{turn}", tuple(h.shape), ctx.dtype)
+        next_weight = next_weight if next_weight.dtype == torch.float32 else self._weight_f32(following, next_weight)
+        ops.gated_norm_add(h, y, gate, bias, weight, eps, next_weight, next_eps, normed)
+        return normed
+
+
+register("block", "sandwich", SandwichBlock)

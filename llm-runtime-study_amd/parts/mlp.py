@@ -1,6 +1,6 @@
 """Feed-forwards.  SwiGLU: down(silu(gate(x)) * up(x)), three bias-free projections (with `activation="clamped"` the gated
 activation is g * sigmoid(alpha g) * (u + 1), g = min(gate(x), limit), u = clamp(up(x), -limit, limit)); DenseMLP (at the end of the file):
-down(act(up(x))), two bias-free projections with an activation between them.
+down(act(up(x))), two bias-free projections with an activation between them (one of them, "xielu", has two learned numbers).
 
 Reference mini_llm/nn/mlp.py:80-87.  gate and up are stacked into one [2I, H] matrix when
 the weights are bound, so one product feeds the gated activation; the down projection adds
@@ -79,27 +79,39 @@ register("feed_forward", "swiglu", SwiGLU)
 
 class DenseMLP(Part):
     """down(act(up(x))): two bias-free projections, `activation` between them: "gelu" (the exact one, 0.5 z (1 + erf(z / sqrt 2))),
-    "gelu_tanh", "silu" or "relu" (kernels/ops.py, ACTIVATIONS).  The down projection adds into the float32 rows it is given, or
+    "gelu_tanh", "silu" or "relu" (kernels/ops.py, ACTIVATIONS), or "xielu", which has two learned numbers (p, q): with z = up(x),
+    softplus(p) z^2 + z / 2 for z > 0 and (1/2 + softplus(q)) (exp(z) - 1 - z) + z / 2 otherwise.  The down projection adds into the float32 rows it is given, or
     stores into them with `accumulate=False`."""
 
     graph_safe = True
     plan_safe = True
     can_overwrite = True
 
+    @property
+    def carries_rows(self) -> bool:
+        return self.activation == "xielu"      # its kernel reads rows of any stride
+
     def __init__(self, hidden_size: int, intermediate_size: int, activation: str = "gelu"):
         if hidden_size <= 0 or intermediate_size <= 0:
             raise ValueError("hidden_size and intermediate_size must be positive")
-        if activation not in ops.ACTIVATIONS:
-            raise ValueError(f"unknown activation {activation!r}; known: {', '.join(ops.ACTIVATIONS)}")
+        if activation not in ops.ACTIVATIONS and activation != "xielu":
+            raise ValueError(f"unknown activation {activation!r}; known: {', '.join(ops.ACTIVATIONS)}, xielu")
         self.hidden_size, self.intermediate_size, self.activation = hidden_size, intermediate_size, activation
-        self.up = self.down = None
+        self.up = self.down = self.numbers = None
 
     def tensors(self):
-        return {"up_proj.weight": TensorSpec((self.intermediate_size, self.hidden_size)),
-                "down_proj.weight": TensorSpec((self.hidden_size, self.intermediate_size))}
+        specs = {"up_proj.weight": TensorSpec((self.intermediate_size, self.hidden_size)),
+                 "down_proj.weight": TensorSpec((self.hidden_size, self.intermediate_size))}
+        if self.activation == "xielu":
+            specs["act"] = TensorSpec((2,), role="bias")
+        return specs
 
     def bind(self, weights, dtype):
-        self.up = weights["up_proj.weight"].to(dtype).contiguous()
+        up = weights["up_proj.weight"]
+        self.up = up.to(dtype).contiguous() if self._carried is None else self.stack_rows([up], dtype)
+        if self.activation == "xielu":
+            p, q = torch.nn.functional.softplus(weights["act"].double())
+            self.numbers = torch.stack((p, 0.5 + q)).float().contiguous()
         self.down = weights["down_proj.weight"].to(dtype).contiguous()
 
     def weight_bytes(self):
@@ -108,8 +120,18 @@ class DenseMLP(Part):
     def forward(self, ctx, x, residual, then_norm=None, accumulate: bool = True):
         t = rows_of(x)
         act = ctx.scratch("ffn_act", (t, self.intermediate_size), ctx.dtype)
-        linear(ctx, act, x, self.up)
-        ops.activation(act, act, self.activation)
+        rows = self.up.shape[0]
+        if rows == self.intermediate_size:
+            up = act                         # the activation works in place
+        else:
+            up = ctx.scratch("ffn_up_and_carried", (t, rows), ctx.dtype)
+        linear(ctx, up, x, self.up)
+        self.hand_out_carried(ctx, up)
+        up = up[:, :self.intermediate_size]
+        if self.activation == "xielu":
+            ops.xielu(act, up, self.numbers)
+        else:
+            ops.activation(act, up, self.activation)
         return linear(ctx, residual, act, self.down, accumulate=accumulate, then_norm=then_norm)
 
 
