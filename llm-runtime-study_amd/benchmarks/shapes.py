@@ -67,12 +67,27 @@ def napizen_like(shape: dict, layers: int, experts: int = 32, top: int = 8, rank
             "layers": [{"type": "latent_attention", "mixer": mixer, "mlp": routed if index % 2 else dense} for index in range(layers)]}
 
 
-def kaposun_like(shape: dict, layers: int, window: int = 4096, keep_first: int = 8, state: int = 128) -> dict:
+def mutolix_like(shape: dict, layers: int) -> dict:
+    """A Mutolix configuration with the layer sizes of a dense shape above, for measurements beside a model of equal sizes: the same
+    width, vocabulary and attention heads; of every four layers the first and the last are matrix memories without feed-forward
+    (heads of 256 x 512 numbers, one for every 512 values of the width: as many numbers as kaposun_like's state space layers
+    keep) and the two between attention with the dense feed-forward's size (two matrices where the shape has three)."""
+    width, heads, kv_heads, dim = shape["hidden_size"], shape["num_attention_heads"], shape["num_key_value_heads"], shape["head_dim"]
+    memory = {"type": "mlstm", "mlp": None, "mixer": {"heads": width // 512, "dim": 256, "vdim": 512, "gate_cap": 15.0}}
+    attention = {"type": "attention", "mlp": {"kind": "dense", "ff": shape["intermediate_size"]},
+                 "mixer": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": dim ** -0.5, "v_mix": True,
+                           "q_temp": {"coef": 0.1, "every": 1024}}}
+    return {"architecture": "Mutolix", "vocab": shape["vocab_size"], "width": width, "norm": {"eps": 1e-6}, "embedding": {"scale": 1.0},
+            "layers": [(memory, attention, attention, memory)[index % 4] for index in range(layers)]}
+
+
+def kaposun_like(shape: dict, layers: int, window: int = 4096, keep_first: int = 8, state: int = 128, order: str = "each") -> dict:
     """A Kaposun configuration with the layer sizes of a dense shape above, for measurements beside it: the same width,
     vocabulary, heads and dense feed-forward size (two matrices where the shape has three); in turn a state space layer
     (inner size twice the width in heads of 64 values, `state` numbers a value, 8 groups), an attention layer over the whole
     context with stretched rotation, a layer of windowed attention with kept first positions and an output gate beside the
-    gated delta rule with channel decays, and another attention layer; no stretch of layers runs twice."""
+    gated delta rule with channel decays, and another attention layer; no stretch of layers runs twice.  order "ends": mutolix_like's
+    order instead, of every four layers the first and the last state space layers without feed-forward, the two between attention."""
     width, heads, kv_heads, dim = shape["hidden_size"], shape["num_attention_heads"], shape["num_key_value_heads"], shape["head_dim"]
     mlp = {"kind": "dense", "ff": shape["intermediate_size"]}
     sizes = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": dim ** -0.5}
@@ -82,4 +97,5 @@ def kaposun_like(shape: dict, layers: int, window: int = 4096, keep_first: int =
                                                       "right": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "conv": 4},
                                                       "left_scale": 1.0, "right_scale": 1.0}}
     return {"architecture": "Kaposun", "vocab": shape["vocab_size"], "width": width, "norm": {"eps": 1e-6}, "residual_mult": 0.5,
-            "layers": [(state_space, attention, pair, attention)[index % 4] for index in range(layers)]}
+            "layers": [((state_space, attention, pair, attention) if order == "each" else
+                        (dict(state_space, mlp=None), attention, attention, dict(state_space, mlp=None)))[index % 4] for index in range(layers)]}

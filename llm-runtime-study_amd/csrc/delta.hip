@@ -625,6 +625,7 @@ LRS_API int lrs_ssm(void* out, int out_dtype, const void* proj, int proj_dtype, 
 //   mlstm_single steps of one token a request: gates and recurrence in one kernel, a workgroup 16 columns of a head's matrix;
 //   mlstm_read   per (token, head): the read-out over its normaliser, divided by its root mean square, times the norm's weight,
 //                times the sigmoid of the output gate.
+// (mlstm_chunks.hip has the form for long portions on the matrix cores.)
 // A request's state row: S of every head (d padded to 16 lanes of rows, vdim + 1 columns), then m of every head.
 namespace {
 
@@ -728,13 +729,14 @@ __global__ __launch_bounds__(256) void mlstm_single_kernel(const float* __restri
   }
 }
 
-// A wave a (token, head).  raw [tokens, H, dv + 1]: the read-out and, last, n . q (both without q's factor).  maxima given (steps
-// of one token a request): the request's new m, moved into its state row here.
+// A wave a (token, head).  raw [tokens, H, dv + 1]: the read-out and, last, n . q (both without q's factor).  maxima given
+// [requests, H]: the requests' new m, moved into their state rows here (by the wave of a request's last token).
 template <typename TO>
 __global__ __launch_bounds__(256) void mlstm_read_kernel(const float* __restrict__ raw, const float* __restrict__ floors,
                                                          const float* __restrict__ proj, int ld, int g_at, const float* __restrict__ norm_w,
                                                          float q_factor, float eps, int tokens, int H, int dv, TO* __restrict__ out,
-                                                         const float* __restrict__ maxima, const int* __restrict__ slot_ids,
+                                                         const float* __restrict__ maxima, const int* __restrict__ token_request,
+                                                         const int* __restrict__ cu, const int* __restrict__ slot_ids,
                                                          float* __restrict__ state, int64_t state_stride, int64_t m_offset) {
   const int64_t pair = (int64_t)blockIdx.x * (blockDim.x / WAVE) + threadIdx.x / WAVE;
   const int lane = threadIdx.x % WAVE;
@@ -765,10 +767,27 @@ __global__ __launch_bounds__(256) void mlstm_read_kernel(const float* __restrict
     if (i < dv) dst[i] = from_float<TO>(x[n] * inv * w[i] / (1.f + expf(-z[n])));
   }
   for (int i = lane + HELD * WAVE; i < dv; i += WAVE) dst[i] = from_float<TO>(o[i] * scale * inv * w[i] / (1.f + expf(-gate[i])));
-  if (maxima && lane == 0) state[(int64_t)slot_ids[token] * state_stride + m_offset + h] = maxima[pair];
+  if (maxima && lane == 0) {
+    const int r = token_request ? token_request[token] : (int)token;      // (null: one token a request)
+    if (!token_request || token == cu[r + 1] - 1) state[(int64_t)slot_ids[r] * state_stride + m_offset + h] = maxima[(int64_t)r * H + h];
+  }
 }
 
 }  // namespace
+
+int lrs_mlstm_read_out(void* out, int out_dtype, const float* raw, const float* floors, const float* proj, int ld, int g_at, const float* norm_w,
+                       float q_factor, float eps, int tokens, int requests, int H, int dv, const float* maxima, const int* token_request, const int* cu,
+                       const int* slot_ids, float* state, int64_t state_stride, int64_t m_offset, hipStream_t s) {
+  const unsigned blocks = (unsigned)(((int64_t)tokens * H + 3) / 4);
+  if (tokens == requests) token_request = nullptr;
+  if (out_dtype == LRS_F32)
+    mlstm_read_kernel<float><<<blocks, 256, 0, s>>>(raw, floors, proj, ld, g_at, norm_w, q_factor, eps, tokens, H, dv, (float*)out, maxima, token_request,
+                                                    cu, slot_ids, state, state_stride, m_offset);
+  else
+    mlstm_read_kernel<bf16><<<blocks, 256, 0, s>>>(raw, floors, proj, ld, g_at, norm_w, q_factor, eps, tokens, H, dv, (bf16*)out, maxima, token_request,
+                                                   cu, slot_ids, state, state_stride, m_offset);
+  return lrs_check_launch("mlstm_read");
+}
 
 // One step for a ragged batch.  proj [tokens, ld] float32: q (H*d) | k (H*d) | v (H*dv) | output gate (H*dv) | input gate (H) |
 // forget gate (H) | anything.  State rows: H * rows * 16 * (dv + 1) floats, then H.  gates [tokens, 2*H], floors [tokens, H] and raw
@@ -814,14 +833,6 @@ LRS_API int lrs_mlstm(void* out, int out_dtype, const float* proj, int ld, int t
 #undef SCAN
   }
   if (lrs_check_launch("mlstm")) return 1;
-  const int64_t pairs = (int64_t)tokens * H;
-  const unsigned blocks = (unsigned)((pairs + 3) / 4);
-  const float q_factor = 1.0f / sqrtf((float)d);
-  if (out_dtype == LRS_F32)
-    mlstm_read_kernel<float><<<blocks, 256, 0, s>>>(raw, floors, proj, ld, g_at, norm_w, q_factor, eps, tokens, H, dv, (float*)out, maxima, slot_ids,
-                                                    state, state_stride, m_offset);
-  else
-    mlstm_read_kernel<bf16><<<blocks, 256, 0, s>>>(raw, floors, proj, ld, g_at, norm_w, q_factor, eps, tokens, H, dv, (bf16*)out, maxima, slot_ids,
-                                                   state, state_stride, m_offset);
-  return lrs_check_launch("mlstm_read");
+  return lrs_mlstm_read_out(out, out_dtype, raw, floors, proj, ld, g_at, norm_w, 1.0f / sqrtf((float)d), eps, tokens, requests, H, dv, maxima,
+                            nullptr, cu, slot_ids, state, state_stride, m_offset, s);
 }

@@ -132,6 +132,10 @@ _SIGNATURES = {
     "lrs_xielu": (c_int, [c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_int, c_void_p, c_void_p]),
     "lrs_mlstm": (c_int, [c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p, c_int64, c_int, c_int, c_int,
                           c_void_p, c_void_p, c_float, c_void_p, c_float, c_void_p, c_void_p, c_void_p, c_void_p]),
+    "lrs_mlstm_slots": (c_int, [c_int, c_int]),
+    "lrs_mlstm_chunks": (c_int, [c_void_p, c_void_p, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_int64, c_int, c_int, c_int,
+                                 c_void_p, c_void_p, c_float, c_void_p, c_float, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
+                                 c_void_p, c_void_p]),
     "lrs_sigmoid_gate": (c_int, [c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p]),
     "lrs_rotate_unit_prep": (c_int, [c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_void_p, c_void_p, c_int, c_int,
                                      c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p]),
@@ -229,7 +233,7 @@ def library():
 PLAN_OPS = ("lrs_activation", "lrs_add_gathered", "lrs_add_into", "lrs_add_rmsnorm", "lrs_advance_decode", "lrs_advance_slots", "lrs_attention", "lrs_attention_decode",
             "lrs_attention_prefill", "lrs_axpby", "lrs_choose_tokens", "lrs_choose_tokens_split", "lrs_copy_to_pinned", "lrs_delta_rule", "lrs_delta_rule_channels", "lrs_embed", "lrs_fill_i32",
             "lrs_filter_logits", "lrs_gated_clamped", "lrs_gated_norm_add", "lrs_gather_rows", "lrs_gemm", "lrs_gemm_lines_add_rmsnorm", "lrs_gemm_mid_add_norm_begin", "lrs_gemm_mid_qk_prep", "lrs_gemm_mid_scaled",
-            "lrs_gemm_norm_chain", "lrs_head_gemm", "lrs_latent_attention", "lrs_latent_attention_groups", "lrs_latent_prep", "lrs_layernorm", "lrs_library_gemm", "lrs_mlstm", "lrs_moe_align", "lrs_moe_combine", "lrs_moe_experts", "lrs_moe_route", "lrs_moe_route_align", "lrs_norm_add",
+            "lrs_gemm_norm_chain", "lrs_head_gemm", "lrs_latent_attention", "lrs_latent_attention_groups", "lrs_latent_prep", "lrs_layernorm", "lrs_library_gemm", "lrs_mlstm", "lrs_mlstm_chunks", "lrs_moe_align", "lrs_moe_combine", "lrs_moe_experts", "lrs_moe_route", "lrs_moe_route_align", "lrs_norm_add",
             "lrs_qk_prep", "lrs_qkv_norm_prep", "lrs_rmsnorm", "lrs_rope_table", "lrs_rotate_unit_prep", "lrs_round_rows", "lrs_scale_add_layernorm", "lrs_scale_rows", "lrs_scale_values", "lrs_sigmoid_gate", "lrs_silu_mul", "lrs_soft_cap", "lrs_ssm", "lrs_xielu")
 _PLAN_INDEX = {name: index for index, name in enumerate(PLAN_OPS)}
 
@@ -1531,27 +1535,58 @@ def mlstm_state_floats(heads: int, dim: int, vdim: int) -> int:
     return heads * library().lrs_delta_state_rows(dim) * 16 * (vdim + 1) + heads
 
 
+def _mlstm_arguments(who: str, out, proj, state, cu_seqlens, slot_ids, requests, heads, dim, vdim, i_bias, f_bias, norm_weight, floors, raw) -> int:
+    tokens = out.shape[0]
+    _need(out.is_contiguous() and out.shape[1] == heads * vdim, f"{who}: out must be contiguous [T, heads*vdim]")
+    _need(proj.dtype == torch.float32 and proj.shape[0] >= tokens and proj.shape[1] >= 2 * heads * (dim + vdim + 1), f"{who}: proj must be float32 and hold every column")
+    _need(state.dim() == 2 and state.dtype == torch.float32 and state.is_contiguous() and state.shape[1] >= mlstm_state_floats(heads, dim, vdim),
+          f"{who}: state rows are too short")
+    for name, t, count in (("i_bias", i_bias, heads), ("f_bias", f_bias, heads), ("norm_weight", norm_weight, heads * vdim)):
+        _need(t.dtype == torch.float32 and t.numel() == count and t.is_contiguous(), f"{who}: {name} must hold {count} float32 values")
+    for name, t, count in (("cu_seqlens", cu_seqlens, requests + 1), ("slot_ids", slot_ids, requests)):
+        _need(t.dtype == torch.int32 and t.numel() >= count and t.is_contiguous(), f"{who}: {name} must be int32 [{count}]")
+    for name, t, count in (("floors", floors, tokens * heads), ("raw", raw, tokens * heads * (vdim + 1))):
+        _need(t.dtype == torch.float32 and t.is_contiguous() and t.numel() >= count, f"{who}: {name} scratch too small")
+    return tokens
+
+
 def mlstm(out: torch.Tensor, proj: torch.Tensor, state: torch.Tensor, cu_seqlens: torch.Tensor, slot_ids: torch.Tensor, requests: int, heads: int,
           dim: int, vdim: int, i_bias: torch.Tensor, f_bias: torch.Tensor, cap: float, norm_weight: torch.Tensor, eps: float,
           gates: torch.Tensor, floors: torch.Tensor, raw: torch.Tensor) -> None:
     """One step of the matrix memory for a ragged batch.  proj float32 [T, >= C], columns q (heads*dim) | k (heads*dim) |
     v (heads*vdim) | output gate (heads*vdim) | input gate (heads) | forget gate (heads); state [slots, floats] float32 is read and
     written at the rows slot_ids names; i_bias, f_bias [heads], norm_weight [heads*vdim]; out [T, heads*vdim]."""
-    tokens = out.shape[0]
-    _need(out.is_contiguous() and out.shape[1] == heads * vdim, "mlstm: out must be contiguous [T, heads*vdim]")
-    _need(proj.dtype == torch.float32 and proj.shape[0] >= tokens and proj.shape[1] >= 2 * heads * (dim + vdim + 1), "mlstm: proj must be float32 and hold every column")
-    _need(state.dim() == 2 and state.dtype == torch.float32 and state.is_contiguous() and state.shape[1] >= mlstm_state_floats(heads, dim, vdim),
-          "mlstm: state rows are too short")
-    for name, t, count in (("i_bias", i_bias, heads), ("f_bias", f_bias, heads), ("norm_weight", norm_weight, heads * vdim)):
-        _need(t.dtype == torch.float32 and t.numel() == count and t.is_contiguous(), f"mlstm: {name} must hold {count} float32 values")
-    for name, t, count in (("cu_seqlens", cu_seqlens, requests + 1), ("slot_ids", slot_ids, requests)):
-        _need(t.dtype == torch.int32 and t.numel() >= count and t.is_contiguous(), f"mlstm: {name} must be int32 [{count}]")
-    for name, t, count in (("gates", gates, tokens * 2 * heads), ("floors", floors, tokens * heads), ("raw", raw, tokens * heads * (vdim + 1))):
-        _need(t.dtype == torch.float32 and t.is_contiguous() and t.numel() >= count, f"mlstm: {name} scratch too small")
+    tokens = _mlstm_arguments("mlstm", out, proj, state, cu_seqlens, slot_ids, requests, heads, dim, vdim, i_bias, f_bias, norm_weight, floors, raw)
+    _need(gates.dtype == torch.float32 and gates.is_contiguous() and gates.numel() >= tokens * 2 * heads, "mlstm: gates scratch too small")
     _launch("lrs_mlstm", _dev(out, "out"), dtype_code(out.dtype), _dev(proj, "proj"), _rows(proj, "proj"), tokens, requests,
             _dev(cu_seqlens, "cu_seqlens"), _dev(slot_ids, "slot_ids"), _dev(state, "state"), state.stride(0), heads, dim, vdim,
             _dev(i_bias, "i_bias"), _dev(f_bias, "f_bias"), cap, _dev(norm_weight, "norm_weight"), eps, _dev(gates, "gates"),
             _dev(floors, "floors"), _dev(raw, "raw"), _stream())
+
+
+def mlstm_pack_sizes(tokens: int, requests: int, heads: int, dim: int) -> tuple:
+    """Elements of mlstm_chunks()'s packs (q, k, the scores: bfloat16; the gates: float32) for a step of that shape."""
+    pairs = library().lrs_mlstm_slots(tokens, requests) * heads
+    padded = 16 * library().lrs_delta_state_rows(dim)
+    return pairs * 64 * padded, pairs * 64 * padded, pairs * 2 * 64 * 64, pairs * 3 * 64
+
+
+def mlstm_chunks(out: torch.Tensor, proj: torch.Tensor, state: torch.Tensor, token_request: torch.Tensor, cu_seqlens: torch.Tensor,
+                 slot_ids: torch.Tensor, requests: int, heads: int, dim: int, vdim: int, i_bias: torch.Tensor, f_bias: torch.Tensor, cap: float,
+                 norm_weight: torch.Tensor, eps: float, maxima: torch.Tensor, floors: torch.Tensor, raw: torch.Tensor, packs: tuple) -> None:
+    """mlstm() for steps with long portions in bfloat16: chunks of 64 tokens on the matrix cores (the state in float32).  maxima
+    float32 [requests, heads] scratch, packs: four buffers of mlstm_pack_sizes()."""
+    tokens = _mlstm_arguments("mlstm_chunks", out, proj, state, cu_seqlens, slot_ids, requests, heads, dim, vdim, i_bias, f_bias, norm_weight, floors, raw)
+    _need(out.dtype == torch.bfloat16, "mlstm_chunks: serves bfloat16 runs only")
+    _need(token_request.dtype == torch.int32 and token_request.numel() >= tokens and token_request.is_contiguous(), "mlstm_chunks: token_request must be int32 [T]")
+    _need(maxima.dtype == torch.float32 and maxima.is_contiguous() and maxima.numel() >= requests * heads, "mlstm_chunks: maxima scratch too small")
+    for name, t, count, dtype in zip(("q", "k", "score", "gate"), packs, mlstm_pack_sizes(tokens, requests, heads, dim),
+                                     (torch.bfloat16, torch.bfloat16, torch.bfloat16, torch.float32)):
+        _need(t.dtype == dtype and t.is_contiguous() and t.numel() >= count, f"mlstm_chunks: the {name} pack is too small")
+    _launch("lrs_mlstm_chunks", _dev(out, "out"), _dev(proj, "proj"), _rows(proj, "proj"), tokens, requests, _dev(token_request, "token_request"),
+            _dev(cu_seqlens, "cu_seqlens"), _dev(slot_ids, "slot_ids"), _dev(state, "state"), state.stride(0), heads, dim, vdim,
+            _dev(i_bias, "i_bias"), _dev(f_bias, "f_bias"), cap, _dev(norm_weight, "norm_weight"), eps, _dev(maxima, "maxima"),
+            _dev(floors, "floors"), _dev(raw, "raw"), *(_dev(t, "pack") for t in packs), _stream())
 
 
 # ------------------------------------------------------------------- routed experts

@@ -17,6 +17,10 @@ The recurrence is the scan of the gated delta rule's kernels without its correct
 (csrc/delta.hip, RULE_WEIGHTED); n is one more column of S, whose value is always one.  A request keeps one float32 row: the matrices of
 all heads in the order the scan's threads hold them, then m of every head (`StateNeed`; the cache manager clears a row at
 admission, which is what a sequence starts from).
+
+The scan is sequential over a request's tokens.  bfloat16 runs take another form for steps that hold more than single tokens: chunks
+of 64 tokens on the matrix cores, the state carried between them in float32 (csrc/mlstm_chunks.hip).  float32 runs always scan, so
+that their sums do not depend on how a prompt was cut.
 """
 
 from __future__ import annotations
@@ -30,6 +34,8 @@ from .linear import linear, materialize, rows_of
 
 
 class MatrixMemory(Part):
+    CHUNK_FROM = 16     # tokens of a step beyond one a request from which on the chunked form serves a bfloat16 run
+
     graph_safe = True   # launches only this package's kernels on arena buffers, reads the step's data on the device
     plan_safe = True
     can_overwrite = True
@@ -89,11 +95,18 @@ class MatrixMemory(Part):
         linear(ctx, proj, x, self.w_in)
         self.hand_out_carried(ctx, proj)
         out = ctx.scratch("mlstm_out", (t, heads * self.value_dim), ctx.dtype)
-        gates = ctx.scratch("mlstm_gates", (t, 2 * heads), torch.float32)
         floors = ctx.scratch("mlstm_floors", (t, heads), torch.float32)
         raw = ctx.scratch("mlstm_read_out", (t, heads * (self.value_dim + 1)), torch.float32)
-        ops.mlstm(out, proj, cache.state, ctx.cu_seqlens_q, ctx.slot_ids, ctx.R, heads, self.head_dim, self.value_dim, self.i_bias, self.f_bias,
-                  self.gate_cap, self.norm, self.norm_eps, gates, floors, raw)
+        if ctx.dtype == torch.bfloat16 and t - ctx.R >= self.CHUNK_FROM:
+            packs = tuple(ctx.scratch(f"mlstm_pack{number}", (size,), torch.float32 if number == 3 else torch.bfloat16)
+                          for number, size in enumerate(ops.mlstm_pack_sizes(t, ctx.R, heads, self.head_dim)))
+            maxima = ctx.scratch("mlstm_maxima", (ctx.R, heads), torch.float32)
+            ops.mlstm_chunks(out, proj, cache.state, ctx.token_request, ctx.cu_seqlens_q, ctx.slot_ids, ctx.R, heads, self.head_dim, self.value_dim,
+                             self.i_bias, self.f_bias, self.gate_cap, self.norm, self.norm_eps, maxima, floors, raw, packs)
+        else:
+            gates = ctx.scratch("mlstm_gates", (t, 2 * heads), torch.float32)
+            ops.mlstm(out, proj, cache.state, ctx.cu_seqlens_q, ctx.slot_ids, ctx.R, heads, self.head_dim, self.value_dim, self.i_bias, self.f_bias,
+                      self.gate_cap, self.norm, self.norm_eps, gates, floors, raw)
         linear(ctx, residual, out, self.w_o, accumulate=accumulate)
         return None
 
