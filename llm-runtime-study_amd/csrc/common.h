@@ -57,6 +57,19 @@ __device__ __forceinline__ float block_sum(float v, float* scratch) {
   for (int i = 0; i < waves; ++i) total += scratch[i];
   return total;
 }
+
+// Two such sums at once (`scratch` holds 32 floats): the price of one.
+__device__ __forceinline__ void block_sum2(float& a, float& b, float* scratch) {
+  a = wave_sum(a);
+  b = wave_sum(b);
+  const int wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;
+  const int waves = (blockDim.x + WAVE - 1) / WAVE;
+  __syncthreads();
+  if (lane == 0) scratch[2 * wave] = a, scratch[2 * wave + 1] = b;
+  __syncthreads();
+  a = b = 0.f;
+  for (int w = 0; w < waves; ++w) a += scratch[2 * w], b += scratch[2 * w + 1];
+}
 __device__ __forceinline__ float block_max(float v, float* scratch) {
   v = wave_max(v);
   const int wave = threadIdx.x / WAVE, lane = threadIdx.x % WAVE;

@@ -32,8 +32,12 @@ __device__ __forceinline__ void split_bf16(float x, bf16& hi, bf16& lo) {
   lo = (bf16)(x - (float)hi);
 }
 
-// q_pack [slot, H, L, DP], k_pack [slot, H, DP, L], p_pack [slot, H, 2, L, L] (the two halves of P, [t][s]), gate_pack
-// [slot, H, 3, L]: F, J, mu (tokens past the request's end: F and mu of its last token, J -inf, q, k and P zero).
+// The packs hold operands in the order in which a wave's lanes take them: of every 16 rows and 32 columns of the product, row
+// r's eight columns 8 g .. 8 g + 7 are lane 16 g + r's 16 bytes, so that a load is 1,024 bytes in a row.
+__device__ __forceinline__ int fragment(int rows16, int steps, int step, int row, int g) { return ((rows16 * steps + step) * WAVE + g * 16 + row) * 8; }
+
+// q_pack [slot, H, L, DP], k_pack [slot, H, DP, L], p_pack [slot, H, 2, L, L] (the two halves of P, [t][s]), each in fragments,
+// gate_pack [slot, H, 3, L]: F, J, mu (tokens past the request's end: F and mu of its last token, J -inf, q, k and P zero).
 template <int DP>
 __global__ __launch_bounds__(256) void mlstm_pack_kernel(const float* __restrict__ proj, int ld, int k_at, int i_at, int f_at,
                                                          const float* __restrict__ i_bias, const float* __restrict__ f_bias, float cap,
@@ -97,7 +101,7 @@ __global__ __launch_bounds__(256) void mlstm_pack_kernel(const float* __restrict
     const bf16x4 qa = {(bf16)a[0], (bf16)a[1], (bf16)a[2], (bf16)a[3]}, kb = {(bf16)b[0], (bf16)b[1], (bf16)b[2], (bf16)b[3]};
     *(bf16x4*)(qs + t * LD + i) = qa;
     *(bf16x4*)(ks + t * LD + i) = kb;
-    *(bf16x4*)(q_pack + (pack * L + t) * DP + i) = qa;
+    *(bf16x4*)(q_pack + pack * L * DP + fragment(t / 16, DP / 32, i / 32, t % 16, i % 32 / 8) + i % 8) = qa;
   }
   __syncthreads();
 
@@ -108,8 +112,8 @@ __global__ __launch_bounds__(256) void mlstm_pack_kernel(const float* __restrict
 #pragma unroll
     for (int c = 0; c < DP / 32; ++c) qf[c] = *(const bf16x8*)(qs + t * LD + c * 32 + g * 8);
     const float ft = f_sum[t] - mu_of[t];
-    bf16* hi_row = p_pack + (pack * 2 * L + t) * L;
-    bf16* lo_row = hi_row + L * L;
+    bf16* hi_pack = p_pack + pack * 2 * L * L;
+    bf16* lo_pack = hi_pack + L * L;
     for (int b = 0; b <= (wave | 1); ++b) {               // (whole pairs of blocks: what the second product reads at a time)
       floatx4 acc = {0.f, 0.f, 0.f, 0.f};
       if (b <= wave) {
@@ -126,196 +130,203 @@ __global__ __launch_bounds__(256) void mlstm_pack_kernel(const float* __restrict
         split_bf16(p, ph, pl);
         hi[i] = ph, lo[i] = pl;
       }
-      *(bf16x4*)(hi_row + b * 16 + g * 4) = hi;
-      *(bf16x4*)(lo_row + b * 16 + g * 4) = lo;
+      const int s0 = b * 16 + g * 4, at = fragment(wave, 2, s0 / 32, col, s0 % 32 / 8) + s0 % 8;
+      *(bf16x4*)(hi_pack + at) = hi;
+      *(bf16x4*)(lo_pack + at) = lo;
     }
   }
   // k by columns: eight tokens of a dim in one store
   for (int e = tid; e < DP * (L / 8); e += 256) {
-    const int i = e % DP, j = e / DP * 8;
+    const int i = e % 16 + e / 64 / 2 * 16, x = e / 64 % 2, piece = e / 16 % 4, j = x * 32 + piece * 8;      // (in the order of the pack: whole lines)
     bf16x8 v;
 #pragma unroll
-    for (int x = 0; x < 8; ++x) v[x] = ks[(j + x) * LD + i];
-    *(bf16x8*)(k_pack + (pack * DP + i) * L + j) = v;
+    for (int y = 0; y < 8; ++y) v[y] = ks[(j + y) * LD + i];
+    *(bf16x8*)(k_pack + pack * DP * L + fragment(i / 16, 2, x, i % 16, piece)) = v;
   }
 }
 
-// A workgroup of four waves owns C = 16 * CB columns of one head's S (dv values and the normaliser, `columns` in all) for one
-// request.  Per chunk: S goes into LDS as two bfloat16 halves, the columns' values as they are and weighted (two halves); wave w
-// makes the read-outs of tokens 16 w .. 16 w + 15 and updates the rows of S of its DP / 64 blocks of 16.  The operands that only one
-// wave reads (its rows of q, P and k) come straight from the packs, the next chunk's on their way while this one is worked on.
+// A workgroup owns C = 16 * CB columns of one head's S (dv values and the normaliser, `columns` in all) for one request, four waves
+// every 16 columns.  Per chunk: S goes into LDS as two bfloat16 halves, the columns' values as they are and weighted (two halves);
+// the quarter w of a column block's waves makes the read-outs of tokens 16 w .. 16 w + 15 and updates the rows of S of its DP / 64
+// blocks of 16.  The operands that a wave has for itself (its rows of q, P and k) come straight from the packs, the next chunk's on
+// their way while this one is worked on.
 template <int DP, int CB>
-__global__ __launch_bounds__(256, 1) void mlstm_chunks_kernel(const float* __restrict__ proj, int ld, int v_at, const bf16* __restrict__ q_pack,
+__global__ __launch_bounds__(256 * CB, 2) void mlstm_chunks_kernel(const float* __restrict__ proj, int ld, int v_at, const bf16* __restrict__ q_pack,
                                                               const bf16* __restrict__ k_pack, const bf16* __restrict__ p_pack,
                                                               const float* __restrict__ gate_pack, const int* __restrict__ cu,
                                                               const int* __restrict__ slot_ids, float* __restrict__ state, int64_t state_stride,
                                                               int64_t m_offset, int H, int columns, float* __restrict__ raw,
                                                               float* __restrict__ floors, float* __restrict__ maxima) {
   constexpr int C = 16 * CB, ROWS = DP / 16, QK = DP / 32, DB = DP / 64, SLD = DP + 16, VLD = L + 16, FLD = DP + 4;
-  constexpr int TOKENS = C / 4;                            // tokens of one column a thread brings in
+  constexpr int THREADS = 256 * CB, TOKENS = 4;            // ... tokens of one column a thread brings in
   constexpr int HALVES = 2 * C * SLD * 2, PLAIN = C * FLD * 4;
   __shared__ __attribute__((aligned(16))) unsigned char s_room[HALVES > PLAIN ? HALVES : PLAIN];
   __shared__ __attribute__((aligned(16))) bf16 v_t[3][C * VLD];    // the values, the weighted values' first and second halves: [column][token]
-  __shared__ float of_state[L], of_chunk[L];               // what a token's two sums are multiplied by
+  __shared__ __attribute__((aligned(16))) float of_state[L], of_chunk[L];               // what a token's two sums are multiplied by
   bf16* s_hi = (bf16*)s_room;
   bf16* s_lo = s_hi + C * SLD;
   float* s_f32 = (float*)s_room;
   typedef bf16 run_t __attribute__((ext_vector_type(TOKENS)));
-  const int r = blockIdx.x, h = blockIdx.y, c0 = blockIdx.z * C, tid = threadIdx.x, lane = tid % WAVE, wave = tid / WAVE;
-  const int col = lane & 15, g = lane >> 4;
+  const int r = blockIdx.x, h = blockIdx.y, c0 = blockIdx.z * C, tid = threadIdx.x, lane = tid % WAVE;
+  const int wave = tid / WAVE % 4, block = tid / WAVE / 4; // the quarter and the column block of this wave
+  const int col = lane & 15, g = lane >> 4, c = block * 16 + col;
   const int start = cu[r], n = cu[r + 1] - start, chunks = (n + L - 1) / L, slot0 = first_slot(cu, r);
   float* own = state + (int64_t)slot_ids[r] * state_stride;
   float* st = own + (int64_t)h * ROWS * columns * SPLIT;
   float m = own[m_offset + h];
 
   // S from the state row, whose lines run over columns and 16ths of the rows, through LDS into the accumulators' layout
-  for (int e = tid; e < ROWS * C * SPLIT; e += 256) {
-    const int row = e / (C * SPLIT), c = e / SPLIT % C, s = e % SPLIT;
-    s_f32[c * FLD + s * ROWS + row] = c0 + c < columns ? st[((int64_t)row * columns + c0 + c) * SPLIT + s] : 0.f;
+  for (int e = tid; e < ROWS * C * SPLIT; e += THREADS) {
+    const int row = e / (C * SPLIT), cc = e / SPLIT % C, s = e % SPLIT;
+    s_f32[cc * FLD + s * ROWS + row] = c0 + cc < columns ? st[((int64_t)row * columns + c0 + cc) * SPLIT + s] : 0.f;
   }
   __syncthreads();
-  floatx4 S[DB][CB];
+  floatx4 S[DB];
 #pragma unroll
-  for (int b = 0; b < DB; ++b)
-#pragma unroll
-    for (int c = 0; c < CB; ++c) S[b][c] = *(const floatx4*)(s_f32 + (c * 16 + col) * FLD + (wave * DB + b) * 16 + g * 4);
+  for (int b = 0; b < DB; ++b) S[b] = *(const floatx4*)(s_f32 + c * FLD + (wave * DB + b) * 16 + g * 4);
   __syncthreads();
 
   const int vc = tid % C, vt0 = tid / C * TOKENS;          // the column and the first token of the values a thread brings in
   const int values = columns - 1;
-  struct Operands {
-    bf16x8 q[QK], k[DB][2], p[2][2];
-    float v[TOKENS], j[TOKENS];
-    float f, mu, f_last, mu_last;
-  };
-  auto fetch = [&](int chunk, Operands& o) {
-    const int64_t pack = (int64_t)(slot0 + chunk) * H + h;
+  // What a wave has on its way: every operand of the next chunk is asked for as soon as this chunk's has been used (no second set of
+  // registers), without a branch around a load (behind one, every use would have to wait for all loads): past the end, of the
+  // portion or of the values, any number will do and is not used.
+  bf16x8 q[QK], p[2][2], k[DB][2];
+  float v[TOKENS], f, mu, f_last, mu_last;
+  floatx4 j;
+  auto pack_of = [&](int chunk) { return (int64_t)(slot0 + min(chunk, chunks - 1)) * H + h; };
+  auto fetch_values = [&](int chunk) {
+    chunk = min(chunk, chunks - 1);
     const int count = min(L, n - chunk * L);
-    const bf16* q = q_pack + (pack * L + wave * 16 + col) * DP + g * 8;
+    const float* gates = gate_pack + pack_of(chunk) * 3 * L;
+    const float* from = proj + (int64_t)(start + chunk * L) * ld + v_at + (int64_t)h * values + min(c0 + vc, values - 1);
 #pragma unroll
-    for (int c = 0; c < QK; ++c) o.q[c] = *(const bf16x8*)(q + c * 32);
-    const bf16* p = p_pack + (pack * 2 * L + wave * 16 + col) * L + g * 8;
+    for (int x = 0; x < TOKENS; ++x) v[x] = from[(int64_t)min(vt0 + x, count - 1) * ld];
+    j = *(const floatx4*)(gates + L + vt0);
+    f = gates[lane], mu = gates[2 * L + lane];
+    f_last = gates[L - 1], mu_last = gates[3 * L - 1];
+  };
+  auto fetch_q = [&](int chunk) {
+    const bf16* from = q_pack + pack_of(chunk) * L * DP + lane * 8;
 #pragma unroll
-    for (int half = 0; half < 2; ++half) {
-      o.p[half][0] = *(const bf16x8*)(p + half * L * L);
-      if (wave >= 2) o.p[half][1] = *(const bf16x8*)(p + half * L * L + 32);
-    }
+    for (int x = 0; x < QK; ++x) q[x] = *(const bf16x8*)(from + fragment(wave, QK, x, 0, 0));
+  };
+  auto fetch_p = [&](int chunk) {
+    const bf16* from = p_pack + pack_of(chunk) * 2 * L * L + lane * 8;
+#pragma unroll
+    for (int half = 0; half < 2; ++half)
+#pragma unroll
+      for (int x = 0; x < 2; ++x) p[half][x] = *(const bf16x8*)(from + half * L * L + fragment(wave, 2, x, 0, 0));
+  };
+  auto fetch_k = [&](int chunk) {
+    const bf16* from = k_pack + pack_of(chunk) * DP * L + lane * 8;
 #pragma unroll
     for (int b = 0; b < DB; ++b)
 #pragma unroll
-      for (int c = 0; c < 2; ++c) o.k[b][c] = *(const bf16x8*)(k_pack + (pack * DP + (wave * DB + b) * 16 + col) * L + c * 32 + g * 8);
-    const float* gates = gate_pack + pack * 3 * L;
-#pragma unroll
-    for (int x = 0; x < TOKENS; ++x) {
-      const int t = vt0 + x;
-      o.v[x] = t < count && c0 + vc <= values ? 1.f : 0.f;
-      if (t < count && c0 + vc < values) o.v[x] = proj[(int64_t)(start + chunk * L + t) * ld + v_at + (int64_t)h * values + c0 + vc];
-      o.j[x] = gates[L + t];
-    }
-    o.f = gates[lane], o.mu = gates[2 * L + lane];
-    o.f_last = gates[L - 1], o.mu_last = gates[3 * L - 1];
+      for (int x = 0; x < 2; ++x) k[b][x] = *(const bf16x8*)(from + fragment(wave * DB + b, 2, x, 0, 0));
   };
-  Operands now, next;
-  fetch(0, now);
+  fetch_values(0);
+  fetch_q(0);
+  fetch_p(0);
+  fetch_k(0);
   for (int chunk = 0; chunk < chunks; ++chunk) {
     const int count = min(L, n - chunk * L);
-    const float m_last = fmaxf(m + now.f_last, now.mu_last);
-    if (wave == 0) {
-      const float mt = fmaxf(m + now.f, now.mu);
-      of_state[lane] = expf(m + now.f - mt);
-      of_chunk[lane] = expf(now.mu - mt);
-      if (blockIdx.z == 0 && lane < count) floors[(int64_t)(start + chunk * L + lane) * H + h] = expf(-mt);
+    const float m_last = fmaxf(m + f_last, mu_last);
+    float floor_here = 0.f;
+    if (tid < L) {
+      const float mt = fmaxf(m + f, mu);
+      of_state[lane] = expf(m + f - mt);
+      of_chunk[lane] = expf(mu - mt);
+      floor_here = expf(-mt);
     }
     {
       run_t plain, hi, lo;
 #pragma unroll
       for (int x = 0; x < TOKENS; ++x) {
-        const bf16 v = (bf16)now.v[x];
+        const bf16 value = (bf16)(vt0 + x < count && c0 + vc < columns ? (c0 + vc < values ? v[x] : 1.f) : 0.f);
         bf16 wh, wl;
-        split_bf16(expf(now.f_last + now.j[x] - m_last) * (float)v, wh, wl);
-        plain[x] = v, hi[x] = wh, lo[x] = wl;
+        split_bf16(expf(f_last + j[x] - m_last) * (float)value, wh, wl);
+        plain[x] = value, hi[x] = wh, lo[x] = wl;
       }
       *(run_t*)(v_t[0] + vc * VLD + vt0) = plain;
       *(run_t*)(v_t[1] + vc * VLD + vt0) = hi;
       *(run_t*)(v_t[2] + vc * VLD + vt0) = lo;
     }
 #pragma unroll
-    for (int b = 0; b < DB; ++b)
+    for (int b = 0; b < DB; ++b) {
+      bf16x4 hi, lo;
 #pragma unroll
-      for (int c = 0; c < CB; ++c) {
-        bf16x4 hi, lo;
-#pragma unroll
-        for (int i = 0; i < 4; ++i) {
-          bf16 sh, sl;
-          split_bf16(S[b][c][i], sh, sl);
-          hi[i] = sh, lo[i] = sl;
-        }
-        const int at = (c * 16 + col) * SLD + (wave * DB + b) * 16 + g * 4;
-        *(bf16x4*)(s_hi + at) = hi;
-        *(bf16x4*)(s_lo + at) = lo;
+      for (int i = 0; i < 4; ++i) {
+        bf16 sh, sl;
+        split_bf16(S[b][i], sh, sl);
+        hi[i] = sh, lo[i] = sl;
       }
-    __syncthreads();
-    if (chunk + 1 < chunks) fetch(chunk + 1, next);
-    floatx4 past[CB], here[CB];
-#pragma unroll
-    for (int c = 0; c < CB; ++c) past[c] = here[c] = floatx4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-    for (int x = 0; x < QK; ++x)
-#pragma unroll
-      for (int c = 0; c < CB; ++c) {
-        const int at = (c * 16 + col) * SLD + x * 32 + g * 8;
-        past[c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(now.q[x], *(const bf16x8*)(s_hi + at), past[c], 0, 0, 0);
-        past[c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(now.q[x], *(const bf16x8*)(s_lo + at), past[c], 0, 0, 0);
-      }
-#pragma unroll
-    for (int x = 0; x < 2; ++x) {
-      if (x == 1 && wave < 2) break;                       // (tokens of the chunk's first half see nothing of its second)
-#pragma unroll
-      for (int c = 0; c < CB; ++c) {
-        const bf16x8 v = *(const bf16x8*)(v_t[0] + (c * 16 + col) * VLD + x * 32 + g * 8);
-        here[c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(now.p[0][x], v, here[c], 0, 0, 0);
-        here[c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(now.p[1][x], v, here[c], 0, 0, 0);
-      }
+      const int at = c * SLD + (wave * DB + b) * 16 + g * 4;
+      *(bf16x4*)(s_hi + at) = hi;
+      *(bf16x4*)(s_lo + at) = lo;
     }
-    const float decay = expf(m + now.f_last - m_last);
+    __syncthreads();
+    const float decay = expf(m + f_last - m_last);
+    fetch_values(chunk + 1);
+    // (the state's fragments two products' worth ahead, and a sum of its own for each half: no product waits for the LDS or for the
+    // one before it)
+    floatx4 past = {0.f, 0.f, 0.f, 0.f}, past_lo = past, here = past, here_lo = past;
+    bf16x8 part[3][2];
+    auto state_part = [&](int x) {
+      part[x % 3][0] = *(const bf16x8*)(s_hi + c * SLD + x * 32 + g * 8);
+      part[x % 3][1] = *(const bf16x8*)(s_lo + c * SLD + x * 32 + g * 8);
+    };
+    state_part(0);
+    state_part(1);
+    bf16x8 vf[3][2];
 #pragma unroll
-    for (int b = 0; b < DB; ++b)
+    for (int x = 0; x < QK; ++x) {
+      if (x + 2 < QK) {
+        state_part(x + 2);
+      } else {
+        const int y = x - (QK - 2);                        // the values' fragments behind the state's last
 #pragma unroll
-      for (int c = 0; c < CB; ++c) S[b][c] *= decay;
+        for (int n = 0; n < 3; ++n) vf[n][y] = *(const bf16x8*)(v_t[n] + c * VLD + y * 32 + g * 8);
+      }
+      __builtin_amdgcn_sched_barrier(0);
+      past = __builtin_amdgcn_mfma_f32_16x16x32_bf16(q[x], part[x % 3][0], past, 0, 0, 0);
+      past_lo = __builtin_amdgcn_mfma_f32_16x16x32_bf16(q[x], part[x % 3][1], past_lo, 0, 0, 0);
+      __builtin_amdgcn_sched_barrier(0);
+    }
+    fetch_q(chunk + 1);
+#pragma unroll
+    for (int b = 0; b < DB; ++b) S[b] *= decay;
+    here = __builtin_amdgcn_mfma_f32_16x16x32_bf16(p[0][0], vf[0][0], here, 0, 0, 0);
+    here_lo = __builtin_amdgcn_mfma_f32_16x16x32_bf16(p[1][0], vf[0][0], here_lo, 0, 0, 0);
+    if (wave >= 2) {                                       // (tokens of the chunk's first half see nothing of its second)
+      here = __builtin_amdgcn_mfma_f32_16x16x32_bf16(p[0][1], vf[0][1], here, 0, 0, 0);
+      here_lo = __builtin_amdgcn_mfma_f32_16x16x32_bf16(p[1][1], vf[0][1], here_lo, 0, 0, 0);
+    }
 #pragma unroll
     for (int x = 0; x < 2; ++x)
 #pragma unroll
-      for (int c = 0; c < CB; ++c) {
-        const int at = (c * 16 + col) * VLD + x * 32 + g * 8;
-        const bf16x8 hi = *(const bf16x8*)(v_t[1] + at), lo = *(const bf16x8*)(v_t[2] + at);
+      for (int half = 0; half < 2; ++half)
 #pragma unroll
-        for (int b = 0; b < DB; ++b) {
-          S[b][c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(now.k[b][x], hi, S[b][c], 0, 0, 0);
-          S[b][c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(now.k[b][x], lo, S[b][c], 0, 0, 0);
-        }
-      }
+        for (int b = 0; b < DB; ++b) S[b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k[b][x], vf[1 + half][x], S[b], 0, 0, 0);
+    fetch_p(chunk + 1);
+    fetch_k(chunk + 1);
+    const floatx4 from_state = *(const floatx4*)(of_state + wave * 16 + g * 4), from_chunk = *(const floatx4*)(of_chunk + wave * 16 + g * 4);
+    float* row = raw + ((int64_t)(start + chunk * L + wave * 16 + g * 4) * H + h) * columns + c0 + c;
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const int t = wave * 16 + g * 4 + i;
-      const float from_state = of_state[t], from_chunk = of_chunk[t];
-      float* row = raw + ((int64_t)(start + chunk * L + t) * H + h) * columns;
-#pragma unroll
-      for (int c = 0; c < CB; ++c)
-        if (t < count && c0 + c * 16 + col < columns) row[c0 + c * 16 + col] = fmaf(from_state, past[c][i], from_chunk * here[c][i]);
-    }
+    for (int i = 0; i < 4; ++i)
+      if (wave * 16 + g * 4 + i < count && c0 + c < columns)
+        row[(int64_t)i * H * columns] = fmaf(from_state[i], past[i] + past_lo[i], from_chunk[i] * (here[i] + here_lo[i]));
+    if (blockIdx.z == 0 && tid < count) floors[(int64_t)(start + chunk * L + tid) * H + h] = floor_here;
     m = m_last;
-    now = next;
     __syncthreads();
   }
 
 #pragma unroll
-  for (int b = 0; b < DB; ++b)
-#pragma unroll
-    for (int c = 0; c < CB; ++c) *(floatx4*)(s_f32 + (c * 16 + col) * FLD + (wave * DB + b) * 16 + g * 4) = S[b][c];
+  for (int b = 0; b < DB; ++b) *(floatx4*)(s_f32 + c * FLD + (wave * DB + b) * 16 + g * 4) = S[b];
   __syncthreads();
-  for (int e = tid; e < ROWS * C * SPLIT; e += 256) {
-    const int row = e / (C * SPLIT), c = e / SPLIT % C, s = e % SPLIT;
-    if (c0 + c < columns) st[((int64_t)row * columns + c0 + c) * SPLIT + s] = s_f32[c * FLD + s * ROWS + row];
+  for (int e = tid; e < ROWS * C * SPLIT; e += THREADS) {
+    const int row = e / (C * SPLIT), cc = e / SPLIT % C, s = e % SPLIT;
+    if (c0 + cc < columns) st[((int64_t)row * columns + c0 + cc) * SPLIT + s] = s_f32[cc * FLD + s * ROWS + row];
   }
   if (tid == 0 && blockIdx.z == 0) maxima[(int64_t)r * H + h] = m;
 }
@@ -347,7 +358,7 @@ LRS_API int lrs_mlstm_chunks(void* out, const float* proj, int ld, int tokens, i
   const bool wide = (int64_t)requests * H * ((columns + 31) / 32) >= 96;
   const dim3 grid(requests, H, wide ? (columns + 31) / 32 : (columns + 15) / 16);
 #define WALK(DP, CB)                                                                                                                        \
-  mlstm_chunks_kernel<DP, CB><<<grid, 256, 0, s>>>(proj, ld, v_at, (const bf16*)q_pack, (const bf16*)k_pack, (const bf16*)p_pack, gate_pack, \
+  mlstm_chunks_kernel<DP, CB><<<grid, 256 * CB, 0, s>>>(proj, ld, v_at, (const bf16*)q_pack, (const bf16*)k_pack, (const bf16*)p_pack, gate_pack, \
                                                    cu, slot_ids, state, state_stride, m_offset, H, columns, raw, floors, maxima)
 #define RUN(DP)                                                                                                                        \
   do {                                                                                                                                 \

@@ -32,10 +32,10 @@ __global__ __launch_bounds__(256) void qkv_norm_prep_kernel(T* __restrict__ qkv,
                                                             int rot_half, T* __restrict__ k_pages, T* __restrict__ v_pages,
                                                             const int* __restrict__ slots, int page_size, const float* __restrict__ bias,
                                                             QueryTemperature temperature, ValuePath<T> path) {
-  __shared__ float scratch[16];
+  __shared__ float scratch[32];
   const int token = blockIdx.x, tid = threadIdx.x;
   T* row = qkv + (int64_t)token * row_stride;
-  const int qn = nq * d, kn = nkv * d, vn = nkv * dv;
+  const int qn = nq * d, kn = nkv * d;
   float ssq = 0.f, ssk = 0.f;
   for (int e = tid; e < qn; e += 256) {
     const float x = to_float(row[e]) + (bias ? bias[e] : 0.f);
@@ -45,8 +45,7 @@ __global__ __launch_bounds__(256) void qkv_norm_prep_kernel(T* __restrict__ qkv,
     const float x = to_float(row[qn + e]) + (bias ? bias[qn + e] : 0.f);
     ssk = fmaf(x, x, ssk);
   }
-  ssq = block_sum(ssq, scratch);
-  ssk = block_sum(ssk, scratch);
+  block_sum2(ssq, ssk, scratch);
   const float inv_q = (q_weight ? 1.0f / sqrtf(ssq / (float)qn + eps) : 1.f) * temperature_of(temperature, token);
   const float inv_k = k_weight ? 1.0f / sqrtf(ssk / (float)kn + eps) : 1.f;
   const int slot = slots ? slots[token] : -1;
@@ -83,10 +82,7 @@ __global__ __launch_bounds__(256) void qkv_norm_prep_kernel(T* __restrict__ qkv,
     }
   }
   if (slot >= 0 && v_pages) {           // (null: values_in_runs_kernel stores them)
-    for (int e = tid; e < vn; e += 256) {
-      const int kvh = e / dv, i = e % dv;
-      v_pages[((page * nkv + kvh) * dv + i) * page_size + off] = value_on_its_way(path, row[qn + kn + e], qn + kn + e, token, vn, e);
-    }
+    store_values(path, row, qn + kn, token, nkv, dv, v_pages, page, off, page_size, tid, 256);
   }
 }
 
@@ -101,10 +97,10 @@ __global__ __launch_bounds__(256) void qkv_norm_prep_vec_kernel(bf16* __restrict
                                                                 int rot_half, bf16* __restrict__ k_pages, bf16* __restrict__ v_pages,
                                                                 const int* __restrict__ slots, int page_size, const float* __restrict__ bias,
                                                                 QueryTemperature temperature, ValuePath<bf16> path) {
-  __shared__ float scratch[16];
+  __shared__ float scratch[32];
   const int token = blockIdx.x, tid = threadIdx.x;
   bf16* row = qkv + (int64_t)token * row_stride;
-  const int qn = nq * d, kn = nkv * d, vn = nkv * dv;
+  const int qn = nq * d, kn = nkv * d;
   const int rot8 = rot_half / 8, items = (d - rot_half) / 8, total = (nq + nkv) * items;
   bf16x8 lo[PREP_ITEMS], hi[PREP_ITEMS];
   // eight values of a run with their biases added (asked for twice, for the sum of squares and for the write: the same bits)
@@ -114,6 +110,12 @@ __global__ __launch_bounds__(256) void qkv_norm_prep_vec_kernel(bf16* __restrict
 #pragma unroll
     for (int i = 0; i < 8; ++i) out[i] = (float)x[i] + (i < 4 ? b0[i] : b1[i - 4]);
   };
+  const int slot = slots ? slots[token] : -1;
+  const int64_t page = slot >= 0 ? slot / page_size : 0, off = slot >= 0 ? slot % page_size : 0;
+  // (the values need no sum: theirs are on their way while the others' are made)
+  if (slot >= 0 && v_pages) {           // (null: values_in_runs_kernel stores them)
+    store_values(path, row, qn + kn, token, nkv, dv, v_pages, page, off, page_size, tid, 256);
+  }
   float ssq = 0.f, ssk = 0.f;
 #pragma unroll
   for (int n = 0; n < PREP_ITEMS; ++n) {
@@ -139,12 +141,9 @@ __global__ __launch_bounds__(256) void qkv_norm_prep_vec_kernel(bf16* __restrict
       else ssk += ss;
     }
   }
-  ssq = block_sum(ssq, scratch);
-  ssk = block_sum(ssk, scratch);
+  block_sum2(ssq, ssk, scratch);
   const float inv_q = (q_weight ? 1.0f / sqrtf(ssq / (float)qn + eps) : 1.f) * temperature_of(temperature, token);
   const float inv_k = k_weight ? 1.0f / sqrtf(ssk / (float)kn + eps) : 1.f;
-  const int slot = slots ? slots[token] : -1;
-  const int64_t page = slot >= 0 ? slot / page_size : 0, off = slot >= 0 ? slot % page_size : 0;
   const float* cosrow = cosv + (int64_t)token * rot_half;
   const float* sinrow = sinv + (int64_t)token * rot_half;
 #pragma unroll
@@ -192,12 +191,6 @@ __global__ __launch_bounds__(256) void qkv_norm_prep_vec_kernel(bf16* __restrict
 #pragma unroll
       for (int i = 0; i < 8; ++i) only[i] = (bf16)(xl[i] * inv * wa[i / 4][i % 4]);
       *(bf16x8*)(dst + at) = only;
-    }
-  }
-  if (slot >= 0 && v_pages) {           // (null: values_in_runs_kernel stores them)
-    for (int e = tid; e < vn; e += 256) {
-      const int kvh = e / dv, i = e % dv;
-      v_pages[((page * nkv + kvh) * dv + i) * page_size + off] = value_on_its_way(path, row[qn + kn + e], qn + kn + e, token, vn, e);
     }
   }
 }

@@ -30,6 +30,37 @@ __device__ __forceinline__ T value_on_its_way(const ValuePath<T>& path, T raw, i
   return out;
 }
 
+// One token's values into its slot by `threads` threads (this one is `tid`), four at a time: every load of the four is on its way
+// before the first is used.
+template <typename T>
+__device__ __forceinline__ void store_values(const ValuePath<T>& path, const T* __restrict__ row, int v_offset, int64_t token, int nkv, int dv,
+                                             T* __restrict__ v_pages, int64_t page, int64_t off, int page_size, int tid, int threads) {
+  constexpr int AT_ONCE = 4;
+  const int vn = nkv * dv;
+  const float lambda = path.mix ? path.mix[0] : 0.f;
+  for (int e0 = tid; e0 < vn; e0 += threads * AT_ONCE) {
+    T raw[AT_ONCE], first[AT_ONCE];
+    float bias[AT_ONCE];
+#pragma unroll
+    for (int n = 0; n < AT_ONCE; ++n) {
+      const int e = min(e0 + n * threads, vn - 1);
+      raw[n] = row[v_offset + e];
+      bias[n] = path.bias ? path.bias[v_offset + e] : 0.f;
+      first[n] = path.mix ? path.first[token * vn + e] : raw[n];
+    }
+#pragma unroll
+    for (int n = 0; n < AT_ONCE; ++n) {
+      const int e = e0 + n * threads;
+      if (e >= vn) break;
+      float v = to_float(raw[n]) + bias[n];
+      if (path.mix) v = (1.f - lambda) * v + lambda * to_float(first[n]);
+      const T out = from_float<T>(v);
+      if (path.first && !path.mix) path.first[token * vn + e] = out;
+      v_pages[((page * nkv + e / dv) * dv + e % dv) * page_size + off] = out;
+    }
+  }
+}
+
 // The values of 16 consecutive tokens of the step and one kv head into the value pages, for steps of many tokens: tokens that
 // follow each other inside a page lie side by side there, so a thread gathers one dim of 16 / sizeof(T) such tokens
 // (neighbouring lanes read neighbouring dims of one token) and writes one 16-byte store; where a run is broken (a page's edge,
