@@ -633,6 +633,7 @@ struct LogGates {
   float input, forget;
 };
 __device__ __forceinline__ LogGates log_gates(float i_in, float f_in, float cap) {
+#pragma clang fp contract(off)      // the products are rounded before anything is added to them, the same in every kernel that inlines this
   const float y = cap * tanhf(f_in / cap);
   return {cap * tanhf(i_in / cap), fminf(y, 0.f) - log1pf(expf(-fabsf(y)))};
 }

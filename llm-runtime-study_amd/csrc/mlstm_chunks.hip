@@ -158,7 +158,7 @@ __global__ __launch_bounds__(256 * CB, 2) void mlstm_chunks_kernel(const float* 
                                                               int64_t m_offset, int H, int columns, float* __restrict__ raw,
                                                               float* __restrict__ floors, float* __restrict__ maxima) {
   constexpr int C = 16 * CB, ROWS = DP / 16, QK = DP / 32, DB = DP / 64, SLD = DP + 16, VLD = L + 16, FLD = DP + 4;
-  constexpr int THREADS = 256 * CB, TOKENS = 4;            // ... tokens of one column a thread brings in
+  constexpr int THREADS = 256 * CB, TOKENS = 4;            // a thread brings in the values of so many tokens of one column
   constexpr int HALVES = 2 * C * SLD * 2, PLAIN = C * FLD * 4;
   __shared__ __attribute__((aligned(16))) unsigned char s_room[HALVES > PLAIN ? HALVES : PLAIN];
   __shared__ __attribute__((aligned(16))) bf16 v_t[3][C * VLD];    // the values, the weighted values' first and second halves: [column][token]

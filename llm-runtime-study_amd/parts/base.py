@@ -240,16 +240,18 @@ class Part:
         """Stack `matrix` [rows, in] behind the part's first product when the part is bound next."""
         self._carried = matrix
 
-    def stack_rows(self, matrices: list, dtype: torch.dtype) -> torch.Tensor:
+    def stack_rows(self, matrices: list, dtype: torch.dtype, pad_alone: bool = True) -> torch.Tensor:
         """`matrices` one under the other in `dtype`, zero rows up to a multiple of 16 (whole groups of 16 output columns suit every
-        product kernel), then the carried matrix and zero rows likewise."""
+        product kernel; pad_alone=False: only where something is carried), then the carried matrix and zero rows likewise."""
         width = matrices[0].shape[1]
 
         def padded(parts):
             pad = -sum(m.shape[0] for m in parts) % 16
             return parts + ([parts[0].new_zeros(pad, width)] if pad else [])
 
-        parts = padded([m.to(dtype) for m in matrices])
+        parts = [m.to(dtype) for m in matrices]
+        if pad_alone or self._carried is not None:
+            parts = padded(parts)
         self._carried_rows = 0
         if self._carried is not None:
             self._carried_at, carried = sum(m.shape[0] for m in parts), self._carried.to(dtype)

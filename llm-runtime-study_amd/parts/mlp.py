@@ -108,7 +108,7 @@ class DenseMLP(Part):
 
     def bind(self, weights, dtype):
         up = weights["up_proj.weight"]
-        self.up = up.to(dtype).contiguous() if self._carried is None else self.stack_rows([up], dtype)
+        self.up = self.stack_rows([up], dtype, pad_alone=False)
         if self.activation == "xielu":
             p, q = torch.nn.functional.softplus(weights["act"].double())
             self.numbers = torch.stack((p, 0.5 + q)).float().contiguous()

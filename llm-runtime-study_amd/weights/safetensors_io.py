@@ -153,7 +153,7 @@ def write_safetensors(path, tensors: dict[str, torch.Tensor], metadata: dict | N
         t = tensors[name].detach().cpu().contiguous()
         if t.dtype not in _NAMES:
             raise CheckpointError(f"cannot store tensor {name!r} of dtype {t.dtype}")
-        raw = t.view(torch.uint8).numpy().tobytes() if t.numel() else b""
+        raw = t.reshape(-1).view(torch.uint8).numpy().tobytes() if t.numel() else b""
         header[name] = {"dtype": _NAMES[t.dtype], "shape": list(t.shape), "data_offsets": [offset, offset + len(raw)]}
         offset += len(raw)
         blobs.append(raw)

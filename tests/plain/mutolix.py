@@ -84,13 +84,14 @@ def attention(u: torch.Tensor, w: dict, m: dict, eps: float, first_values: list 
     n, heads, groups, d, e = u.shape[0], m["heads"], m["kv_heads"], m["dim"], m["vdim"]
     q = rms_norm(u @ w["q"].T + w["q.b"], w["q.norm"], eps).view(n, heads, d)
     k = rms_norm(u @ w["k"].T + w["k.b"], w["k.norm"], eps).view(n, groups, d)
-    v = (u @ w["v"].T + w["v.b"]).view(n, groups, e)
+    v = u @ w["v"].T + w["v.b"]                                          # [n, groups * e]: mixed value by value
     q = q * temperature(torch.arange(n), m.get("q_temp"), u.dtype)[:, None, None]
     if m.get("v_mix"):
         if first_values:
             v = (1.0 - w["vmix"]) * v + w["vmix"] * first_values[0]
         else:
             first_values.append(v)
+    v = v.view(n, groups, e)
     out = torch.zeros(n, heads, e, dtype=u.dtype)
     for h in range(heads):
         g = h // (heads // groups)

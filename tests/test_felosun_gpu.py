@@ -23,7 +23,7 @@ F64 = torch.float64
 
 def bf16_values(*shape, scale=1.0, seed=0):
     g = torch.Generator().manual_seed(seed)
-    return (scale * torch.randn(*shape, generator=g)).to(torch.bfloat16).double()
+    return (scale * torch.randn(shape, generator=g)).to(torch.bfloat16).double()
 
 
 def short(name: str) -> str:
