@@ -274,15 +274,19 @@ __device__ __forceinline__ void prepare_head(bf16x8 (&r)[D / 32], const bf16* __
 // PREP: q holds the raw rows of the q/k/v product; the kernel prepares q itself, and the wave that
 // meets the token's own position prepares the new key, takes it and the new value in place of what
 // the pages hold there, and writes both into the pages (see DecodePrep).
-template <int D, bool PREP, int WAVES, bool AHEAD>
+// MORE: values narrower than keys and a bias by distance (dv and distance are looked at); instances of their own, so that the
+// others are spared the checks.
+template <int D, bool PREP, int WAVES, bool AHEAD, bool MORE>
 __global__ __launch_bounds__(WAVES * 64) void attention_decode_bf16_kernel(
     bf16* __restrict__ out, int out_stride, float* __restrict__ part_o, float* __restrict__ part_ml,
     const bf16* __restrict__ q, int q_stride, bf16* __restrict__ k_pages,
     bf16* __restrict__ v_pages, const int* __restrict__ block_table, int table_stride,
     const int* __restrict__ token_request, const int* __restrict__ positions, int nq, int nkv,
     int page_size, float scale, int window, int splits, int slots, DecodePrep prep, const float* __restrict__ sinks,
-    float softcap, const bf16* __restrict__ gates, int gate_stride, int dv, const float* __restrict__ distance) {
+    float softcap, const bf16* __restrict__ gates, int gate_stride, int dv_given, const float* __restrict__ distance_given) {
   constexpr int DS = D / 32, DB = D / 16, THREADS = WAVES * 64;
+  const int dv = MORE ? dv_given : D;
+  const float* __restrict__ distance = MORE ? distance_given : nullptr;
   __shared__ float sm_m[WAVES][16], sm_l[WAVES][16];
   __shared__ float sm_o[WAVES][D][16];
   const int tid = threadIdx.x, lane = tid % WAVE, wave = tid / WAVE;
@@ -735,6 +739,7 @@ LRS_API int lrs_attention_decode(void* out, int out_stride, float* part_o, float
                                  const void* q_weight, const void* k_weight, int w_dtype, float eps,
                                  const float* cosv, const float* sinv, int kv_columns, const float* sinks, float softcap,
                                  const void* gates, int gate_stride, int dv, const float* distance, void* stream) {
+  LRS_REQUIRE(!distance || !prepare, "attention_decode: a bias by distance needs prepared heads");
   LRS_REQUIRE(dv > 0 && dv % 16 == 0 && dv <= d && (dv == d || !prepare),
               "attention_decode: values of %d dims beside keys of %d are not served (a multiple of 16, at most the keys', heads that come prepared)", dv, d);
   LRS_REQUIRE(tokens > 0 && nq > 0 && nkv > 0 && nq % nkv == 0, "attention_decode: bad sizes tokens=%d nq=%d nkv=%d", tokens, nq, nkv);
@@ -771,16 +776,17 @@ LRS_API int lrs_attention_decode(void* out, int out_stride, float* part_o, float
   (bf16*)out, out_stride, part_o, part_ml, (const bf16*)q, q_stride, (bf16*)k_pages, (bf16*)v_pages, block_table, \
       table_stride, token_request, positions, nq, nkv, page_size, scale, window, splits, slots, prep, slots == 1 ? sinks : nullptr, softcap, \
       slots == 1 ? (const bf16*)gates : nullptr, gate_stride, dv, distance
-#define LAUNCH_PREP(D, PREP)                                                                                 \
+#define LAUNCH_PREP(D, PREP, MORE)                                                                           \
   do {                                                                                                       \
-    if (form == 2 && D <= 128) attention_decode_bf16_kernel<D, PREP, 8, (D <= 128)><<<grid, 512, table_lds, s>>>(ARGS); \
-    else if (form == 1 && D <= 128) attention_decode_bf16_kernel<D, PREP, 4, (D <= 128)><<<grid, 256, table_lds, s>>>(ARGS); \
-    else attention_decode_bf16_kernel<D, PREP, 4, false><<<grid, 256, table_lds, s>>>(ARGS);                  \
+    if (form == 2 && D <= 128) attention_decode_bf16_kernel<D, PREP, 8, (D <= 128), MORE><<<grid, 512, table_lds, s>>>(ARGS); \
+    else if (form == 1 && D <= 128) attention_decode_bf16_kernel<D, PREP, 4, (D <= 128), MORE><<<grid, 256, table_lds, s>>>(ARGS); \
+    else attention_decode_bf16_kernel<D, PREP, 4, false, MORE><<<grid, 256, table_lds, s>>>(ARGS);             \
   } while (0)
 #define LAUNCH(D)                        \
   do {                                   \
-    if (prepare) LAUNCH_PREP(D, true);   \
-    else LAUNCH_PREP(D, false);          \
+    if (prepare) LAUNCH_PREP(D, true, false);                       \
+    else if (dv != d || distance) LAUNCH_PREP(D, false, true);      \
+    else LAUNCH_PREP(D, false, false);                              \
   } while (0)
   switch (d) {
     case 32: LAUNCH(32); break;

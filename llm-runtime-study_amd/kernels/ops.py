@@ -1243,6 +1243,7 @@ def attention_decode(out: torch.Tensor, q: torch.Tensor, k_pages: torch.Tensor, 
         _need(part_ml is not None and part_ml.dtype == torch.float32 and part_ml.is_contiguous() and part_ml.numel() >= tokens * nq * slots * 2, "attention_decode: part_ml too small")
     fused = [0, None, None, 0, 0.0, None, None, 0]
     if prepare is not None:
+        _need(distance is None, "attention_decode: a bias by distance needs prepared heads")
         _need(dv == d, "attention_decode: heads whose values are narrower than their keys must come prepared")
         _need(decode_prepare_supported(d, prepare.cos is not None), f"attention_decode: cannot rotate heads of {d} dims itself")
         _need((prepare.q_weight is None) == (prepare.k_weight is None), "attention_decode: q and k norm weights must come together")
