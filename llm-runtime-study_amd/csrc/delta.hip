@@ -776,6 +776,23 @@ __global__ __launch_bounds__(256) void mlstm_read_kernel(const float* __restrict
 
 }  // namespace
 
+// The recurrence of requests that bring one token each: token r is request r's.
+void lrs_mlstm_singles(const float* proj, int ld, int requests, const int* slot_ids, float* state, int64_t state_stride, int H, int d, int dv,
+                       const float* i_bias, const float* f_bias, float cap, float* raw, float* floors, float* maxima, hipStream_t s) {
+  const int rows = lrs_delta_state_rows(d), columns = dv + 1;
+  const ScanRows at{ld, 0, H * d, 2 * H * d};
+  const int i_at = 2 * H * d + 2 * H * dv, f_at = i_at + H;
+  const int64_t m_offset = (int64_t)H * rows * SPLIT * columns;
+  const dim3 grid(requests, H, (columns + COLUMNS - 1) / COLUMNS);
+#define SINGLE(ROWS)                                                                                                                   \
+  mlstm_single_kernel<ROWS><<<grid, 256, 0, s>>>(proj, at, i_at, f_at, slot_ids, state, state_stride, m_offset, H, d, columns, i_bias, \
+                                                 f_bias, cap, raw, floors, maxima)
+  if (rows == 4) SINGLE(4);
+  else if (rows == 8) SINGLE(8);
+  else SINGLE(16);
+#undef SINGLE
+}
+
 int lrs_mlstm_read_out(void* out, int out_dtype, const float* raw, const float* floors, const float* proj, int ld, int g_at, const float* norm_w,
                        float q_factor, float eps, int tokens, int requests, int H, int dv, const float* maxima, const int* token_request, const int* cu,
                        const int* slot_ids, float* state, int64_t state_stride, int64_t m_offset, hipStream_t s) {
@@ -813,13 +830,7 @@ LRS_API int lrs_mlstm(void* out, int out_dtype, const float* proj, int ld, int t
   const bool single = tokens == requests;
   float* maxima = single ? gates : nullptr;      // (the factors of single tokens never leave their kernel)
   if (single) {
-#define SINGLE(ROWS)                                                                                                                    \
-  mlstm_single_kernel<ROWS><<<sgrid, 256, 0, s>>>(proj, at, i_at, f_at, slot_ids, state, state_stride, m_offset, H, d, columns, i_bias, \
-                                                  f_bias, cap, raw, floors, maxima)
-    if (rows == 4) SINGLE(4);
-    else if (rows == 8) SINGLE(8);
-    else SINGLE(16);
-#undef SINGLE
+    lrs_mlstm_singles(proj, ld, requests, slot_ids, state, state_stride, H, d, dv, i_bias, f_bias, cap, raw, floors, maxima, s);
   } else {
     mlstm_gates_kernel<<<dim3(requests, H), WAVE, 0, s>>>(proj, ld, i_at, f_at, cu, slot_ids, state, state_stride, m_offset, H, i_bias, f_bias,
                                                           cap, gates, floors);

@@ -17,6 +17,8 @@
 int lrs_mlstm_read_out(void* out, int out_dtype, const float* raw, const float* floors, const float* proj, int ld, int g_at, const float* norm_w,
                        float q_factor, float eps, int tokens, int requests, int H, int dv, const float* maxima, const int* token_request, const int* cu,
                        const int* slot_ids, float* state, int64_t state_stride, int64_t m_offset, hipStream_t s);
+void lrs_mlstm_singles(const float* proj, int ld, int requests, const int* slot_ids, float* state, int64_t state_stride, int H, int d, int dv,
+                       const float* i_bias, const float* f_bias, float cap, float* raw, float* floors, float* maxima, hipStream_t s);
 extern "C" int lrs_delta_state_rows(int d);
 
 namespace {
@@ -338,13 +340,15 @@ LRS_API int lrs_mlstm_slots(int tokens, int requests) { return tokens / L + requ
 
 // lrs_mlstm for steps with long portions in bfloat16 (out is bfloat16): the same arguments, with maxima [requests, H] float32 for its
 // `gates`, and the packs: q_pack and k_pack bfloat16 [slots, H, 64 * (16 * state rows)], p_pack bfloat16 [slots, H, 2 * 64 * 64],
-// gate_pack float32 [slots, H, 3 * 64], slots = lrs_mlstm_slots(tokens, requests).
+// gate_pack float32 [slots, H, 3 * 64], slots = lrs_mlstm_slots(tokens, requests).  singles: that many requests at the head of the step
+// bring one token each (their tokens are its first); they go to the kernel for single tokens, which does not walk a chunk for one.
 LRS_API int lrs_mlstm_chunks(void* out, const float* proj, int ld, int tokens, int requests, const int* token_request, const int* cu,
                              const int* slot_ids, float* state, int64_t state_stride, int H, int d, int dv, const float* i_bias,
                              const float* f_bias, float cap, const float* norm_w, float eps, float* maxima, float* floors, float* raw,
-                             void* q_pack, void* k_pack, void* p_pack, float* gate_pack, void* stream) {
+                             void* q_pack, void* k_pack, void* p_pack, float* gate_pack, int singles, void* stream) {
   LRS_REQUIRE(tokens > 0 && requests > 0 && requests <= tokens, "mlstm_chunks: bad sizes tokens=%d requests=%d", tokens, requests);
   LRS_REQUIRE(H > 0 && d > 0 && dv > 0 && d <= 256, "mlstm_chunks: bad sizes H=%d d=%d dv=%d (keys of up to 256 values)", H, d, dv);
+  LRS_REQUIRE(singles >= 0 && singles < requests, "mlstm_chunks: %d single tokens leave no portion among %d requests", singles, requests);
   LRS_REQUIRE(cap > 0.f && eps > 0.f, "mlstm_chunks: the gates' cap and eps must be positive");
   const int rows = lrs_delta_state_rows(d), columns = dv + 1;
   const int k_at = H * d, v_at = 2 * H * d, g_at = v_at + H * dv, i_at = g_at + H * dv, f_at = i_at + H;
@@ -353,16 +357,23 @@ LRS_API int lrs_mlstm_chunks(void* out, const float* proj, int ld, int tokens, i
   LRS_REQUIRE(state_stride >= m_offset + H, "mlstm_chunks: a state row of %lld floats is too short", (long long)state_stride);
   LRS_REQUIRE((((uintptr_t)proj | (uintptr_t)q_pack | (uintptr_t)k_pack | (uintptr_t)p_pack) % 16) == 0, "mlstm_chunks: rows and packs must be 16 bytes aligned");
   hipStream_t s = (hipStream_t)stream;
-  const dim3 pgrid(lrs_mlstm_slots(tokens, requests), H);
+  // what follows sees the requests behind the single ones (token numbers stay those of the step)
+  if (singles > 0)
+    lrs_mlstm_singles(proj, ld, singles, slot_ids, state, state_stride, H, d, dv, i_bias, f_bias, cap, raw, floors, maxima, s);
+  const int* rest_cu = cu + singles;
+  const int* rest_slots = slot_ids + singles;
+  float* rest_maxima = maxima + (int64_t)singles * H;
+  const int rest = requests - singles;
+  const dim3 pgrid(lrs_mlstm_slots(tokens, rest), H);
   // 32 columns a workgroup, or 16 where that leaves half of the chip idle
-  const bool wide = (int64_t)requests * H * ((columns + 31) / 32) >= 96;
-  const dim3 grid(requests, H, wide ? (columns + 31) / 32 : (columns + 15) / 16);
+  const bool wide = (int64_t)rest * H * ((columns + 31) / 32) >= 96;
+  const dim3 grid(rest, H, wide ? (columns + 31) / 32 : (columns + 15) / 16);
 #define WALK(DP, CB)                                                                                                                        \
   mlstm_chunks_kernel<DP, CB><<<grid, 256 * CB, 0, s>>>(proj, ld, v_at, (const bf16*)q_pack, (const bf16*)k_pack, (const bf16*)p_pack, gate_pack, \
-                                                   cu, slot_ids, state, state_stride, m_offset, H, columns, raw, floors, maxima)
+                                                   rest_cu, rest_slots, state, state_stride, m_offset, H, columns, raw, floors, rest_maxima)
 #define RUN(DP)                                                                                                                        \
   do {                                                                                                                                 \
-    mlstm_pack_kernel<DP><<<pgrid, 256, 0, s>>>(proj, ld, k_at, i_at, f_at, i_bias, f_bias, cap, cu, requests, H, d, (bf16*)q_pack,     \
+    mlstm_pack_kernel<DP><<<pgrid, 256, 0, s>>>(proj, ld, k_at, i_at, f_at, i_bias, f_bias, cap, rest_cu, rest, H, d, (bf16*)q_pack,     \
                                                 (bf16*)k_pack, (bf16*)p_pack, gate_pack);                                              \
     if (wide) WALK(DP, 2);                                                                                                             \
     else WALK(DP, 1);                                                                                                                  \

@@ -135,7 +135,7 @@ _SIGNATURES = {
     "lrs_mlstm_slots": (c_int, [c_int, c_int]),
     "lrs_mlstm_chunks": (c_int, [c_void_p, c_void_p, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_int64, c_int, c_int, c_int,
                                  c_void_p, c_void_p, c_float, c_void_p, c_float, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
-                                 c_void_p, c_void_p]),
+                                 c_void_p, c_int, c_void_p]),
     "lrs_sigmoid_gate": (c_int, [c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p]),
     "lrs_rotate_unit_prep": (c_int, [c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_void_p, c_void_p, c_int, c_int,
                                      c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p]),
@@ -1574,10 +1574,13 @@ def mlstm_pack_sizes(tokens: int, requests: int, heads: int, dim: int) -> tuple:
 
 def mlstm_chunks(out: torch.Tensor, proj: torch.Tensor, state: torch.Tensor, token_request: torch.Tensor, cu_seqlens: torch.Tensor,
                  slot_ids: torch.Tensor, requests: int, heads: int, dim: int, vdim: int, i_bias: torch.Tensor, f_bias: torch.Tensor, cap: float,
-                 norm_weight: torch.Tensor, eps: float, maxima: torch.Tensor, floors: torch.Tensor, raw: torch.Tensor, packs: tuple) -> None:
+                 norm_weight: torch.Tensor, eps: float, maxima: torch.Tensor, floors: torch.Tensor, raw: torch.Tensor, packs: tuple,
+                 singles: int = 0) -> None:
     """mlstm() for steps with long portions in bfloat16: chunks of 64 tokens on the matrix cores (the state in float32).  maxima
-    float32 [requests, heads] scratch, packs: four buffers of mlstm_pack_sizes()."""
+    float32 [requests, heads] scratch, packs: four buffers of mlstm_pack_sizes().  singles: so many requests at the head of the step
+    bring one token each and are served as single tokens."""
     tokens = _mlstm_arguments("mlstm_chunks", out, proj, state, cu_seqlens, slot_ids, requests, heads, dim, vdim, i_bias, f_bias, norm_weight, floors, raw)
+    _need(0 <= singles < requests, f"mlstm_chunks: {singles} single tokens leave no portion among {requests} requests")
     _need(out.dtype == torch.bfloat16, "mlstm_chunks: serves bfloat16 runs only")
     _need(token_request.dtype == torch.int32 and token_request.numel() >= tokens and token_request.is_contiguous(), "mlstm_chunks: token_request must be int32 [T]")
     _need(maxima.dtype == torch.float32 and maxima.is_contiguous() and maxima.numel() >= requests * heads, "mlstm_chunks: maxima scratch too small")
@@ -1587,7 +1590,7 @@ def mlstm_chunks(out: torch.Tensor, proj: torch.Tensor, state: torch.Tensor, tok
     _launch("lrs_mlstm_chunks", _dev(out, "out"), _dev(proj, "proj"), _rows(proj, "proj"), tokens, requests, _dev(token_request, "token_request"),
             _dev(cu_seqlens, "cu_seqlens"), _dev(slot_ids, "slot_ids"), _dev(state, "state"), state.stride(0), heads, dim, vdim,
             _dev(i_bias, "i_bias"), _dev(f_bias, "f_bias"), cap, _dev(norm_weight, "norm_weight"), eps, _dev(maxima, "maxima"),
-            _dev(floors, "floors"), _dev(raw, "raw"), *(_dev(t, "pack") for t in packs), _stream())
+            _dev(floors, "floors"), _dev(raw, "raw"), *(_dev(t, "pack") for t in packs), singles, _stream())
 
 
 # ------------------------------------------------------------------- routed experts

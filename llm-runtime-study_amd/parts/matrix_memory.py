@@ -102,7 +102,7 @@ class MatrixMemory(Part):
                           for number, size in enumerate(ops.mlstm_pack_sizes(t, ctx.R, heads, self.head_dim)))
             maxima = ctx.scratch("mlstm_maxima", (ctx.R, heads), torch.float32)
             ops.mlstm_chunks(out, proj, cache.state, ctx.token_request, ctx.cu_seqlens_q, ctx.slot_ids, ctx.R, heads, self.head_dim, self.value_dim,
-                             self.i_bias, self.f_bias, self.gate_cap, self.norm, self.norm_eps, maxima, floors, raw, packs)
+                             self.i_bias, self.f_bias, self.gate_cap, self.norm, self.norm_eps, maxima, floors, raw, packs, ctx.single_rows)
         else:
             gates = ctx.scratch("mlstm_gates", (t, 2 * heads), torch.float32)
             ops.mlstm(out, proj, cache.state, ctx.cu_seqlens_q, ctx.slot_ids, ctx.R, heads, self.head_dim, self.value_dim, self.i_bias, self.f_bias,

@@ -104,7 +104,8 @@ def test_chunked_form_against_the_scan_on_the_same_numbers():
     from llm_runtime_study_amd.kernels import ops
 
     g = torch.Generator().manual_seed(1)
-    for heads, dim, vdim, lengths in ((3, 24, 40, (130, 1, 64, 65)), (2, 256, 70, (200, 3)), (10, 128, 96, (64, 128, 5, 1, 63)), (1, 100, 17, (1,) * 70 + (300,))):
+    for heads, dim, vdim, lengths, singles in ((3, 24, 40, (130, 1, 64, 65), 0), (2, 256, 70, (200, 3), 0), (10, 128, 96, (64, 128, 5, 1, 63), 0),
+                                               (1, 100, 17, (1,) * 70 + (300,), 0), (1, 100, 17, (1,) * 70 + (300, 1, 2), 70), (4, 64, 50, (1, 1, 1, 90), 2)):
         tokens, requests = sum(lengths), len(lengths)
         columns = 2 * heads * (dim + vdim + 1)
         proj = torch.randn(tokens, columns + 3, generator=g).to(torch.bfloat16).float().cuda()
@@ -124,7 +125,7 @@ def test_chunked_form_against_the_scan_on_the_same_numbers():
                     packs = tuple(torch.empty(n, dtype=torch.float32 if k == 3 else torch.bfloat16, device="cuda")
                                   for k, n in enumerate(ops.mlstm_pack_sizes(tokens, requests, heads, dim)))
                     ops.mlstm_chunks(out, proj, state, of, cu, slots, requests, heads, dim, vdim, i_bias, f_bias, 12.0, norm, 1e-5,
-                                     torch.empty(requests * heads, device="cuda"), floors, raw, packs)
+                                     torch.empty(requests * heads, device="cuda"), floors, raw, packs, singles)
                 else:
                     ops.mlstm(out, proj, state, cu, slots, requests, heads, dim, vdim, i_bias, f_bias, 12.0, norm, 1e-5,
                               torch.empty(tokens * 2 * heads, device="cuda"), floors, raw)
