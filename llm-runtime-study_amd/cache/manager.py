@@ -2,7 +2,7 @@
 fixed-size per-request state.
 
 What each schedule entry of the model keeps between steps is declared by its mixer:
-  PagedKVNeed(nkv, d, window, dtype, value_dim)  keys and values of every position, or of a sliding window, kept in `dtype`
+  PagedKVNeed(nkv, d, window, dtype, value_dim, chunk=)  keys and values of every position, of a sliding window or of the chunk a sequence is in, kept in `dtype`
                                (None: the run's activation dtype); value_dim: rows of a value page if not d, 0: key pages alone;
   StateNeed(shape, dtype)      a state of fixed size;
   BothNeeds(paged, state)      pages and a state (two mixers side by side in one layer);
@@ -14,8 +14,8 @@ entry (values are kept transposed inside a page, so that the keys of one value c
 contiguous, which is what the matrix-core kernels read; a page id addresses the same page
 in every entry of the group; the extra last page absorbs the writes of padding rows),
 and one block table per request.  Pages are taken when a request grows into them and given
-back when the request ends, is rolled back, or (windowed groups) when every position in
-the page has left the window of all future queries.
+back when the request ends, is rolled back, or (groups with a window or chunks) when every position in
+the page has left the window of all future queries, or lies in a chunk that they are past.
 
 The block tables live on the device for good: one int32 array [groups, max_requests + 1, max_blocks] (row = the
 request's slot; the last row, the trash row, points at the trash page), a copy of the host's.  Whatever changes an
@@ -225,12 +225,12 @@ class CacheManager:
     def pages_for(self, group: int, tokens: int, max_step_tokens: int | None = None) -> int:
         """Pages a request of `tokens` positions can hold at once in `group`."""
         blocks = -(-tokens // self.page_size)
-        window = self.groups[group].need.window
-        if window is None:
+        span = self.groups[group].need.span
+        if span is None:
             return blocks
         step = tokens if max_step_tokens is None else max_step_tokens
         kept = -(-self.groups[group].need.keep_first // self.page_size)
-        return min(blocks, -(-window // self.page_size) + -(-step // self.page_size) + 2 + kept)
+        return min(blocks, -(-span // self.page_size) + -(-step // self.page_size) + 2 + kept)
 
     # -------------------------------------------------------------- admission
     def can_admit(self, tokens: int, max_step_tokens: int | None = None) -> bool:
@@ -312,15 +312,14 @@ class CacheManager:
         request.length = length
 
     def trim(self, request: RequestCache) -> int:
-        """Give back pages whose every position is outside the window of all future queries."""
+        """Give back pages whose every position is outside the window, or before the chunk, of all future queries."""
         self._check_live(request)
         freed = 0
         for index, group in enumerate(self.groups):
-            window = group.need.window
-            if window is None:
+            if group.need.span is None:
                 continue
-            # the next query sits at position `length` and sees keys j > length - window
-            dead_blocks = max(0, (request.length - window + 1) // self.page_size)
+            # the next query sits at position `length`
+            dead_blocks = group.need.first_needed(request.length) // self.page_size
             table = request.tables[index]
             dead_blocks = min(dead_blocks, len(table))
             # the pages of the first keep_first positions stay: those keys are seen for good

@@ -77,12 +77,14 @@ def _load_builtin() -> None:
     from ..models.mutolix import build_spec as build_mutolix
     from ..models.napizen import build_spec as build_napizen
     from ..models.nobodra import build_spec as build_nobodra
+    from ..models.tamilix import build_spec as build_tamilix
     from .felosun import FelosunConfig
     from .kaposun import KaposunConfig
     from .mutolix import MutolixConfig
     from .napizen import NapizenConfig
     from .nobodra import NobodraConfig
     from .qwen3 import Qwen3Config
+    from .tamilix import TamilixConfig
 
     if Qwen3Config.ARCHITECTURE not in _ARCHITECTURES:
         register_architecture(Qwen3Config.ARCHITECTURE, Qwen3Config, build_spec, chat_template=format_qwen3_chat)
@@ -96,6 +98,8 @@ def _load_builtin() -> None:
         register_architecture(FelosunConfig.ARCHITECTURE, FelosunConfig, build_felosun)      # token ids only
     if MutolixConfig.ARCHITECTURE not in _ARCHITECTURES:
         register_architecture(MutolixConfig.ARCHITECTURE, MutolixConfig, build_mutolix)      # token ids only
+    if TamilixConfig.ARCHITECTURE not in _ARCHITECTURES:
+        register_architecture(TamilixConfig.ARCHITECTURE, TamilixConfig, build_tamilix)      # token ids only
     import importlib
     import os
 

@@ -1,6 +1,7 @@
 // Causal attention over the paged cache for a ragged batch: every query token attends to
 // the cached keys of its own request at positions lo..p, p being the token's absolute
-// position and lo = max(0, p - window + 1) when a window is given.  Keys and values of this
+// position and lo = 0, max(0, p - window + 1) with a sliding window, or the start of p's chunk
+// (first_seen in common.h: `window` 0, positive or negative).  Keys and values of this
 // step's tokens are already in the cache when these kernels run.
 //
 // Key pages are [page, kv_head, slot, dim], value pages [page, kv_head, dim, slot] (transposed
@@ -42,14 +43,22 @@ __device__ __forceinline__ float with_sink(float sink2, float top, float& total)
 }
 constexpr float LOG2E = 1.4426950408889634f;
 
-// A bias by distance: a score of query head h loses rate_h * ln(1 + reach_h * (i - j)), i the query's position, j the key's.
-// `distance` holds the rates of all nq heads, then their reaches (null: no bias).  In the bfloat16 kernels the logarithm is the
-// hardware's (base 2, a unit in the last place), and the distance from a query to the first key of a lane's four (or eight) is
-// taken in whole positions before it meets the reach, so that a near key's distance is exact however far on the sequence is.
+// A bias by distance, i the query's position, j the key's, in one of two forms:
+//   DISTANCE_LOG     a score of query head h loses rate_h * ln(1 + reach_h * (i - j)); `distance` holds the rates of all nq heads,
+//                    then their reaches;
+//   DISTANCE_LINEAR  it loses rate_h * (i - j); `distance` holds the rates.
+// (distance null: no bias.)  In the bfloat16 kernels the logarithm is the hardware's (base 2, a unit in the last place), and the
+// distance from a query to the first key of a lane's four (or eight) is taken in whole positions before it meets the reach (or the
+// rate), so that a near key's distance is exact however far on the sequence is.
+enum { DISTANCE_LOG = 0, DISTANCE_LINEAR = 1 };
 __device__ __forceinline__ float distance_loss(float rate2, float reach, float distance) {       // rate2: for base-2 logarithms
   return rate2 * __builtin_amdgcn_logf(fmaf(reach, distance, 1.f));
 }
 constexpr float LN2 = 0.6931471805599453f;
+// Either form, in the base-2 units the scores have where it is taken off.
+__device__ __forceinline__ float distance_loss_of(const float* __restrict__ distance, int form, int nq, int head, float behind) {
+  return form == DISTANCE_LINEAR ? distance[head] * LOG2E * behind : distance_loss(distance[head], distance[nq + head], behind);
+}
 
 // A gate a head: the head's output times sigmoid(gates[token, head]), the gate values lying in rows of their own stride (the
 // columns of the projection that made them).  Null: no gate.
@@ -68,7 +77,7 @@ __global__ __launch_bounds__(THREADS) void attention_generic_kernel(
     const int* __restrict__ block_table, int table_stride, const int* __restrict__ token_request,
     const int* __restrict__ positions, int nq, int nkv, int d, int dv, int page_size, float scale,
     int window, int keep_first, const float* __restrict__ sinks, float softcap, const T* __restrict__ gates, int gate_stride,
-    const float* __restrict__ distance) {
+    const float* __restrict__ distance, int distance_form) {
   extern __shared__ __attribute__((aligned(16))) float smem[];
   float* qs = smem;                           // [d]
   float* probs = qs + d + d % 2;              // [THREADS]
@@ -80,7 +89,7 @@ __global__ __launch_bounds__(THREADS) void attention_generic_kernel(
   const int request = token_request[token];
   const int pos = positions[token];
   const int kv_head = head / (nq / nkv);
-  const int lo = (window > 0 && pos - window + 1 > 0) ? pos - window + 1 : 0;
+  const int lo = first_seen(pos, window);
   const int kept = lo > 0 ? (keep_first < lo ? keep_first : lo) : 0;    // keys 0 .. kept-1 are seen besides lo .. pos
   const int* table = block_table + (int64_t)request * table_stride;
 
@@ -119,7 +128,9 @@ __global__ __launch_bounds__(THREADS) void attention_generic_kernel(
       }
       score = dot * scale;
       if (softcap > 0.f) score = softcap * tanhf(score / softcap);
-      if (distance) score -= distance[head] * logf(1.f + distance[nq + head] * (float)(pos - key));
+      if (distance)
+        score -= distance_form == DISTANCE_LINEAR ? distance[head] * (float)(pos - key)
+                                                  : distance[head] * logf(1.f + distance[nq + head] * (float)(pos - key));
     }
     const float tile_max = block_max(score, scratch);
     const float new_max = fmaxf(running_max, tile_max);
@@ -283,7 +294,8 @@ __global__ __launch_bounds__(WAVES * 64) void attention_decode_bf16_kernel(
     bf16* __restrict__ v_pages, const int* __restrict__ block_table, int table_stride,
     const int* __restrict__ token_request, const int* __restrict__ positions, int nq, int nkv,
     int page_size, float scale, int window, int splits, int slots, DecodePrep prep, const float* __restrict__ sinks,
-    float softcap, const bf16* __restrict__ gates, int gate_stride, int dv_given, const float* __restrict__ distance_given) {
+    float softcap, const bf16* __restrict__ gates, int gate_stride, int dv_given, const float* __restrict__ distance_given,
+    int distance_form) {
   constexpr int DS = D / 32, DB = D / 16, THREADS = WAVES * 64;
   const int dv = MORE ? dv_given : D;
   const float* __restrict__ distance = MORE ? distance_given : nullptr;
@@ -294,7 +306,7 @@ __global__ __launch_bounds__(WAVES * 64) void attention_decode_bf16_kernel(
   const int split = blockIdx.x, kvh = blockIdx.y, token = blockIdx.z;
   const int group = nq / nkv;
   const int pos = positions[token];
-  const int lo = (window > 0 && pos - window + 1 > 0) ? pos - window + 1 : 0;
+  const int lo = first_seen(pos, window);
   const int* table = block_table + (int64_t)token_request[token] * table_stride;
   const int first_tile = lo / 32, last_tile = pos / 32;
   const int per_split = (last_tile - first_tile + splits) / splits;
@@ -424,7 +436,8 @@ __global__ __launch_bounds__(WAVES * 64) void attention_decode_bf16_kernel(
   const float scale2 = scale * 1.4426950408889634f;
   // the column's head's bias by distance, in the base-2 units of the scores below
   const int biased = kvh * group + (col < group ? col : 0);
-  const float rate2 = distance ? distance[biased] : 0.f, reach = distance ? distance[nq + biased] : 0.f;
+  const bool linear = MORE && distance_form == DISTANCE_LINEAR;
+  const float rate2 = distance ? distance[biased] * (linear ? LOG2E : 1.f) : 0.f, reach = distance && !linear ? distance[nq + biased] : 0.f;
 
   auto work = [&](int tile, bf16x8 (&kf)[2][DS], bf16x8 (&vf)[DB]) {
     if (holds_own && tile == last_tile) {
@@ -459,7 +472,7 @@ __global__ __launch_bounds__(WAVES * 64) void attention_decode_bf16_kernel(
         const int key = tile * 32 + g * 8 + h * 4 + i;
         const bool valid = key <= pos && key >= lo;
         float scaled = softcap > 0.f ? capped(s[h][i] * scale, softcap) * LOG2E : s[h][i] * scale2;
-        if (distance) scaled -= distance_loss(rate2, reach, (float)(pos - key));
+        if (distance) scaled -= linear ? rate2 * (float)(pos - key) : distance_loss(rate2, reach, (float)(pos - key));
         s[h][i] = valid ? scaled : -INFINITY;
         tile_max = fmaxf(tile_max, s[h][i]);
       }
@@ -662,7 +675,8 @@ __global__ __launch_bounds__(WAVE) void attention_kept_bf16_kernel(
     const bf16* __restrict__ q, int q_stride, const bf16* __restrict__ k_pages, const bf16* __restrict__ v_pages,
     const int* __restrict__ block_table, int table_stride, const int* __restrict__ token_request,
     const int* __restrict__ positions, int nq, int nkv, int d, int page_size, float scale, int window, int keep_first,
-    int slots, float* __restrict__ part_o, float* __restrict__ part_ml, float softcap, int dv, const float* __restrict__ distance) {
+    int slots, float* __restrict__ part_o, float* __restrict__ part_ml, float softcap, int dv, const float* __restrict__ distance,
+    int distance_form) {
   constexpr int PER_LANE = 4;                                     // heads of up to 256 dims
   const int token = blockIdx.x, head = blockIdx.y, lane = threadIdx.x;
   const int kvh = head / (nq / nkv);
@@ -695,7 +709,7 @@ __global__ __launch_bounds__(WAVE) void attention_kept_bf16_kernel(
 #pragma unroll
     for (int step = 1; step < WAVE; step *= 2) dot += __shfl_xor(dot, step, WAVE);
     float score = softcap > 0.f ? capped(dot * scale, softcap) * LOG2E : dot * scale2;
-    if (distance) score -= distance_loss(distance[head], distance[nq + head], (float)(pos - key));
+    if (distance) score -= distance_loss_of(distance, distance_form, nq, head, (float)(pos - key));
     const float new_top = fmaxf(top, score);
     const float keep = top == -INFINITY ? 0.f : fast_exp2(top - new_top);
     const float weight = fast_exp2(score - new_top);
@@ -718,10 +732,10 @@ __global__ __launch_bounds__(WAVE) void attention_kept_bf16_kernel(
 static void launch_attention_kept(const bf16* q, int q_stride, const bf16* k_pages, const bf16* v_pages, const int* block_table,
                                   int table_stride, const int* token_request, const int* positions, int tokens, int nq, int nkv, int d,
                                   int page_size, float scale, int window, int keep_first, int slots, float* part_o, float* part_ml,
-                                  float softcap, int dv, const float* distance, hipStream_t s) {
+                                  float softcap, int dv, const float* distance, int distance_form, hipStream_t s) {
   attention_kept_bf16_kernel<<<dim3(tokens, nq), WAVE, 0, s>>>(q, q_stride, k_pages, v_pages, block_table, table_stride, token_request,
                                                                positions, nq, nkv, d, page_size, scale, window, keep_first, slots, part_o,
-                                                               part_ml, softcap, dv, distance);
+                                                               part_ml, softcap, dv, distance, distance_form);
 }
 
 // Decode step in bf16: one query token per request.  part_o [tokens, nq, splits, d] and part_ml
@@ -738,14 +752,14 @@ LRS_API int lrs_attention_decode(void* out, int out_stride, float* part_o, float
                                  int page_size, float scale, int window, int keep_first, int splits, int form, int prepare,
                                  const void* q_weight, const void* k_weight, int w_dtype, float eps,
                                  const float* cosv, const float* sinv, int kv_columns, const float* sinks, float softcap,
-                                 const void* gates, int gate_stride, int dv, const float* distance, void* stream) {
-  LRS_REQUIRE(!distance || !prepare, "attention_decode: a bias by distance needs prepared heads");
+                                 const void* gates, int gate_stride, int dv, const float* distance, int distance_form, void* stream) {
+  LRS_REQUIRE(distance_form == DISTANCE_LOG || distance_form == DISTANCE_LINEAR, "attention_decode: unknown form %d of the bias by distance", distance_form);
   LRS_REQUIRE(dv > 0 && dv % 16 == 0 && dv <= d && (dv == d || !prepare),
               "attention_decode: values of %d dims beside keys of %d are not served (a multiple of 16, at most the keys', heads that come prepared)", dv, d);
   LRS_REQUIRE(tokens > 0 && nq > 0 && nkv > 0 && nq % nkv == 0, "attention_decode: bad sizes tokens=%d nq=%d nkv=%d", tokens, nq, nkv);
   LRS_REQUIRE(nq / nkv <= 16, "attention_decode: %d query heads per kv head, at most 16 fit a tile", nq / nkv);
   LRS_REQUIRE(page_size % 16 == 0, "attention_decode: page size %d is not a multiple of 16", page_size);
-  LRS_REQUIRE(window >= 0 && keep_first >= 0 && (keep_first == 0 || (window > 0 && !prepare)),
+  LRS_REQUIRE(keep_first >= 0 && (keep_first == 0 || (window > 0 && !prepare)),
               "attention_decode: kept first positions (%d) need a window and prepared heads", keep_first);
   const int slots = splits + (keep_first > 0 ? 1 : 0);          // the kept keys' share is one more partial result
   LRS_REQUIRE(splits >= 1 && (slots == 1 || (part_o && part_ml)), "attention_decode: %d partial results need their buffers", slots);
@@ -756,7 +770,8 @@ LRS_API int lrs_attention_decode(void* out, int out_stride, float* part_o, float
   hipStream_t s = (hipStream_t)stream;
   // LDS copy of the block table entries one workgroup walks
   LRS_REQUIRE(max_context >= 1, "attention_decode: max_context must be the longest context length of the step");
-  const int span = window > 0 && window + 64 < max_context ? window + 64 : max_context;
+  const int reach = window < 0 ? -window : window;
+  const int span = reach > 0 && reach + 64 < max_context ? reach + 64 : max_context;
   const size_t table_lds = sizeof(int) * (size_t)((span / 32 + splits) / splits * 32 / page_size + 4);
   LRS_REQUIRE(table_lds <= 24 * 1024, "attention_decode: a context of %d tokens in %d splits needs more block table entries than fit LDS", max_context, splits);
   if (prepare) {
@@ -775,7 +790,7 @@ LRS_API int lrs_attention_decode(void* out, int out_stride, float* part_o, float
 #define ARGS                                                                                                 \
   (bf16*)out, out_stride, part_o, part_ml, (const bf16*)q, q_stride, (bf16*)k_pages, (bf16*)v_pages, block_table, \
       table_stride, token_request, positions, nq, nkv, page_size, scale, window, splits, slots, prep, slots == 1 ? sinks : nullptr, softcap, \
-      slots == 1 ? (const bf16*)gates : nullptr, gate_stride, dv, distance
+      slots == 1 ? (const bf16*)gates : nullptr, gate_stride, dv, distance, distance_form
 #define LAUNCH_PREP(D, PREP, MORE)                                                                           \
   do {                                                                                                       \
     if (form == 2 && D <= 128) attention_decode_bf16_kernel<D, PREP, 8, (D <= 128), MORE><<<grid, 512, table_lds, s>>>(ARGS); \
@@ -784,7 +799,8 @@ LRS_API int lrs_attention_decode(void* out, int out_stride, float* part_o, float
   } while (0)
 #define LAUNCH(D)                        \
   do {                                   \
-    if (prepare) LAUNCH_PREP(D, true, false);                       \
+    if (prepare && distance) LAUNCH_PREP(D, true, true);            \
+    else if (prepare) LAUNCH_PREP(D, true, false);                  \
     else if (dv != d || distance) LAUNCH_PREP(D, false, true);      \
     else LAUNCH_PREP(D, false, false);                              \
   } while (0)
@@ -802,7 +818,7 @@ LRS_API int lrs_attention_decode(void* out, int out_stride, float* part_o, float
   if (lrs_check_launch("attention_decode")) return 1;
   if (keep_first > 0) {
     launch_attention_kept((const bf16*)q, q_stride, (const bf16*)k_pages, (const bf16*)v_pages, block_table, table_stride, token_request,
-                          positions, tokens, nq, nkv, d, page_size, scale, window, keep_first, slots, part_o, part_ml, softcap, dv, distance, s);
+                          positions, tokens, nq, nkv, d, page_size, scale, window, keep_first, slots, part_o, part_ml, softcap, dv, distance, distance_form, s);
     if (lrs_check_launch("attention_kept")) return 1;
   }
   if (slots > 1) {
@@ -841,7 +857,7 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void attention_prefill_bf16_
     const int* __restrict__ qblock_count, int n_blocks, int chunk, int nq, int nkv, int page_size, float scale,
     int window, int splits, int slots, float* __restrict__ part_o, float* __restrict__ part_ml,
     const float* __restrict__ sinks, float softcap, const bf16* __restrict__ gates, int gate_stride, int dv,
-    const float* __restrict__ distance) {
+    const float* __restrict__ distance, int distance_form) {
   constexpr int DS = D / 32, DB = D / 16;
   // Padded LDS rows.  Every fragment is read 16 bytes a lane, 16 rows at a time (the lane's row is col, its
   // piece g), which the LDS serves at its full 256 bytes a cycle when rows lie 32 bytes more than a multiple
@@ -864,8 +880,8 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void attention_prefill_bf16_
   const int qblock = chunk_block0 + ((which_chunk & 1) ? chunk_blocks - 1 - in_chunk / nkv : in_chunk / nkv);
   const int token0 = qblock_token0[qblock], count = qblock_count[qblock];
   const int pos_first = positions[token0], pos_last = positions[token0 + count - 1];
-  const int lo_first = (window > 0 && pos_first - window + 1 > 0) ? pos_first - window + 1 : 0;
-  const int lo_last = (window > 0 && pos_last - window + 1 > 0) ? pos_last - window + 1 : 0;
+  const int lo_first = first_seen(pos_first, window);
+  const int lo_last = first_seen(pos_last, window);
   const int* table = block_table + (int64_t)token_request[token0] * table_stride;
   const bf16x8 zero8 = {0, 0, 0, 0, 0, 0, 0, 0};
   const float scale2 = scale * 1.4426950408889634f;
@@ -958,7 +974,7 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void attention_prefill_bf16_
       live[b] = active && b * 16 + col < count;
       const int token = token0 + (live[b] ? b * 16 + col : 0);
       pos[b] = live[b] ? positions[token] : -1;                // a dead column sees no key
-      lo[b] = (window > 0 && pos[b] - window + 1 > 0) ? pos[b] - window + 1 : 0;
+      lo[b] = first_seen(pos[b], window);
       run_max[b] = -INFINITY;
       run_sum[b] = 0.f;
 #pragma unroll
@@ -970,13 +986,22 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void attention_prefill_bf16_
 
     // the head's bias by distance, in units of the unscaled scores
     const int biased = active ? head : head0;
-    const float rate = distance ? distance[biased] * LN2 / scale : 0.f, reach = distance ? distance[nq + biased] : 0.f;
+    const bool linear = distance && distance_form == DISTANCE_LINEAR;
+    const float rate = distance ? distance[biased] * (linear ? 1.f : LN2) / scale : 0.f, reach = distance && !linear ? distance[nq + biased] : 0.f;
+    // the linear form: what the products of keys first .. first + 3 are added to (with a cap on the scores, what is added to them)
+    auto linear_bias = [&](int b, int first) {
+      const float before = -rate * (float)((live[b] ? pos[b] : pos_last) - first);
+      return floatx4{before, fmaf(rate, 1.f, before), fmaf(rate, 2.f, before), fmaf(rate, 3.f, before)};
+    };
+    const bool linear_first = linear && !(softcap > 0.f);
     // The three parts of a tile's work.
     // scores: S[key, query] = K Q^T, unscaled (the scale enters with the exponent).
     auto scores = [&](int tile, int buffer, floatx4 (&sc)[QB][2]) {
       const bf16* kt = ks[buffer];
 #pragma unroll
-      for (int b = 0; b < QB; ++b) sc[b][0] = sc[b][1] = floatx4{0.f, 0.f, 0.f, 0.f};
+      for (int b = 0; b < QB; ++b)
+#pragma unroll
+        for (int h = 0; h < 2; ++h) sc[b][h] = linear_first ? linear_bias(b, tile * 32 + h * 16 + g * 4) : floatx4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
       for (int h = 0; h < 2; ++h)
 #pragma unroll
@@ -994,7 +1019,13 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void attention_prefill_bf16_
 #pragma unroll
             for (int i = 0; i < 4; ++i) sc[b][h][i] = capped(sc[b][h][i], cap);
       }
-      if (distance) {            // (a key ahead of the query gives no number here; the mask takes it out)
+      if (linear && !linear_first) {
+#pragma unroll
+        for (int b = 0; b < QB; ++b)
+#pragma unroll
+          for (int h = 0; h < 2; ++h) sc[b][h] += linear_bias(b, tile * 32 + h * 16 + g * 4);
+      }
+      if (distance && !linear) { // (a key ahead of the query gives no number here; the mask takes it out)
 #pragma unroll
         for (int b = 0; b < QB; ++b)
 #pragma unroll
@@ -1189,8 +1220,9 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void attention_prefill_bf16_
 // tile to the others; the fetches of the tile after it stay in flight.  The fetches are written in
 // assembly because the compiler would wait for all of them before any LDS read it cannot tell apart.
 // SCORES: what happens to the scores before the softmax, by instances of their own so that the others keep their registers:
-// nothing, a cap (softcap * tanh(score / softcap) of the scaled scores), a bias by distance, or the cap and then the bias.
-enum { SCORES_PLAIN = 0, SCORES_CAPPED = 1, SCORES_DISTANCE = 2, SCORES_BOTH = 3 };
+// nothing, a cap (softcap * tanh(score / softcap) of the scaled scores), a bias by distance (in the form with a logarithm, or the
+// linear one, which without a cap is what the products are added to and costs nothing), or the cap and then the bias.
+enum { SCORES_PLAIN = 0, SCORES_CAPPED = 1, SCORES_DISTANCE = 2, SCORES_BOTH = 3, SCORES_LINEAR = 4, SCORES_CAPPED_LINEAR = 5 };
 template <int QB, bool MANY_WAVES, bool IDLE_WAVES, int SCORES>
 __global__ __launch_bounds__(MANY_WAVES ? 512 : 256, MANY_WAVES ? 1 : 2) void attention_prefill_d128_bf16_kernel(
     bf16* __restrict__ out, int out_stride, const bf16* __restrict__ q, int q_stride,
@@ -1201,7 +1233,7 @@ __global__ __launch_bounds__(MANY_WAVES ? 512 : 256, MANY_WAVES ? 1 : 2) void at
     int window, int splits, int slots, float* __restrict__ part_o, float* __restrict__ part_ml, int prepare_q, DecodePrep prep,
     const float* __restrict__ sinks, float softcap, const bf16* __restrict__ gates, int gate_stride, int dv,
     const float* __restrict__ distance) {
-  constexpr bool CAPPED = (SCORES & SCORES_CAPPED) != 0, DISTANCE = (SCORES & SCORES_DISTANCE) != 0;
+  constexpr bool CAPPED = (SCORES & SCORES_CAPPED) != 0, DISTANCE = (SCORES & SCORES_DISTANCE) != 0, LINEAR = (SCORES & SCORES_LINEAR) != 0;
   constexpr int D = 128, DS = D / 32, DB = D / 16, STAGES = 3;
   constexpr int KBLOCK = 1024 + 32, KBYTES = 8 * KBLOCK, VHALF = 16 * D * 2 + 16, VBYTES = 2 * VHALF;
   constexpr int VSTAGE = (VBYTES + 63) / 64 * 64;
@@ -1220,8 +1252,8 @@ __global__ __launch_bounds__(MANY_WAVES ? 512 : 256, MANY_WAVES ? 1 : 2) void at
   const int qblock = chunk_block0 + ((which_chunk & 1) ? chunk_blocks - 1 - in_chunk / nkv : in_chunk / nkv);
   const int token0 = qblock_token0[qblock], count = qblock_count[qblock];
   const int pos_first = positions[token0], pos_last = positions[token0 + count - 1];
-  const int lo_first = (window > 0 && pos_first - window + 1 > 0) ? pos_first - window + 1 : 0;
-  const int lo_last = (window > 0 && pos_last - window + 1 > 0) ? pos_last - window + 1 : 0;
+  const int lo_first = first_seen(pos_first, window);
+  const int lo_last = first_seen(pos_last, window);
   const int* table = block_table + (int64_t)token_request[token0] * table_stride;
   const bf16x8 zero8 = {0, 0, 0, 0, 0, 0, 0, 0};
   const float scale2 = scale * 1.4426950408889634f;
@@ -1316,7 +1348,7 @@ __global__ __launch_bounds__(MANY_WAVES ? 512 : 256, MANY_WAVES ? 1 : 2) void at
       live[b] = active && b * 16 + col < count;
       const int token = token0 + (live[b] ? b * 16 + col : 0);
       pos[b] = live[b] ? positions[token] : -1;                // a dead column sees no key
-      lo[b] = (window > 0 && pos[b] - window + 1 > 0) ? pos[b] - window + 1 : 0;
+      lo[b] = first_seen(pos[b], window);
       run_max[b] = -INFINITY;
       run_sum[b] = 0.f;
       if (prepare_q) {
@@ -1354,6 +1386,29 @@ __global__ __launch_bounds__(MANY_WAVES ? 512 : 256, MANY_WAVES ? 1 : 2) void at
       rate = distance[biased] * LN2 / scale;
       reach = distance[nq + biased];
     }
+    if constexpr (LINEAR) rate = distance[active ? head : head0] / scale;
+    // the linear form for the lane's keys 4 h .. 4 h + 3 of a tile
+    auto linear_bias = [&](int tile, int b, int h) {
+      const float before = -rate * (float)((live[b] ? pos[b] : pos_last) - (tile * 32 + key_chunk * 8));
+      return floatx4{fmaf(rate, (float)(4 * h), before), fmaf(rate, (float)(4 * h + 1), before), fmaf(rate, (float)(4 * h + 2), before),
+                     fmaf(rate, (float)(4 * h + 3), before)};
+    };
+    // what a tile's products are added to
+    auto begin_scores = [&](int tile, floatx4 (&sc)[QB][2]) {
+#pragma unroll
+      for (int b = 0; b < QB; ++b)
+#pragma unroll
+        for (int h = 0; h < 2; ++h) {
+          if constexpr (LINEAR && !CAPPED) sc[b][h] = linear_bias(tile, b, h);
+          else sc[b][h] = floatx4{0.f, 0.f, 0.f, 0.f};
+        }
+    };
+    auto take_off_linear = [&](int tile, floatx4 (&sc)[QB][2]) {
+#pragma unroll
+      for (int b = 0; b < QB; ++b)
+#pragma unroll
+        for (int h = 0; h < 2; ++h) sc[b][h] += linear_bias(tile, b, h);
+    };
     auto take_off_distance = [&](int tile, floatx4 (&sc)[QB][2]) {
 #pragma unroll
       for (int b = 0; b < QB; ++b) {
@@ -1368,8 +1423,7 @@ __global__ __launch_bounds__(MANY_WAVES ? 512 : 256, MANY_WAVES ? 1 : 2) void at
     // scores: S[key, query] = K Q^T, unscaled (the scale enters with the exponent)
     auto scores = [&](int tile, int stage, floatx4 (&sc)[QB][2]) {
       const unsigned char* kt = key_tiles + stage * KBYTES + key_fragment;
-#pragma unroll
-      for (int b = 0; b < QB; ++b) sc[b][0] = sc[b][1] = floatx4{0.f, 0.f, 0.f, 0.f};
+      begin_scores(tile, sc);
 #pragma unroll
       for (int h = 0; h < 2; ++h)
 #pragma unroll
@@ -1380,6 +1434,7 @@ __global__ __launch_bounds__(MANY_WAVES ? 512 : 256, MANY_WAVES ? 1 : 2) void at
         }
       if constexpr (CAPPED) cap_scores(sc);
       if constexpr (DISTANCE) take_off_distance(tile, sc);
+      if constexpr (LINEAR && CAPPED) take_off_linear(tile, sc);
     };
     // weights: as in attention_prefill_bf16_kernel; sc[b][h][i] belongs to key tile * 32 + 8 m + 4 h + i
     auto weights_with_maximum = [&](int tile, floatx4 (&sc)[QB][2], auto masked, bf16x8 (&pf)[QB]) {
@@ -1442,9 +1497,9 @@ __global__ __launch_bounds__(MANY_WAVES ? 512 : 256, MANY_WAVES ? 1 : 2) void at
 #pragma unroll
       for (int f = 0; f < READ_AHEAD; ++f) kf[f] = *(const bf16x8*)(kt + (f / DS) * 512 + (f % DS) * 64);
       float shift[QB], tile_sum[QB], weight[QB * 8];
+      begin_scores(next_tile, next);
 #pragma unroll
       for (int b = 0; b < QB; ++b) {
-        next[b][0] = next[b][1] = floatx4{0.f, 0.f, 0.f, 0.f};
         shift[b] = -run_max[b] * scale2;                         // +inf before the query's first tile: the sum then says "again"
         tile_sum[b] = 0.f;
       }
@@ -1472,6 +1527,7 @@ __global__ __launch_bounds__(MANY_WAVES ? 512 : 256, MANY_WAVES ? 1 : 2) void at
       for (int b = 0; b < QB; ++b) run_sum[b] += tile_sum[b];
       if constexpr (CAPPED) cap_scores(next);
       if constexpr (DISTANCE) take_off_distance(next_tile, next);
+      if constexpr (LINEAR && CAPPED) take_off_linear(next_tile, next);
       return true;
     };
     // values: O^T[dim, query] += V^T P
@@ -1659,7 +1715,8 @@ LRS_API int lrs_attention_prefill(void* out, int out_stride, const void* q, int 
                                   int nkv, int d, int page_size, float scale, int window, int keep_first, int tokens, int splits,
                                   float* part_o, float* part_ml, int prepare, const void* q_weight, int w_dtype, float eps,
                                   const float* cosv, const float* sinv, const float* sinks, float softcap, const void* gates,
-                                  int gate_stride, int dv, const float* distance, void* stream) {
+                                  int gate_stride, int dv, const float* distance, int distance_form, void* stream) {
+  LRS_REQUIRE(distance_form == DISTANCE_LOG || distance_form == DISTANCE_LINEAR, "attention_prefill: unknown form %d of the bias by distance", distance_form);
   LRS_REQUIRE(dv > 0 && dv % 16 == 0 && dv <= d, "attention_prefill: values of %d dims beside keys of %d are not served (a multiple of 16, at most the keys')", dv, d);
   LRS_REQUIRE(n_blocks > 0 && nq > 0 && nkv > 0 && nq % nkv == 0, "attention_prefill: bad sizes blocks=%d nq=%d nkv=%d", n_blocks, nq, nkv);
   if (prepare) {
@@ -1673,7 +1730,7 @@ LRS_API int lrs_attention_prefill(void* out, int out_stride, const void* q, int 
   LRS_REQUIRE(max_count >= 1 && max_count <= 32, "attention_prefill: query groups hold 1..32 tokens, got %d", max_count);
   LRS_REQUIRE(softcap >= 0.f, "attention_prefill: the cap on the scores must be positive (0 = none), got %g", (double)softcap);
   LRS_REQUIRE(page_size % 16 == 0, "attention_prefill: page size %d is not a multiple of 16", page_size);
-  LRS_REQUIRE(window >= 0 && keep_first >= 0 && (keep_first == 0 || (window > 0 && !prepare)),
+  LRS_REQUIRE(keep_first >= 0 && (keep_first == 0 || (window > 0 && !prepare)),
               "attention_prefill: kept first positions (%d) need a window and prepared heads", keep_first);
   const int slots = splits + (keep_first > 0 ? 1 : 0);          // the kept keys' share is one more partial result
   const float* own_sinks = slots == 1 ? sinks : nullptr;          // with partial results the merge adds the sink
@@ -1689,7 +1746,8 @@ LRS_API int lrs_attention_prefill(void* out, int out_stride, const void* q, int 
   const int chunk = nkv >= compute_units() ? nkv : compute_units() / nkv * nkv;
   // LDS copy of the block table entries a workgroup walks: at most those of the longest context
   LRS_REQUIRE(max_context >= 1, "attention_prefill: max_context must be the longest context length of the step");
-  const int span = window > 0 && window + 32 + 64 < max_context ? window + 32 + 64 : max_context;
+  const int reach = window < 0 ? -window : window;
+  const int span = reach > 0 && reach + 32 + 64 < max_context ? reach + 32 + 64 : max_context;
   const size_t table_lds = sizeof(int) * (size_t)(span / page_size + 2);
   // (the kernel for heads of 128 reads the block table with scalar loads and keeps no copy)
   LRS_REQUIRE(d == 128 || table_lds <= 24 * 1024, "attention_prefill: a context of %d tokens needs more block table entries than fit LDS", max_context);
@@ -1699,7 +1757,7 @@ LRS_API int lrs_attention_prefill(void* out, int out_stride, const void* q, int 
                                                               (const bf16*)k_pages, (const bf16*)v_pages, block_table, \
                                                               table_stride, token_request, positions, qblock_token0, \
                                                               qblock_count, n_blocks, chunk, nq, nkv, page_size, scale, window, \
-                                                              splits, slots, part_o, part_ml, own_sinks, softcap, own_gates, gate_stride, dv, distance)
+                                                              splits, slots, part_o, part_ml, own_sinks, softcap, own_gates, gate_stride, dv, distance, distance_form)
 #define LAUNCH(D)                                \
   if (max_count <= 16) LAUNCH2(D, 1);            \
   else LAUNCH2(D, 2)
@@ -1716,7 +1774,10 @@ LRS_API int lrs_attention_prefill(void* out, int out_stride, const void* q, int 
         const bool many = nq / nkv > 4 && (int64_t)n_blocks * nkv * splits <= 2 * compute_units();
         if (many) block = dim3((nq / nkv < 8 ? nq / nkv : 8) * WAVE);
 #define D128(QB, MANY, IDLE)                                                                                                      \
-        if (softcap > 0.f && distance) D128C(QB, MANY, IDLE, SCORES_BOTH);                                                            \
+        const bool linear = distance && distance_form == DISTANCE_LINEAR;                                                             \
+        if (softcap > 0.f && linear) D128C(QB, MANY, IDLE, SCORES_CAPPED_LINEAR);                                                     \
+        else if (linear) D128C(QB, MANY, IDLE, SCORES_LINEAR);                                                                        \
+        else if (softcap > 0.f && distance) D128C(QB, MANY, IDLE, SCORES_BOTH);                                                       \
         else if (softcap > 0.f) D128C(QB, MANY, IDLE, SCORES_CAPPED);                                                                 \
         else if (distance) D128C(QB, MANY, IDLE, SCORES_DISTANCE);                                                                    \
         else D128C(QB, MANY, IDLE, SCORES_PLAIN)
@@ -1746,7 +1807,7 @@ LRS_API int lrs_attention_prefill(void* out, int out_stride, const void* q, int 
   if (lrs_check_launch("attention_prefill")) return 1;
   if (keep_first > 0) {
     launch_attention_kept((const bf16*)q, q_stride, (const bf16*)k_pages, (const bf16*)v_pages, block_table, table_stride, token_request,
-                          positions, tokens, nq, nkv, d, page_size, scale, window, keep_first, slots, part_o, part_ml, softcap, dv, distance, s);
+                          positions, tokens, nq, nkv, d, page_size, scale, window, keep_first, slots, part_o, part_ml, softcap, dv, distance, distance_form, s);
     if (lrs_check_launch("attention_kept")) return 1;
   }
   if (slots > 1) {
@@ -1764,12 +1825,13 @@ LRS_API int lrs_attention(void* out, int out_stride, const void* q, int q_stride
                           const void* v_pages, const int* block_table, int table_stride,
                           const int* token_request, const int* positions, int dtype, int tokens,
                           int nq, int nkv, int d, int dv, int page_size, float scale, int window, int keep_first,
-                          const float* sinks, float softcap, const void* gates, int gate_stride, const float* distance, void* stream) {
+                          const float* sinks, float softcap, const void* gates, int gate_stride, const float* distance, int distance_form, void* stream) {
   // value pages [P, nkv, dv, page]; out rows hold nq heads of dv values
   LRS_REQUIRE(tokens > 0 && nq > 0 && nkv > 0 && d > 0 && dv > 0 && page_size > 0, "attention: bad sizes tokens=%d nq=%d nkv=%d d=%d dv=%d page=%d", tokens, nq, nkv, d, dv, page_size);
   LRS_REQUIRE(nq % nkv == 0, "attention: %d query heads do not divide into %d kv heads", nq, nkv);
   LRS_REQUIRE(d <= 512 && dv <= 512, "attention: head sizes %d and %d above the supported 512", d, dv);
-  LRS_REQUIRE(window >= 0 && keep_first >= 0, "attention: window and keep_first must be >= 0 (0 = none)");
+  LRS_REQUIRE(keep_first >= 0 && (keep_first == 0 || window >= 0), "attention: keep_first must be >= 0 (0 = none) and comes with a window, not with chunks");
+  LRS_REQUIRE(distance_form == DISTANCE_LOG || distance_form == DISTANCE_LINEAR, "attention: unknown form %d of the bias by distance", distance_form);
   LRS_REQUIRE(softcap >= 0.f, "attention: the cap on the scores must be positive (0 = none), got %g", (double)softcap);
   constexpr int THREADS = 128;
   dim3 grid(tokens, nq);
@@ -1778,11 +1840,11 @@ LRS_API int lrs_attention(void* out, int out_stride, const void* q, int q_stride
   if (dtype == LRS_F32)
     attention_generic_kernel<float, THREADS><<<grid, THREADS, lds, s>>>(
         (float*)out, out_stride, (const float*)q, q_stride, (const float*)k_pages, (const float*)v_pages,
-        block_table, table_stride, token_request, positions, nq, nkv, d, dv, page_size, scale, window, keep_first, sinks, softcap, (const float*)gates, gate_stride, distance);
+        block_table, table_stride, token_request, positions, nq, nkv, d, dv, page_size, scale, window, keep_first, sinks, softcap, (const float*)gates, gate_stride, distance, distance_form);
   else if (dtype == LRS_BF16)
     attention_generic_kernel<bf16, THREADS><<<grid, THREADS, lds, s>>>(
         (bf16*)out, out_stride, (const bf16*)q, q_stride, (const bf16*)k_pages, (const bf16*)v_pages,
-        block_table, table_stride, token_request, positions, nq, nkv, d, dv, page_size, scale, window, keep_first, sinks, softcap, (const bf16*)gates, gate_stride, distance);
+        block_table, table_stride, token_request, positions, nq, nkv, d, dv, page_size, scale, window, keep_first, sinks, softcap, (const bf16*)gates, gate_stride, distance, distance_form);
   else
     return lrs_fail("attention: unknown dtype %d", dtype);
   return lrs_check_launch("attention");

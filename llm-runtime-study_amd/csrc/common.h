@@ -44,6 +44,15 @@ __device__ __forceinline__ float wave_max(float v) {
   return v;
 }
 
+// The first position that a query at `pos` sees, by the one number that every attention kernel takes as its `window`:
+//   window > 0   a sliding window: itself and the window - 1 positions before it;
+//   window < 0   chunks of -window positions, counted from position 0: those of its own chunk;
+//   window = 0   all.
+__device__ __forceinline__ int first_seen(int pos, int window) {
+  if (window < 0) return pos - pos % -window;
+  return window > 0 && pos - window + 1 > 0 ? pos - window + 1 : 0;
+}
+
 // Sum over a whole workgroup of up to 1024 threads; `scratch` holds 16 floats of LDS.
 // Every thread gets the result.  Contains two barriers.
 __device__ __forceinline__ float block_sum(float v, float* scratch) {

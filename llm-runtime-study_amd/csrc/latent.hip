@@ -11,9 +11,12 @@
 //
 //   latent_prep       per token: RMS norm of the projected latent values and rotation of the shared key part,
 //                     both written into the token's row of the pages; rotation of every head's rotated query part
-//                     into the query rows.  Pairs (2i, 2i + 1) are rotated (the interleaved layout).
+//                     into the query rows.  Pairs (2i, 2i + 1) are rotated (the interleaved layout).  Where the queries are
+//                     made from a latent row of their own, it normalises that row instead (a second workgroup a token), and
+//                     the queries, which are a product of it, are rotated by head_gemm.
 //   head_gemm         a small product per (token, head), with a matrix of the head's own: the two steps above that
-//                     move between a head's own dims and the latent ones.
+//                     move between a head's own dims and the latent ones.  On the way, where asked for: the rotation of
+//                     the values behind a head's inputs, put behind its outputs; a sigmoid gate a value on the outputs.
 //   latent_attention  scores, softmax with the sink, weighted sum of latent rows and the gate.
 //
 // Scores, weights, sums, norms and rotations are float32.  Key tiles start at multiples of the tile size counted
@@ -28,10 +31,22 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(
     const T* __restrict__ proj, int proj_stride, int q_col, int kv_col, int heads, int dim, int rot, int rank,
     const TW* __restrict__ norm_weight, float eps, const float* __restrict__ cosv, const float* __restrict__ sinv,
     T* __restrict__ pages, T* __restrict__ value_pages, int page_size, const int* __restrict__ slots, T* __restrict__ queries,
-    int query_stride) {
+    int query_stride, int q_rank, const TW* __restrict__ q_norm, T* __restrict__ q_latent, int q_latent_stride) {
   __shared__ float scratch[16];
   const int token = blockIdx.x, tid = threadIdx.x, half = rot / 2, width = rank + rot;
   const T* row = proj + (int64_t)token * proj_stride;
+  if (blockIdx.y == 1) {       // the queries' latent row, normalised; zeros behind it up to the rows' stride
+    float sq = 0.f;
+    for (int i = tid; i < q_rank; i += blockDim.x) {
+      const float v = to_float(row[q_col + i]);
+      sq += v * v;
+    }
+    const float inv_q = 1.0f / sqrtf(block_sum(sq, scratch) / (float)q_rank + eps);
+    T* dst = q_latent + (int64_t)token * q_latent_stride;
+    for (int i = tid; i < q_latent_stride; i += blockDim.x)
+      dst[i] = from_float<T>(i < q_rank ? to_float(row[q_col + i]) * inv_q * to_float(q_norm[i]) : 0.f);
+    return;
+  }
   const T* latent = row + kv_col;
   const int slot = slots[token];
   float ss = 0.f;
@@ -78,10 +93,31 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(
 // (TRANS true).  A workgroup takes TT tokens of one head; the sum runs in the order of k.
 constexpr int HG_TOKENS = 8;
 
+// What else happens on the way: the `rot` values behind a (token, head)'s k inputs are rotated in pairs (2i, 2i + 1) and put behind
+// its n outputs (rot 0: nothing); output j of head h is multiplied by sigmoid(gate[t, h * n + j]) (null: no gate).
+template <typename T>
+struct HeadExtras {
+  int rot;
+  const float *cosv, *sinv;      // [tokens, rot / 2]
+  const T* gate;
+  int gate_stride;
+};
+template <typename T>
+__device__ __forceinline__ void rotate_behind(const HeadExtras<T>& ex, T* __restrict__ out_row, const T* __restrict__ a_row, int t, int n, int k, int pair) {
+  const float c = ex.cosv[(int64_t)t * (ex.rot / 2) + pair], s = ex.sinv[(int64_t)t * (ex.rot / 2) + pair];
+  const float u = to_float(a_row[k + 2 * pair]), v = to_float(a_row[k + 2 * pair + 1]);
+  out_row[n + 2 * pair] = from_float<T>(u * c - v * s);
+  out_row[n + 2 * pair + 1] = from_float<T>(v * c + u * s);
+}
+template <typename T>
+__device__ __forceinline__ float gated_value(const HeadExtras<T>& ex, float v, int t, int h, int n, int j) {
+  return ex.gate ? v / (1.0f + expf(-to_float(ex.gate[(int64_t)t * ex.gate_stride + (int64_t)h * n + j]))) : v;
+}
+
 template <typename T, bool TRANS>
 __global__ __launch_bounds__(256) void head_gemm_kernel(T* __restrict__ out, int out_token, int out_head, const T* __restrict__ a,
                                                         int a_token, int a_head, const T* __restrict__ w, int64_t w_head, int tokens,
-                                                        int n, int k) {
+                                                        int n, int k, const HeadExtras<T> ex) {
   extern __shared__ __attribute__((aligned(16))) float rows[];     // [HG_TOKENS][k]
   const int t0 = blockIdx.x * HG_TOKENS, h = blockIdx.y, tid = threadIdx.x;
   const int count = min(HG_TOKENS, tokens - t0);
@@ -90,6 +126,10 @@ __global__ __launch_bounds__(256) void head_gemm_kernel(T* __restrict__ out, int
     rows[i] = t < count ? to_float(a[(int64_t)(t0 + t) * a_token + (int64_t)h * a_head + c]) : 0.f;
   }
   __syncthreads();
+  for (int i = tid; i < count * (ex.rot / 2); i += blockDim.x) {
+    const int t = t0 + i / (ex.rot / 2);
+    rotate_behind(ex, out + (int64_t)t * out_token + (int64_t)h * out_head, a + (int64_t)t * a_token + (int64_t)h * a_head, t, n, k, i % (ex.rot / 2));
+  }
   const T* wh = w + (int64_t)h * w_head;
   for (int j = tid; j < n; j += blockDim.x) {
     float acc[HG_TOKENS];
@@ -102,7 +142,7 @@ __global__ __launch_bounds__(256) void head_gemm_kernel(T* __restrict__ out, int
     }
 #pragma unroll
     for (int t = 0; t < HG_TOKENS; ++t)
-      if (t < count) out[(int64_t)(t0 + t) * out_token + (int64_t)h * out_head + j] = from_float<T>(acc[t]);
+      if (t < count) out[(int64_t)(t0 + t) * out_token + (int64_t)h * out_head + j] = from_float<T>(gated_value(ex, acc[t], t0 + t, h, n, j));
   }
 }
 
@@ -126,7 +166,7 @@ __global__ __launch_bounds__(LA_THREADS) void latent_attention_kernel(
   const int token = blockIdx.x, head = blockIdx.y, tid = threadIdx.x;
   const int request = token_request[token];
   const int pos = positions[token];
-  const int lo = (window > 0 && pos - window + 1 > 0) ? pos - window + 1 : 0;
+  const int lo = first_seen(pos, window);
   const int* table = block_table + (int64_t)request * table_stride;
   for (int i = tid; i < width; i += THREADS) qs[i] = to_float(queries[(int64_t)token * query_stride + (int64_t)head * width + i]);
   __syncthreads();
@@ -208,10 +248,17 @@ __global__ __launch_bounds__(LA_THREADS) void latent_attention_kernel(
 // bfloat16, w[h] stored [n, k]: a wave makes 16 tokens x 64 outputs with both operands straight from memory (16 bytes a lane).
 __global__ __launch_bounds__(256) void head_gemm_bf16_kernel(bf16* __restrict__ out, int out_token, int out_head, const bf16* __restrict__ a,
                                                              int a_token, int a_head, const bf16* __restrict__ w, int64_t w_head, int tokens,
-                                                             int n, int k) {
+                                                             int n, int k, const HeadExtras<bf16> ex) {
   const int lane = threadIdx.x % WAVE, wave = threadIdx.x / WAVE, col = lane & 15, g = lane >> 4;
   const int h = blockIdx.z, n0 = blockIdx.y * 64, t0 = blockIdx.x * 64 + wave * 16;
   if (t0 >= tokens) return;
+  if (ex.rot && blockIdx.y == 0) {
+    const int half = ex.rot / 2;
+    for (int i = lane; i < 16 * half; i += WAVE) {
+      const int at = t0 + i / half;
+      if (at < tokens) rotate_behind(ex, out + (int64_t)at * out_token + (int64_t)h * out_head, a + (int64_t)at * a_token + (int64_t)h * a_head, at, n, k, i % half);
+    }
+  }
   const int t = t0 + col;
   const bf16* a_row = a + (int64_t)(t < tokens ? t : tokens - 1) * a_token + (int64_t)h * a_head + g * 8;
   const bf16* w_row = w + (int64_t)h * w_head + (int64_t)(n0 + col) * k + g * 8;
@@ -237,7 +284,7 @@ __global__ __launch_bounds__(256) void head_gemm_bf16_kernel(bf16* __restrict__ 
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
       const int row = t0 + 4 * g + i, nn = n0 + 16 * c + col;
-      if (row < tokens && nn < n) out[(int64_t)row * out_token + (int64_t)h * out_head + nn] = (bf16)acc[c][i];
+      if (row < tokens && nn < n) out[(int64_t)row * out_token + (int64_t)h * out_head + nn] = (bf16)gated_value(ex, acc[c][i], row, h, n, nn);
     }
 }
 
@@ -269,7 +316,7 @@ __global__ __launch_bounds__(256) void latent_attention_bf16_kernel(
   const int last_row = row0 + 15 < rows ? row0 + 15 : rows - 1;
   const int* table = block_table + (int64_t)token_request[token0] * table_stride;
   const int pos_first = positions[token0 + row0 / heads], pos_last = positions[token0 + last_row / heads];
-  const int lo = (window > 0 && pos_first - window + 1 > 0) ? pos_first - window + 1 : 0;
+  const int lo = first_seen(pos_first, window);
   const int first_tile = lo / 32, last_tile = pos_last / 32;
   const int per_split = (last_tile - first_tile + splits) / splits;
   const int tile_begin = first_tile + split * per_split;
@@ -284,7 +331,7 @@ __global__ __launch_bounds__(256) void latent_attention_bf16_kernel(
   for (int i = 0; i < 4; ++i) {
     const int r = row0 + 4 * g + i;
     c_pos[i] = r < rows ? positions[token0 + r / heads] : -1;
-    c_lo[i] = (window > 0 && c_pos[i] - window + 1 > 0) ? c_pos[i] - window + 1 : 0;
+    c_lo[i] = first_seen(c_pos[i], window);
   }
   const float scale2 = scale * LOG2E;
   float top[4], total[4];
@@ -458,17 +505,23 @@ __global__ __launch_bounds__(256) void latent_merge_kernel(bf16* __restrict__ ou
 // proj [tokens, >= columns] holds, per token, the heads' queries from column q_col on ([dim plain | rot rotated] a head)
 // and [rank latent | rot shared key] from column kv_col on.  pages [P, page, rank + rot]; value_pages (may be null)
 // [P, rank, page]; slots[t] the token's row (negative: not kept).  queries [tokens, heads, rank + rot]: the rotated parts are written, the others left.
+// q_rank > 0: instead of queries, column q_col begins a latent row of q_rank values that the queries will be made of: its RMS norm
+// (weight q_norm [q_rank], of weight_dtype) goes into q_latent [tokens, q_latent_stride], zeros behind it; heads is 0 then.
 LRS_API int lrs_latent_prep(const void* proj, int proj_stride, int dtype, int tokens, int q_col, int kv_col, int heads, int dim, int rot,
                             int rank, const void* norm_weight, int weight_dtype, float eps, const float* cosv, const float* sinv,
-                            void* pages, void* value_pages, int page_size, const int* slots, void* queries, int query_stride, void* stream) {
-  LRS_REQUIRE(tokens > 0 && heads > 0 && dim >= 0 && rot >= 0 && rank > 0, "latent_prep: bad sizes tokens=%d heads=%d dim=%d rot=%d rank=%d", tokens, heads,
+                            void* pages, void* value_pages, int page_size, const int* slots, void* queries, int query_stride, int q_rank,
+                            const void* q_norm, void* q_latent, int q_latent_stride, void* stream) {
+  LRS_REQUIRE(tokens > 0 && heads >= 0 && dim >= 0 && rot >= 0 && rank > 0, "latent_prep: bad sizes tokens=%d heads=%d dim=%d rot=%d rank=%d", tokens, heads,
               dim, rot, rank);
+  LRS_REQUIRE(q_rank > 0 ? heads == 0 && q_norm && q_latent && q_latent_stride >= q_rank : heads > 0 && queries,
+              "latent_prep: either queries of some heads or the latent row they are made of (heads=%d q_rank=%d)", heads, q_rank);
   LRS_REQUIRE(eps > 0.f, "latent_prep: eps must be positive");
   LRS_REQUIRE((cosv == nullptr) == (sinv == nullptr), "latent_prep: cos and sin come together");
   hipStream_t s = (hipStream_t)stream;
 #define LRS_PREP(T, TW)                                                                                                              \
-  latent_prep_kernel<T, TW><<<tokens, 256, 0, s>>>((const T*)proj, proj_stride, q_col, kv_col, heads, dim, rot, rank, (const TW*)norm_weight, \
-                                                   eps, cosv, sinv, (T*)pages, (T*)value_pages, page_size, slots, (T*)queries, query_stride)
+  latent_prep_kernel<T, TW><<<dim3(tokens, q_rank > 0 ? 2 : 1), 256, 0, s>>>((const T*)proj, proj_stride, q_col, kv_col, heads, dim, rot, rank, (const TW*)norm_weight, \
+                                                   eps, cosv, sinv, (T*)pages, (T*)value_pages, page_size, slots, (T*)queries, query_stride, \
+                                                   q_rank, (const TW*)q_norm, (T*)q_latent, q_latent_stride)
   if (dtype == LRS_F32 && weight_dtype == LRS_F32) LRS_PREP(float, float);
   else if (dtype == LRS_F32 && weight_dtype == LRS_BF16) LRS_PREP(float, bf16);
   else if (dtype == LRS_BF16 && weight_dtype == LRS_F32) LRS_PREP(bf16, float);
@@ -479,9 +532,12 @@ LRS_API int lrs_latent_prep(const void* proj, int proj_stride, int dtype, int to
 }
 
 // out[t, h, :n] = w[h] a[t, h, :k] with w[h] stored [n, k] (trans 0) or [k, n] (trans 1), w_head elements from one head's
-// matrix to the next; strides in elements.
+// matrix to the next; strides in elements.  rot > 0 (even; cosv, sinv [tokens, rot / 2]): the rot values behind a's k are rotated and
+// put behind out's n.  gate (rows of gate_stride, or null): out[t, h, j] is multiplied by sigmoid(gate[t, h * n + j]).
 LRS_API int lrs_head_gemm(void* out, int out_token, int out_head, const void* a, int a_token, int a_head, const void* w, int64_t w_head,
-                          int trans, int dtype, int tokens, int heads, int n, int k, void* stream) {
+                          int trans, int dtype, int tokens, int heads, int n, int k, int rot, const float* cosv, const float* sinv,
+                          const void* gate, int gate_stride, void* stream) {
+  LRS_REQUIRE(rot >= 0 && rot % 2 == 0 && (rot == 0 || (cosv && sinv)), "head_gemm: %d values to rotate need tables and are even", rot);
   LRS_REQUIRE(tokens > 0 && heads > 0 && n > 0 && k > 0, "head_gemm: bad sizes tokens=%d heads=%d n=%d k=%d", tokens, heads, n, k);
   LRS_REQUIRE(heads <= 65535, "head_gemm: at most 65535 heads");
   LRS_REQUIRE(k <= 4096, "head_gemm: k %d above the supported 4096", k);
@@ -489,13 +545,15 @@ LRS_API int lrs_head_gemm(void* out, int out_token, int out_head, const void* a,
   if (dtype == LRS_BF16 && !trans && k % 8 == 0 && a_token % 8 == 0 && a_head % 8 == 0 && (uintptr_t)a % 16 == 0 && (uintptr_t)w % 16 == 0 &&
       (n + 63) / 64 <= 65535) {
     head_gemm_bf16_kernel<<<dim3((tokens + 63) / 64, (n + 63) / 64, heads), 256, 0, s>>>((bf16*)out, out_token, out_head, (const bf16*)a, a_token, a_head,
-                                                                                       (const bf16*)w, w_head, tokens, n, k);
+                                                                                       (const bf16*)w, w_head, tokens, n, k,
+                                                                                       HeadExtras<bf16>{rot, cosv, sinv, (const bf16*)gate, gate_stride});
     return lrs_check_launch("head_gemm");
   }
   const dim3 grid((tokens + HG_TOKENS - 1) / HG_TOKENS, heads);
   const size_t lds = sizeof(float) * HG_TOKENS * k;
 #define LRS_HG(T, TR) \
-  head_gemm_kernel<T, TR><<<grid, 256, lds, s>>>((T*)out, out_token, out_head, (const T*)a, a_token, a_head, (const T*)w, w_head, tokens, n, k)
+  head_gemm_kernel<T, TR><<<grid, 256, lds, s>>>((T*)out, out_token, out_head, (const T*)a, a_token, a_head, (const T*)w, w_head, tokens, n, k, \
+                                            HeadExtras<T>{rot, cosv, sinv, (const T*)gate, gate_stride})
   if (dtype == LRS_F32) { if (trans) LRS_HG(float, true); else LRS_HG(float, false); }
   else if (dtype == LRS_BF16) { if (trans) LRS_HG(bf16, true); else LRS_HG(bf16, false); }
   else return lrs_fail("head_gemm: unknown dtype %d", dtype);
@@ -512,7 +570,7 @@ LRS_API int lrs_latent_attention(void* out, int out_stride, const void* queries,
   LRS_REQUIRE(tokens > 0 && heads > 0 && rank > 0 && width >= rank && page_size > 0, "latent_attention: bad sizes tokens=%d heads=%d rank=%d width=%d page=%d",
               tokens, heads, rank, width, page_size);
   LRS_REQUIRE(rank <= LA_THREADS * LA_MAX_OUT, "latent_attention: rank %d above the supported %d", rank, LA_THREADS * LA_MAX_OUT);
-  LRS_REQUIRE(heads <= 65535 && window >= 0, "latent_attention: at most 65535 heads, window >= 0 (0 = none)");
+  LRS_REQUIRE(heads <= 65535, "latent_attention: at most 65535 heads");
   const dim3 grid(tokens, heads);
   const size_t lds = sizeof(float) * (width + width % 2 + LA_THREADS) + sizeof(int64_t) * LA_THREADS;
   hipStream_t s = (hipStream_t)stream;
@@ -549,7 +607,6 @@ LRS_API int lrs_latent_attention_groups(void* out, int out_stride, const void* q
   LRS_REQUIRE((uintptr_t)queries % 16 == 0 && (uintptr_t)pages % 16 == 0 && (uintptr_t)value_pages % 16 == 0 && query_stride % 8 == 0, "latent_attention_groups: operands must be 16-byte aligned");
   LRS_REQUIRE((group_token0 == nullptr) == (group_count == nullptr), "latent_attention_groups: the groups' first tokens and counts come together");
   LRS_REQUIRE(splits >= 1 && splits <= 64 && (splits == 1 || (part_o && part_ml)), "latent_attention_groups: splits 1..64, with room for the parts");
-  LRS_REQUIRE(window >= 0, "latent_attention_groups: window must be >= 0 (0 = none)");
   const int tiles = ((int64_t)max_count * heads + 63) / 64;
   LRS_REQUIRE(tiles <= 65535 && splits <= 65535, "latent_attention_groups: too many rows a group");
   const dim3 grid(groups, tiles, splits);

@@ -76,7 +76,8 @@ __device__ __forceinline__ void route_token(const float* __restrict__ logits, in
 //                         groups > 0 the experts form that many equal groups of neighbours, a group's score is the sum of
 //                         its two largest (s + bias), and only experts of the `keep` best groups can be chosen.
 //   ROUTE_SIGMOID_SCORES  chosen as under ROUTE_SIGMOID; weights: the chosen s themselves, times `scale` (not divided by their sum)
-enum { ROUTE_SOFTMAX_CHOSEN = 0, ROUTE_SIGMOID = 1, ROUTE_SIGMOID_SCORES = 2 };
+//   ROUTE_SOFTMAX_SCORES  the same with the scores s = softmax(logits) over all experts (no groups)
+enum { ROUTE_SOFTMAX_CHOSEN = 0, ROUTE_SIGMOID = 1, ROUTE_SIGMOID_SCORES = 2, ROUTE_SOFTMAX_SCORES = 3 };
 struct RouteRule {
   int kind, groups, keep;
   float scale;
@@ -99,18 +100,31 @@ __device__ __forceinline__ float route_max(const float (&v)[ROUTE_MAX_PER_LANE])
   return wave_max(best);
 }
 
-// One token by one wave, ROUTE_SIGMOID.
-__device__ __forceinline__ void route_token_sigmoid(const float* __restrict__ logits, int ld, const float* __restrict__ bias,
+// One token by one wave: every rule that chooses by scores of all experts.
+__device__ __forceinline__ void route_token_scores(const float* __restrict__ logits, int ld, const float* __restrict__ bias,
                                                     int* ids, float* __restrict__ weights, int t, int experts, int top, int lane,
                                                     const RouteRule rule) {
-  float s[ROUTE_MAX_PER_LANE], v[ROUTE_MAX_PER_LANE];
+  float s[ROUTE_MAX_PER_LANE], v[ROUTE_MAX_PER_LANE], zs[ROUTE_MAX_PER_LANE];
 #pragma unroll
   for (int c = 0; c < ROUTE_MAX_PER_LANE; ++c) {
     const int e = lane + WAVE * c;
-    const float z = e < experts ? logits[(int64_t)t * ld + e] : 0.f;
-    s[c] = e < experts ? 1.0f / (1.0f + expf(-z)) : 0.f;
+    zs[c] = e < experts ? logits[(int64_t)t * ld + e] : -INFINITY;
+  }
+  float highest = 0.f, all = 1.f;
+  if (rule.kind == ROUTE_SOFTMAX_SCORES) {
+    highest = route_max(zs);
+    all = 0.f;
+#pragma unroll
+    for (int c = 0; c < ROUTE_MAX_PER_LANE; ++c) all += lane + WAVE * c < experts ? expf(zs[c] - highest) : 0.f;
+    all = wave_sum(all);
+  }
+#pragma unroll
+  for (int c = 0; c < ROUTE_MAX_PER_LANE; ++c) {
+    const int e = lane + WAVE * c;
+    const float z = zs[c];
+    s[c] = e >= experts ? 0.f : rule.kind == ROUTE_SOFTMAX_SCORES ? expf(z - highest) / all : 1.0f / (1.0f + expf(-z));
     // without a bias and without groups the order of the scores is the order of the logits, which does not run out of
-    // digits where the sigmoid nears one (logits of 17 and of 30 both give 1.0f)
+    // digits where the sigmoid nears one (logits of 17 and of 30 both give 1.0f) or the softmax nears zero
     v[c] = e < experts ? (bias || rule.groups > 0 ? s[c] + (bias ? bias[e] : 0.f) : z) : -INFINITY;
   }
   if (rule.groups > 0 && rule.keep < rule.groups) {
@@ -172,7 +186,7 @@ __device__ __forceinline__ void route_token_sigmoid(const float* __restrict__ lo
     }
   }
   // the same lane wrote them: it reads its own stores
-  if (lane == 0 && rule.kind == ROUTE_SIGMOID_SCORES) {
+  if (lane == 0 && rule.kind >= ROUTE_SIGMOID_SCORES) {
     if (rule.scale != 1.f)
       for (int k = 0; k < top; ++k) weights[(int64_t)t * top + k] *= rule.scale;
   } else if (lane == 0) {
@@ -185,14 +199,15 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const float* __restrict_
                                                         int experts, int top, const RouteRule rule) {
   const int t = blockIdx.x * (blockDim.x / WAVE) + threadIdx.x / WAVE;
   if (t >= tokens) return;
-  if (rule.kind != ROUTE_SOFTMAX_CHOSEN) route_token_sigmoid(logits, ld, bias, ids, weights, t, experts, top, threadIdx.x % WAVE, rule);
+  if (rule.kind != ROUTE_SOFTMAX_CHOSEN) route_token_scores(logits, ld, bias, ids, weights, t, experts, top, threadIdx.x % WAVE, rule);
   else route_token(logits, ld, bias, ids, weights, t, experts, top, threadIdx.x % WAVE);
 }
 
 // sorted [capacity]: the pair (token * top + choice) at each row of the sorted order, -1 for the rows that pad an
 // expert's run to whole tiles; place [pairs]: the row of each pair; tile_expert [max_tiles]: the expert of each
-// tile of `tile` rows, -1 for tiles not in use.
-__device__ __forceinline__ void align_pairs(const int* ids, int pairs, int experts, int tile, int* __restrict__ sorted,
+// tile of `tile` rows, -1 for tiles not in use.  The `identity` ids behind the experts' stand for the token itself: such a pair
+// has no row (place -1), no tile and no place in the list.
+__device__ __forceinline__ void align_pairs(const int* ids, int pairs, int experts, int identity, int tile, int* __restrict__ sorted,
                                             int capacity, int* __restrict__ place, int* __restrict__ tile_expert, int max_tiles,
                                             int* shared) {
   int* count = shared;                  // [experts]
@@ -203,7 +218,11 @@ __device__ __forceinline__ void align_pairs(const int* ids, int pairs, int exper
   for (int i = tid; i < capacity; i += blockDim.x) sorted[i] = -1;
   for (int i = tid; i < max_tiles; i += blockDim.x) tile_expert[i] = -1;
   __syncthreads();
-  for (int i = tid; i < pairs; i += blockDim.x) atomicAdd(&count[min((unsigned)ids[i], (unsigned)experts - 1)], 1);
+  auto itself = [&](int id) { return id >= experts && id < experts + identity; };
+  for (int i = tid; i < pairs; i += blockDim.x) {
+    const int id = ids[i];
+    if (!itself(id)) atomicAdd(&count[min((unsigned)id, (unsigned)experts - 1)], 1);
+  }
   __syncthreads();
   if (tid == 0) {
     int at = 0;
@@ -217,32 +236,37 @@ __device__ __forceinline__ void align_pairs(const int* ids, int pairs, int exper
   for (int e = tid; e < experts; e += blockDim.x)
     for (int i = first[e] / tile; i < first[e + 1] / tile; ++i) tile_expert[i] = e;
   for (int i = tid; i < pairs; i += blockDim.x) {
-    const int e = min((unsigned)ids[i], (unsigned)experts - 1), row = first[e] + atomicAdd(&cursor[e], 1);
+    const int id = ids[i];
+    if (itself(id)) {
+      place[i] = -1;
+      continue;
+    }
+    const int e = min((unsigned)id, (unsigned)experts - 1), row = first[e] + atomicAdd(&cursor[e], 1);
     sorted[row] = i;
     place[i] = row;
   }
 }
 
-__global__ __launch_bounds__(1024) void moe_align_kernel(const int* __restrict__ ids, int pairs, int experts, int tile,
+__global__ __launch_bounds__(1024) void moe_align_kernel(const int* __restrict__ ids, int pairs, int experts, int identity, int tile,
                                                          int* __restrict__ sorted, int capacity, int* __restrict__ place,
                                                          int* __restrict__ tile_expert, int max_tiles) {
   extern __shared__ int shared[];
-  align_pairs(ids, pairs, experts, tile, sorted, capacity, place, tile_expert, max_tiles, shared);
+  align_pairs(ids, pairs, experts, identity, tile, sorted, capacity, place, tile_expert, max_tiles, shared);
 }
 
 // Both in one workgroup, for steps of few tokens (single tokens above all), where a launch costs more than either does.
 __global__ __launch_bounds__(1024) void moe_route_align_kernel(const float* __restrict__ logits, int ld, const float* __restrict__ bias,
                                                                int* ids, float* __restrict__ weights, int tokens, int experts,
-                                                               int top, int tile, int* __restrict__ sorted, int capacity,
+                                                               int identity, int top, int tile, int* __restrict__ sorted, int capacity,
                                                                int* __restrict__ place, int* __restrict__ tile_expert, int max_tiles,
                                                                const RouteRule rule) {
   extern __shared__ int shared[];
   for (int t = threadIdx.x / WAVE; t < tokens; t += blockDim.x / WAVE) {
-    if (rule.kind != ROUTE_SOFTMAX_CHOSEN) route_token_sigmoid(logits, ld, bias, ids, weights, t, experts, top, threadIdx.x % WAVE, rule);
-    else route_token(logits, ld, bias, ids, weights, t, experts, top, threadIdx.x % WAVE);
+    if (rule.kind != ROUTE_SOFTMAX_CHOSEN) route_token_scores(logits, ld, bias, ids, weights, t, experts + identity, top, threadIdx.x % WAVE, rule);
+    else route_token(logits, ld, bias, ids, weights, t, experts + identity, top, threadIdx.x % WAVE);
   }
   __syncthreads();          // the choices are in memory for every thread of the workgroup
-  align_pairs(ids, tokens * top, experts, tile, sorted, capacity, place, tile_expert, max_tiles, shared);
+  align_pairs(ids, tokens * top, experts, identity, tile, sorted, capacity, place, tile_expert, max_tiles, shared);
 }
 
 // ACT_SILU_PAIRS: the matrix holds, for every feature j, a gate row 2j and an up row 2j + 1; the output has half as many columns,
@@ -635,13 +659,24 @@ __global__ __launch_bounds__(256, 2) void moe_experts_bf16_fetch_kernel(TO* __re
 //   COMBINE_ADD        residual += y
 //   COMBINE_ADD_RMS    residual += w * y * rsqrt(mean(y^2) + eps)                       (a layer that normalises what a sublayer gives out)
 //   COMBINE_LAYERNORM  residual = w * (z - mean z) / sqrt(variance of z + eps), z = alpha * residual + y   (one that normalises the sum)
-enum { COMBINE_ADD = 0, COMBINE_ADD_RMS = 1, COMBINE_LAYERNORM = 2 };
+//   COMBINE_STORE      residual = y
+// A choice without a row (place -1) is the token's own input (self, of the expert's input dtype).  With COMBINE_ADD_RMS the RMS norm
+// of the new row can be left beside it (next): the input of the sublayer that runs next.
+enum { COMBINE_ADD = 0, COMBINE_ADD_RMS = 1, COMBINE_LAYERNORM = 2, COMBINE_STORE = 3 };
+struct CombineMore {
+  const void* self;            // [tokens, hidden] rows of self_stride, or null
+  int self_f32, self_stride;
+  const float* next_weight;    // [hidden], with `normed`
+  float next_eps;
+  void* normed;                // [tokens, hidden], or null
+  int normed_f32;
+};
 
 template <typename TW>
 __global__ __launch_bounds__(1024) void moe_combine_kernel(float* __restrict__ residual, const float* __restrict__ rows, int hidden,
                                                            const int* __restrict__ place, const float* __restrict__ weights, int top,
                                                            const TW* __restrict__ norm_w, float eps, bf16* __restrict__ rounded, int kind,
-                                                           float alpha, const float* __restrict__ extra) {
+                                                           float alpha, const float* __restrict__ extra, const CombineMore more) {
   extern __shared__ float sum[];        // [hidden], 16 floats for the reduction, then the token's rows and weights [top] each
   float* share = sum + hidden + 16;
   int* where = (int*)(share + top);
@@ -655,7 +690,13 @@ __global__ __launch_bounds__(1024) void moe_combine_kernel(float* __restrict__ r
   float ss = 0.f;
   for (int i = threadIdx.x; i < hidden; i += blockDim.x) {
     float acc = 0.f;
-    for (int c = 0; c < top; ++c) acc = fmaf(share[c], rows[(int64_t)where[c] * hidden + i], acc);
+    if (more.self == nullptr) {
+      for (int c = 0; c < top; ++c) acc = fmaf(share[c], rows[(int64_t)where[c] * hidden + i], acc);
+    } else {
+      const int64_t at = (int64_t)t * more.self_stride + i;
+      const float mine = more.self_f32 ? ((const float*)more.self)[at] : (float)((const bf16*)more.self)[at];
+      for (int c = 0; c < top; ++c) acc = fmaf(share[c], where[c] < 0 ? mine : rows[(int64_t)where[c] * hidden + i], acc);
+    }
     if (extra) acc += extra[(int64_t)t * hidden + i];          // what a part that runs for every token gave out
     if (kind == COMBINE_LAYERNORM) {
       acc = fmaf(alpha, out[i], acc);
@@ -680,7 +721,11 @@ __global__ __launch_bounds__(1024) void moe_combine_kernel(float* __restrict__ r
     }
     return;
   }
-  float inv = 1.f;
+  if (kind == COMBINE_STORE) {
+    for (int i = threadIdx.x; i < hidden; i += blockDim.x) out[i] = sum[i];
+    return;
+  }
+  float inv = 1.f, next = 0.f;
   if (kind == COMBINE_ADD_RMS) {
     ss = block_sum(ss, sum + hidden);
     inv = 1.0f / sqrtf(ss / (float)hidden + eps);
@@ -689,6 +734,15 @@ __global__ __launch_bounds__(1024) void moe_combine_kernel(float* __restrict__ r
     const float v = out[i] + (kind == COMBINE_ADD_RMS ? sum[i] * inv * to_float(norm_w[i]) : sum[i]);
     out[i] = v;
     if (rounded) rounded[(int64_t)t * hidden + i] = (bf16)v;       // the stream as the next sublayer reads it
+    sum[i] = v;                                                    // (this thread's own element)
+    next = fmaf(v, v, next);
+  }
+  if (more.normed == nullptr) return;
+  const float next_inv = 1.0f / sqrtf(block_sum(next, sum + hidden) / (float)hidden + more.next_eps);
+  for (int i = threadIdx.x; i < hidden; i += blockDim.x) {
+    const float v = sum[i] * next_inv * more.next_weight[i];
+    if (more.normed_f32) ((float*)more.normed)[(int64_t)t * hidden + i] = v;
+    else ((bf16*)more.normed)[(int64_t)t * hidden + i] = (bf16)v;
   }
 }
 
@@ -709,11 +763,9 @@ LRS_API int lrs_moe_max_tiles(int pairs, int experts) {
 }
 
 static int check_rule(const char* who, int kind, int groups, int keep, float scale, int experts, int top) {
-  LRS_REQUIRE(kind >= ROUTE_SOFTMAX_CHOSEN && kind <= ROUTE_SIGMOID_SCORES, "%s: unknown routing rule %d", who, kind);
-  if (kind == ROUTE_SOFTMAX_CHOSEN) {
-    LRS_REQUIRE(groups == 0, "%s: groups of experts come with the sigmoid rule only", who);
-    return 0;
-  }
+  LRS_REQUIRE(kind >= ROUTE_SOFTMAX_CHOSEN && kind <= ROUTE_SOFTMAX_SCORES, "%s: unknown routing rule %d", who, kind);
+  LRS_REQUIRE(groups == 0 || kind == ROUTE_SIGMOID || kind == ROUTE_SIGMOID_SCORES, "%s: groups of experts come with the sigmoid rules only", who);
+  if (kind == ROUTE_SOFTMAX_CHOSEN) return 0;
   LRS_REQUIRE(scale > 0.f, "%s: the weights' scale must be positive", who);
   if (groups > 0) {
     LRS_REQUIRE(experts % groups == 0 && keep > 0 && keep <= groups, "%s: %d experts do not form %d equal groups of which %d are kept", who, experts, groups, keep);
@@ -733,29 +785,31 @@ LRS_API int lrs_moe_route(const float* logits, int ld, const float* bias, int* i
   return lrs_check_launch("moe_route");
 }
 
-LRS_API int lrs_moe_align(const int* ids, int pairs, int experts, int* sorted, int capacity, int* place, int* tile_expert,
+// experts: those that have matrices; identity: how many ids behind theirs stand for the token itself.
+LRS_API int lrs_moe_align(const int* ids, int pairs, int experts, int identity, int* sorted, int capacity, int* place, int* tile_expert,
                           int max_tiles, void* stream) {
-  LRS_REQUIRE(pairs > 0 && experts > 0, "moe_align: bad sizes pairs=%d experts=%d", pairs, experts);
+  LRS_REQUIRE(pairs > 0 && experts > 0 && identity >= 0, "moe_align: bad sizes pairs=%d experts=%d identity=%d", pairs, experts, identity);
   const int tile = lrs_moe_tile_rows(pairs, experts);
   LRS_REQUIRE(max_tiles >= lrs_moe_max_tiles(pairs, experts), "moe_align: %d tiles may not hold %d pairs of %d experts", max_tiles, pairs, experts);
   LRS_REQUIRE(capacity >= max_tiles * tile, "moe_align: the sorted list holds %d rows, %d tiles need %d", capacity, max_tiles, max_tiles * tile);
   const size_t lds = (size_t)(3 * experts + 1) * sizeof(int);
   LRS_REQUIRE(lds <= 48 * 1024, "moe_align: %d experts are too many", experts);
-  moe_align_kernel<<<1, 1024, lds, (hipStream_t)stream>>>(ids, pairs, experts, tile, sorted, capacity, place, tile_expert, max_tiles);
+  moe_align_kernel<<<1, 1024, lds, (hipStream_t)stream>>>(ids, pairs, experts, identity, tile, sorted, capacity, place, tile_expert, max_tiles);
   return lrs_check_launch("moe_align");
 }
 
 LRS_API int lrs_moe_route_align(const float* logits, int ld, const float* bias, int* ids, float* weights, int tokens, int experts,
-                                int top, int* sorted, int capacity, int* place, int* tile_expert, int max_tiles, int rule, int groups, int keep,
+                                int identity, int top, int* sorted, int capacity, int* place, int* tile_expert, int max_tiles, int rule, int groups, int keep,
                                 float scale, void* stream) {
-  if (int rc = check_rule("moe_route_align", rule, groups, keep, scale, experts, top)) return rc;
-  LRS_REQUIRE(tokens > 0 && tokens <= 256 && experts > 0 && top > 0 && top <= experts, "moe_route_align: bad sizes tokens=%d experts=%d top=%d", tokens, experts, top);
-  LRS_REQUIRE(experts <= WAVE * ROUTE_MAX_PER_LANE && ld >= experts, "moe_route_align: at most %d experts in rows of at least as many logits", WAVE * ROUTE_MAX_PER_LANE);
+  if (int rc = check_rule("moe_route_align", rule, groups, keep, scale, experts + identity, top)) return rc;
+  LRS_REQUIRE(tokens > 0 && tokens <= 256 && experts > 0 && identity >= 0 && top > 0 && top <= experts + identity,
+              "moe_route_align: bad sizes tokens=%d experts=%d identity=%d top=%d", tokens, experts, identity, top);
+  LRS_REQUIRE(experts + identity <= WAVE * ROUTE_MAX_PER_LANE && ld >= experts + identity, "moe_route_align: at most %d experts in rows of at least as many logits", WAVE * ROUTE_MAX_PER_LANE);
   const int pairs = tokens * top, tile = lrs_moe_tile_rows(pairs, experts);
   LRS_REQUIRE(max_tiles >= lrs_moe_max_tiles(pairs, experts), "moe_route_align: %d tiles may not hold %d pairs of %d experts", max_tiles, pairs, experts);
   LRS_REQUIRE(capacity >= max_tiles * tile, "moe_route_align: the sorted list holds %d rows, %d tiles need %d", capacity, max_tiles, max_tiles * tile);
   const size_t lds = (size_t)(3 * experts + 1) * sizeof(int);
-  moe_route_align_kernel<<<1, 1024, lds, (hipStream_t)stream>>>(logits, ld, bias, ids, weights, tokens, experts, top, tile, sorted, capacity, place,
+  moe_route_align_kernel<<<1, 1024, lds, (hipStream_t)stream>>>(logits, ld, bias, ids, weights, tokens, experts, identity, top, tile, sorted, capacity, place,
                                                                 tile_expert, max_tiles, RouteRule{rule, groups, keep, scale});
   return lrs_check_launch("moe_route_align");
 }
@@ -822,22 +876,29 @@ LRS_API int lrs_moe_experts(void* out, int out_dtype, int ldc, const void* a, co
 
 // residual [tokens, hidden] += (norm of) sum_c weights[t, c] * rows[place[t, c]]; norm_w null: the plain sum; rounded:
 // where the updated rows are left in bfloat16 as well, or null.  weights null: every choice counts once.  extra [tokens, hidden]
-// (or null): rows added to the sum before the norm.
+// (or null): rows added to the sum before the norm.  store: residual = the sum (no norm).  self [tokens, hidden] (self_dtype, rows of
+// self_stride; or null): what a choice with place -1 stands for.  normed (normed_dtype, or null; with an RMS norm): the RMS norm of
+// the updated rows, times next_weight (float32).
 LRS_API int lrs_moe_combine(float* residual, const float* rows, int tokens, int hidden, const int* place, const float* weights,
                             int top, const void* norm_w, int norm_dtype, float eps, void* rounded, int layer_norm, float alpha,
-                            const float* extra, void* stream) {
+                            const float* extra, int store, const void* self, int self_dtype, int self_stride, const float* next_weight,
+                            float next_eps, void* normed, int normed_dtype, void* stream) {
   // layer_norm (with a norm weight): the stream becomes the layer norm of alpha * stream + sum, instead of taking the sum's RMS norm on top
   LRS_REQUIRE(tokens > 0 && hidden > 0 && top > 0, "moe_combine: bad sizes tokens=%d hidden=%d top=%d", tokens, hidden, top);
   LRS_REQUIRE(!norm_w || eps > 0.f, "moe_combine: eps must be positive");
   LRS_REQUIRE(!layer_norm || norm_w, "moe_combine: a layer norm needs its weight");
-  const int kind = !norm_w ? COMBINE_ADD : layer_norm ? COMBINE_LAYERNORM : COMBINE_ADD_RMS;
+  LRS_REQUIRE(!store || (!norm_w && !rounded), "moe_combine: what is stored is the plain sum");
+  LRS_REQUIRE(!self || self_stride >= hidden, "moe_combine: rows of %d hold fewer than %d values", self_stride, hidden);
+  LRS_REQUIRE(!normed || (norm_w && !layer_norm && next_weight && next_eps > 0.f), "moe_combine: the norm that follows comes with an RMS norm, its weight and a positive eps");
+  const CombineMore more{self, self_dtype == LRS_F32, self_stride, next_weight, next_eps, normed, normed_dtype == LRS_F32};
+  const int kind = store ? COMBINE_STORE : !norm_w ? COMBINE_ADD : layer_norm ? COMBINE_LAYERNORM : COMBINE_ADD_RMS;
   const size_t lds = (size_t)(hidden + 16 + 2 * top) * sizeof(float);
   LRS_REQUIRE(lds <= 64 * 1024, "moe_combine: a width of %d with %d choices is too much", hidden, top);
   hipStream_t s = (hipStream_t)stream;
   const int threads = hidden >= 2048 ? 1024 : 256;
   if (norm_w && norm_dtype == LRS_BF16)
-    moe_combine_kernel<bf16><<<tokens, threads, lds, s>>>(residual, rows, hidden, place, weights, top, (const bf16*)norm_w, eps, (bf16*)rounded, kind, alpha, extra);
+    moe_combine_kernel<bf16><<<tokens, threads, lds, s>>>(residual, rows, hidden, place, weights, top, (const bf16*)norm_w, eps, (bf16*)rounded, kind, alpha, extra, more);
   else
-    moe_combine_kernel<float><<<tokens, threads, lds, s>>>(residual, rows, hidden, place, weights, top, (const float*)norm_w, eps, (bf16*)rounded, kind, alpha, extra);
+    moe_combine_kernel<float><<<tokens, threads, lds, s>>>(residual, rows, hidden, place, weights, top, (const float*)norm_w, eps, (bf16*)rounded, kind, alpha, extra, more);
   return lrs_check_launch("moe_combine");
 }

@@ -10,7 +10,7 @@
 //   sigmoid_gate    out[t, c] *= sigmoid(gate[t, c / group]): the output gate of the heads, a value a column or one a head;
 //   axpby           out = alpha * a + beta * b over float32 rows: sums of sublayer outputs and the scaled residual add,
 //                   optionally followed by the RMS norm of the new rows (the next layer's input) in the same pass;
-//   activation      out = act(x) elementwise: exact (erf) gelu, tanh gelu, silu, relu.
+//   activation      out = act(x) elementwise: exact (erf) gelu, tanh gelu, silu, relu, the square of relu.
 #include "value_pages.h"
 
 namespace {
@@ -278,13 +278,14 @@ __global__ __launch_bounds__(256) void axpby_norm_vec_kernel(float* __restrict__
   }
 }
 
-enum { ACT_GELU_ERF = 0, ACT_GELU_TANH = 1, ACT_SILU = 2, ACT_RELU = 3 };
+enum { ACT_GELU_ERF = 0, ACT_GELU_TANH = 1, ACT_SILU = 2, ACT_RELU = 3, ACT_RELU_SQUARE = 4 };
 
 __device__ __forceinline__ float activate(float x, int kind) {
   switch (kind) {
     case ACT_GELU_ERF: return 0.5f * x * (1.f + erff(x * 0.70710678118654752f));
     case ACT_GELU_TANH: return 0.5f * x * (1.f + tanhf(0.7978845608028654f * (x + 0.044715f * x * x * x)));
     case ACT_SILU: return x / (1.f + expf(-x));
+    case ACT_RELU_SQUARE: return x > 0.f ? x * x : 0.f;
     default: return fmaxf(x, 0.f);
   }
 }
@@ -295,6 +296,19 @@ __global__ void activation_kernel(T* __restrict__ out, const T* __restrict__ x, 
   if (e < count) out[e] = from_float<T>(activate(to_float(x[e]), kind));
 }
 
+// The same 16 bytes at a time, for counts that are a multiple of that.
+template <typename T, int KIND>
+__global__ __launch_bounds__(256) void activation_vec_kernel(T* __restrict__ out, const T* __restrict__ x, int64_t pieces) {
+  constexpr int RUN = 16 / sizeof(T);
+  typedef T vec __attribute__((ext_vector_type(RUN)));
+  const int64_t e = (int64_t)blockIdx.x * 256 + threadIdx.x;
+  if (e >= pieces) return;
+  vec v = ((const vec*)x)[e];
+#pragma unroll
+  for (int i = 0; i < RUN; ++i) v[i] = from_float<T>(activate(to_float(v[i]), KIND));
+  ((vec*)out)[e] = v;
+}
+
 }  // namespace
 
 // qkv [tokens, row_stride] in dtype: q (nq*d) | k (nkv*d) | v (nkv*dv) | anything else.  q_weight [nq*d], k_weight [nkv*d]
@@ -302,17 +316,17 @@ __global__ void activation_kernel(T* __restrict__ out, const T* __restrict__ x, 
 // token's key and value are not stored).  bias (float32 [nq*d + nkv*d + nkv*dv], or null) is added to q, k and v as they are read.
 // every > 0: queries are multiplied by 1 + coef * ln(floor((positions[t] + 1) / every) + 1).  first_values [tokens, nkv*dv] in
 // dtype, or null: value_mix null leaves the step's values there, value_mix given (one float32 on the device) mixes
-// v <- (1 - value_mix) v + value_mix first_values.
+// v <- (1 - value_mix) v + value_mix first_values.  nq may be 0 (rows that begin with the key heads: queries that stay as they are).
 LRS_API int lrs_qkv_norm_prep(void* qkv, int dtype, int tokens, int row_stride, int nq, int nkv, int d, int dv, const float* q_weight,
                               const float* k_weight, float eps, const float* cosv, const float* sinv, int rot_half, void* k_pages,
                               void* v_pages, const int* slots, int page_size, const float* bias, const int* positions, float coef, int every,
                               void* first_values, const float* value_mix, void* stream) {
-  LRS_REQUIRE(tokens > 0 && nq > 0 && nkv > 0 && d > 0 && dv > 0, "qkv_norm_prep: bad sizes tokens=%d nq=%d nkv=%d d=%d dv=%d", tokens, nq, nkv, d, dv);
+  LRS_REQUIRE(tokens > 0 && nq >= 0 && nkv > 0 && d > 0 && dv > 0, "qkv_norm_prep: bad sizes tokens=%d nq=%d nkv=%d d=%d dv=%d", tokens, nq, nkv, d, dv);
   LRS_REQUIRE(row_stride >= nq * d + nkv * d + nkv * dv, "qkv_norm_prep: rows of %d hold fewer than q, k and v", row_stride);
   LRS_REQUIRE(rot_half >= 0 && 2 * rot_half <= d, "qkv_norm_prep: rotary width %d exceeds head_dim %d", 2 * rot_half, d);
   LRS_REQUIRE(rot_half == 0 || (cosv && sinv), "qkv_norm_prep: rotation asked for without tables");
   LRS_REQUIRE((q_weight == nullptr) == (k_weight == nullptr), "qkv_norm_prep: q and k norm weights must come together");
-  LRS_REQUIRE(!q_weight || eps > 0.f, "qkv_norm_prep: eps must be positive");
+  LRS_REQUIRE(!q_weight || (eps > 0.f && nq > 0), "qkv_norm_prep: eps must be positive, and norms come with query heads");
   LRS_REQUIRE(k_pages && v_pages && slots && page_size > 0, "qkv_norm_prep: cache write needs pages, slots and a page size");
   LRS_REQUIRE(every >= 0 && (every == 0 || positions), "qkv_norm_prep: a temperature needs a positive step and the positions");
   LRS_REQUIRE(!value_mix || first_values, "qkv_norm_prep: nothing to mix the values with");
@@ -384,9 +398,28 @@ LRS_API int lrs_axpby(float* out, const float* a, float alpha, const float* b, f
 }
 
 LRS_API int lrs_activation(void* out, const void* x, int dtype, int64_t count, int kind, void* stream) {
-  LRS_REQUIRE(count > 0 && kind >= 0 && kind <= 3, "activation: bad arguments count=%lld kind=%d", (long long)count, kind);
+  LRS_REQUIRE(count > 0 && kind >= 0 && kind <= ACT_RELU_SQUARE, "activation: bad arguments count=%lld kind=%d", (long long)count, kind);
   const unsigned blocks = (unsigned)((count + 255) / 256);
   hipStream_t s = (hipStream_t)stream;
+  const int run = dtype == LRS_F32 ? 4 : 8;
+  if ((dtype == LRS_F32 || dtype == LRS_BF16) && count % run == 0 && ((uintptr_t)out | (uintptr_t)x) % 16 == 0) {
+    const int64_t pieces = count / run;
+    const unsigned grid = (unsigned)((pieces + 255) / 256);
+#define VEC(KIND)                                                                                                               \
+  case KIND:                                                                                                                    \
+    if (dtype == LRS_F32) activation_vec_kernel<float, KIND><<<grid, 256, 0, s>>>((float*)out, (const float*)x, pieces);        \
+    else activation_vec_kernel<bf16, KIND><<<grid, 256, 0, s>>>((bf16*)out, (const bf16*)x, pieces);                            \
+    break
+    switch (kind) {
+      VEC(ACT_GELU_ERF);
+      VEC(ACT_GELU_TANH);
+      VEC(ACT_SILU);
+      VEC(ACT_RELU);
+      VEC(ACT_RELU_SQUARE);
+    }
+#undef VEC
+    return lrs_check_launch("activation");
+  }
   if (dtype == LRS_F32) activation_kernel<float><<<blocks, 256, 0, s>>>((float*)out, (const float*)x, count, kind);
   else if (dtype == LRS_BF16) activation_kernel<bf16><<<blocks, 256, 0, s>>>((bf16*)out, (const bf16*)x, count, kind);
   else return lrs_fail("activation: unknown dtype %d", dtype);

@@ -124,7 +124,7 @@ _SIGNATURES = {
                                             c_void_p, c_int64, c_void_p]),
     "lrs_norm_begin_parts": (c_int, [c_int]),
     "lrs_attention": (c_int, [c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p,
-                              c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_int, c_void_p, c_float, c_void_p, c_int, c_void_p, c_void_p]),
+                              c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_int, c_void_p, c_float, c_void_p, c_int, c_void_p, c_int, c_void_p]),
     "lrs_qkv_norm_prep": (c_int, [c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_float, c_void_p, c_void_p,
                                   c_int, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_float, c_int, c_void_p, c_void_p, c_void_p]),
     "lrs_gated_norm_add": (c_int, [c_void_p, c_void_p, c_void_p, c_int, c_int, c_void_p, c_void_p, c_float, c_int, c_int, c_void_p, c_float,
@@ -152,10 +152,10 @@ _SIGNATURES = {
                         c_void_p, c_void_p, c_void_p, c_void_p, c_void_p]),
     "lrs_attention_decode": (c_int, [c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_void_p,
                                      c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_int, c_int, c_int, c_int,
-                                     c_void_p, c_void_p, c_int, c_float, c_void_p, c_void_p, c_int, c_void_p, c_float, c_void_p, c_int, c_int, c_void_p, c_void_p]),
+                                     c_void_p, c_void_p, c_int, c_float, c_void_p, c_void_p, c_int, c_void_p, c_float, c_void_p, c_int, c_int, c_void_p, c_int, c_void_p]),
     "lrs_attention_prefill": (c_int, [c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p,
                                       c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_int,
-                                      c_int, c_int, c_void_p, c_void_p, c_int, c_void_p, c_int, c_float, c_void_p, c_void_p, c_void_p, c_float, c_void_p, c_int, c_int, c_void_p, c_void_p]),
+                                      c_int, c_int, c_void_p, c_void_p, c_int, c_void_p, c_int, c_float, c_void_p, c_void_p, c_void_p, c_float, c_void_p, c_int, c_int, c_void_p, c_int, c_void_p]),
     "lrs_attention_prefill_prepares": (c_int, [c_int]),
     "lrs_compute_units": (c_int, []),
     "lrs_gemm_lines_width": (c_int, [c_int, c_int, c_int]),
@@ -177,24 +177,26 @@ _SIGNATURES = {
     "lrs_moe_tile_rows": (c_int, [c_int, c_int]),
     "lrs_moe_max_tiles": (c_int, [c_int, c_int]),
     "lrs_moe_route": (c_int, [c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_void_p]),
-    "lrs_moe_route_align": (c_int, [c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_void_p, c_int, c_void_p, c_void_p, c_int,
+    "lrs_moe_route_align": (c_int, [c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_void_p, c_int, c_void_p, c_void_p, c_int,
                                     c_int, c_int, c_int, c_float, c_void_p]),
-    "lrs_moe_align": (c_int, [c_void_p, c_int, c_int, c_void_p, c_int, c_void_p, c_void_p, c_int, c_void_p]),
+    "lrs_moe_align": (c_int, [c_void_p, c_int, c_int, c_int, c_void_p, c_int, c_void_p, c_void_p, c_int, c_void_p]),
     "lrs_moe_experts": (c_int, [c_void_p, c_int, c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_int, c_int, c_int,
                                 c_int, c_int, c_void_p, c_float, c_float, c_void_p]),
     "lrs_layernorm": (c_int, [c_void_p, c_int, c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_float, c_void_p]),
     "lrs_scale_add_layernorm": (c_int, [c_void_p, c_void_p, c_float, c_void_p, c_int, c_int, c_int, c_float, c_void_p, c_void_p]),
     "lrs_soft_cap": (c_int, [c_void_p, c_int64, c_float, c_void_p]),
     "lrs_latent_prep": (c_int, [c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p, c_int, c_float, c_void_p, c_void_p,
-                                c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_int, c_void_p]),
+                                c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_int, c_int, c_void_p, c_void_p, c_int, c_void_p]),
     "lrs_latent_attention_groups_takes": (c_int, [c_int, c_int, c_int]),
     "lrs_latent_attention_groups": (c_int, [c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p,
                                             c_int, c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_int,
                                             c_void_p, c_void_p, c_void_p]),
-    "lrs_head_gemm": (c_int, [c_void_p, c_int, c_int, c_void_p, c_int, c_int, c_void_p, c_int64, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p]),
+    "lrs_head_gemm": (c_int, [c_void_p, c_int, c_int, c_void_p, c_int, c_int, c_void_p, c_int64, c_int, c_int, c_int, c_int, c_int, c_int, c_int,
+                              c_void_p, c_void_p, c_void_p, c_int, c_void_p]),
     "lrs_latent_attention": (c_int, [c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_int,
                                      c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_void_p]),
-    "lrs_moe_combine": (c_int, [c_void_p, c_void_p, c_int, c_int, c_void_p, c_void_p, c_int, c_void_p, c_int, c_float, c_void_p, c_int, c_float, c_void_p, c_void_p]),
+    "lrs_moe_combine": (c_int, [c_void_p, c_void_p, c_int, c_int, c_void_p, c_void_p, c_int, c_void_p, c_int, c_float, c_void_p, c_int, c_float, c_void_p,
+                                c_int, c_void_p, c_int, c_int, c_void_p, c_float, c_void_p, c_int, c_void_p]),
 }
 
 
@@ -990,12 +992,12 @@ def _sinks(sinks: torch.Tensor | None, nq: int, who: str):
 
 
 def _distance(distance: torch.Tensor | None, nq: int, who: str):
-    """Address of a bias by distance, float32 [2, nq]: the heads' rates, then their reaches (a score at distance x loses
-    rate * ln(1 + reach * x)); None: no bias."""
+    """(address, form) of a bias by distance: float32 [2, nq], the heads' rates and then their reaches (a score at distance x loses
+    rate * ln(1 + reach * x)), or [nq], their rates (it loses rate * x); None: no bias."""
     if distance is None:
-        return None
-    _need(distance.dtype == torch.float32 and distance.shape == (2, nq) and distance.is_contiguous(), f"{who}: distance must be float32 [2, {nq}]")
-    return _dev(distance, "distance")
+        return None, 0
+    _need(distance.dtype == torch.float32 and distance.shape in ((2, nq), (nq,)) and distance.is_contiguous(), f"{who}: distance must be float32 [2, {nq}] or [{nq}]")
+    return _dev(distance, "distance"), int(distance.dim() == 1)
 
 
 def attention(out: torch.Tensor, q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor, block_table: torch.Tensor,
@@ -1007,7 +1009,9 @@ def attention(out: torch.Tensor, q: torch.Tensor, k_pages: torch.Tensor, v_pages
     sinks (float32 [nq]): the softmax's denominator of head h has one more term exp(sinks[h]), without key or value.
     softcap > 0: the scaled scores pass softcap * tanh(score / softcap) before the softmax.
     gates ([T, nq], rows of any stride): head h's output is multiplied by sigmoid(gates[t, h]).
-    distance (float32 [2, nq]): head h's score of a key x positions back loses distance[0, h] * ln(1 + distance[1, h] * x)."""
+    distance (float32 [2, nq]): head h's score of a key x positions back loses distance[0, h] * ln(1 + distance[1, h] * x); float32
+    [nq]: it loses distance[h] * x.  A negative window stands for chunks of -window positions counted from position 0: a token sees
+    those of its own chunk (here and in every function that takes a window)."""
     tokens = out.shape[0]
     _need(k_pages.dim() == 4 and v_pages.dim() == 4 and k_pages.is_contiguous() and v_pages.is_contiguous(), "attention: pages must be contiguous")
     _, nkv, page_size, d = k_pages.shape
@@ -1022,7 +1026,7 @@ def attention(out: torch.Tensor, q: torch.Tensor, k_pages: torch.Tensor, v_pages
         _dev(out, "out"), _rows(out, "out"), _dev(q, "q"), _rows(q, "q"), _dev(k_pages, "k_pages"), _dev(v_pages, "v_pages"),
         _dev(block_table, "block_table"), block_table.stride(0), _dev(token_request, "token_request"), _dev(positions, "positions"),
         dtype_code(q.dtype), tokens, nq, nkv, d, dv, page_size, scale, window, keep_first, _sinks(sinks, nq, "attention"), float(softcap),
-        *_gates(gates, tokens, nq, q.dtype, "attention"), _distance(distance, nq, "attention"), _stream())
+        *_gates(gates, tokens, nq, q.dtype, "attention"), *_distance(distance, nq, "attention"), _stream())
 
 
 def qkv_norm_prep(qkv: torch.Tensor, nq: int, nkv: int, d: int, dv: int, q_weight, k_weight, eps: float, cos, sin,
@@ -1033,7 +1037,7 @@ def qkv_norm_prep(qkv: torch.Tensor, nq: int, nkv: int, d: int, dv: int, q_weigh
     square of the whole part (all heads at once) and multiplied by a weight per column (float32 [nq*d], [nkv*d]; None: no
     norm), the first 2 * cos.shape[1] dims of every head rotated; q in place, k and v into the pages.  On the way: `bias` (float32,
     a value per column of q, k and v) is added first; `temperature` (coef, every) multiplies the queries of a token at position p
-    by 1 + coef * ln(floor((p + 1) / every) + 1); `first_values` [T, nkv*dv] receives the step's values, or, with `value_mix`
+    by 1 + coef * ln(floor((p + 1) / every) + 1); nq may be 0 (rows that begin with the key heads); `first_values` [T, nkv*dv] receives the step's values, or, with `value_mix`
     (float32 [1] on the device), is what they are mixed with: v <- (1 - value_mix) v + value_mix first_values."""
     tokens = qkv.shape[0]
     stride = _rows(qkv, "qkv")
@@ -1173,11 +1177,11 @@ def axpby(out: torch.Tensor, a: torch.Tensor, alpha: float, b: torch.Tensor, bet
             0 if norm_weight is None else dtype_code(normed.dtype), _stream())
 
 
-ACTIVATIONS = {"gelu": 0, "gelu_tanh": 1, "silu": 2, "relu": 3}
+ACTIVATIONS = {"gelu": 0, "gelu_tanh": 1, "silu": 2, "relu": 3, "relu_squared": 4}
 
 
 def activation(out: torch.Tensor, x: torch.Tensor, kind: str) -> None:
-    """out = act(x) elementwise (out may be x): "gelu" (0.5 x (1 + erf(x / sqrt 2))), "gelu_tanh", "silu", "relu"."""
+    """out = act(x) elementwise (out may be x): "gelu" (0.5 x (1 + erf(x / sqrt 2))), "gelu_tanh", "silu", "relu", "relu_squared"."""
     _need(kind in ACTIVATIONS, f"activation: unknown kind {kind!r}; known: {', '.join(ACTIVATIONS)}")
     _need(out.shape == x.shape and out.dtype == x.dtype and out.is_contiguous() and x.is_contiguous() and x.numel() > 0,
           "activation: out and x must be contiguous, of one shape and dtype")
@@ -1243,7 +1247,6 @@ def attention_decode(out: torch.Tensor, q: torch.Tensor, k_pages: torch.Tensor, 
         _need(part_ml is not None and part_ml.dtype == torch.float32 and part_ml.is_contiguous() and part_ml.numel() >= tokens * nq * slots * 2, "attention_decode: part_ml too small")
     fused = [0, None, None, 0, 0.0, None, None, 0]
     if prepare is not None:
-        _need(distance is None, "attention_decode: a bias by distance needs prepared heads")
         _need(dv == d, "attention_decode: heads whose values are narrower than their keys must come prepared")
         _need(decode_prepare_supported(d, prepare.cos is not None), f"attention_decode: cannot rotate heads of {d} dims itself")
         _need((prepare.q_weight is None) == (prepare.k_weight is None), "attention_decode: q and k norm weights must come together")
@@ -1264,7 +1267,7 @@ def attention_decode(out: torch.Tensor, q: torch.Tensor, k_pages: torch.Tensor, 
         _dev(token_request, "token_request"), _dev(positions, "positions"), tokens,
         block_table.shape[1] * page_size if max_context is None else max_context, nq, nkv, d, page_size, scale, window, keep_first, splits,
         form, *fused, _sinks(sinks, nq, "attention_decode"), float(softcap), *_gates(gates, tokens, nq, q.dtype, "attention_decode"), dv,
-        _distance(distance, nq, "attention_decode"), _stream())
+        *_distance(distance, nq, "attention_decode"), _stream())
 
 
 def attention_prefill(out: torch.Tensor, q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor, block_table: torch.Tensor,
@@ -1324,7 +1327,7 @@ def attention_prefill(out: torch.Tensor, q: torch.Tensor, k_pages: torch.Tensor,
         block_table.shape[1] * page_size if max_context is None else max_context, nq, nkv, d, page_size, scale, window, keep_first,
         tokens, splits, None if slots == 1 else _dev(part_o, "part_o"), None if slots == 1 else _dev(part_ml, "part_ml"), *fused,
         _sinks(sinks, nq, "attention_prefill"), float(softcap), *_gates(gates, tokens, nq, q.dtype, "attention_prefill"), dv,
-        _distance(distance, nq, "attention_prefill"), _stream())
+        *_distance(distance, nq, "attention_prefill"), _stream())
 
 
 def attention_prefill_prepares(d: int) -> bool:
@@ -1611,13 +1614,14 @@ class RouteRule:
     softmax over the chosen (logit + bias) alone.  kind "sigmoid": scores s = sigmoid(logit); the largest (s + bias) are
     chosen (the bias takes part in the choice only), weighted by the chosen s over their sum (+ 1e-20), times `scale`; with
     `groups` the experts form that many equal groups of neighbours, a group scores the sum of its two largest (s + bias),
-    and only experts of the `keep` best groups can be chosen."""
+    and only experts of the `keep` best groups can be chosen.  kind "sigmoid_scores": chosen as under "sigmoid", weighted by the
+    chosen s themselves, times `scale`; "softmax_scores": the same with s = softmax(logits) over all of them (no groups)."""
     kind: str = "softmax_chosen"
     groups: int = 0
     keep: int = 0
     scale: float = 1.0
 
-    KINDS = ("softmax_chosen", "sigmoid", "sigmoid_scores")     # the last: chosen as under "sigmoid", weighted by the chosen s themselves (times scale)
+    KINDS = ("softmax_chosen", "sigmoid", "sigmoid_scores", "softmax_scores")
 
     def words(self) -> tuple:
         _need(self.kind in self.KINDS, f"unknown routing rule {self.kind!r}; known: {', '.join(self.KINDS)}")
@@ -1639,16 +1643,17 @@ def moe_route(logits: torch.Tensor, bias: torch.Tensor | None, ids: torch.Tensor
             _dev(weights, "weights"), tokens, experts, top, *rule.words(), _stream())
 
 
-def moe_align(ids: torch.Tensor, experts: int, sorted_pairs: torch.Tensor, place: torch.Tensor, tile_expert: torch.Tensor) -> None:
+def moe_align(ids: torch.Tensor, experts: int, sorted_pairs: torch.Tensor, place: torch.Tensor, tile_expert: torch.Tensor, identity: int = 0) -> None:
     """Sorts the (token, choice) pairs of ids [T, top] by expert: sorted_pairs [tiles * tile rows] (pair index, -1 in the
-    rows that pad an expert's run), place [T * top] (the row of each pair), tile_expert [tiles] (-1: tile not in use)."""
+    rows that pad an expert's run), place [T * top] (the row of each pair), tile_expert [tiles] (-1: tile not in use).
+    identity: ids experts .. experts + identity - 1 stand for the token itself; such a pair has no row (place -1)."""
     pairs, tiles = ids.numel(), tile_expert.numel()
     tile = moe_tile_rows(pairs, experts)
     for name, t in (("ids", ids), ("sorted_pairs", sorted_pairs), ("place", place), ("tile_expert", tile_expert)):
         _need(t.dtype == torch.int32 and t.is_contiguous(), f"moe_align: {name} must be contiguous int32")
     _need(tiles >= moe_max_tiles(pairs, experts) and sorted_pairs.numel() >= tiles * tile and place.numel() >= pairs,
           "moe_align: the lists are too short for the step")
-    _launch("lrs_moe_align", _dev(ids, "ids"), pairs, experts, _dev(sorted_pairs, "sorted_pairs"), sorted_pairs.numel(), _dev(place, "place"),
+    _launch("lrs_moe_align", _dev(ids, "ids"), pairs, experts, identity, _dev(sorted_pairs, "sorted_pairs"), sorted_pairs.numel(), _dev(place, "place"),
             _dev(tile_expert, "tile_expert"), tiles, _stream())
 
 
@@ -1656,13 +1661,13 @@ ROUTE_ALIGN_TOKENS = 32      # steps up to which one workgroup both chooses and 
 
 
 def moe_route_align(logits: torch.Tensor, bias: torch.Tensor | None, ids: torch.Tensor, weights: torch.Tensor, sorted_pairs: torch.Tensor,
-                    place: torch.Tensor, tile_expert: torch.Tensor, rule: RouteRule = DEFAULT_RULE) -> None:
-    """moe_route() and moe_align() as one launch, for steps of at most ROUTE_ALIGN_TOKENS tokens."""
+                    place: torch.Tensor, tile_expert: torch.Tensor, rule: RouteRule = DEFAULT_RULE, identity: int = 0) -> None:
+    """moe_route() and moe_align() as one launch, for steps of at most ROUTE_ALIGN_TOKENS tokens.  logits [T, experts + identity]."""
     tokens, top = ids.shape
-    experts, pairs, tiles = logits.shape[1], ids.numel(), tile_expert.numel()
+    experts, pairs, tiles = logits.shape[1] - identity, ids.numel(), tile_expert.numel()
     _need(tokens <= ROUTE_ALIGN_TOKENS, f"moe_route_align: at most {ROUTE_ALIGN_TOKENS} tokens")
     _need(logits.dtype == torch.float32 and logits.shape[0] >= tokens and logits.stride(1) == 1, "moe_route_align: logits must be float32 [T, E]")
-    _need(bias is None or (bias.dtype == torch.float32 and bias.numel() == experts and bias.is_contiguous()), "moe_route_align: bias must hold E float32 values")
+    _need(bias is None or (bias.dtype == torch.float32 and bias.numel() == experts + identity and bias.is_contiguous()), "moe_route_align: bias must hold E float32 values")
     _need(ids.dtype == torch.int32 and ids.is_contiguous() and weights.dtype == torch.float32 and weights.is_contiguous()
           and weights.shape == ids.shape, "moe_route_align: ids must be int32 [T, top] and weights float32 [T, top]")
     for name, t in (("sorted_pairs", sorted_pairs), ("place", place), ("tile_expert", tile_expert)):
@@ -1670,7 +1675,7 @@ def moe_route_align(logits: torch.Tensor, bias: torch.Tensor | None, ids: torch.
     _need(tiles >= moe_max_tiles(pairs, experts) and sorted_pairs.numel() >= tiles * moe_tile_rows(pairs, experts) and place.numel() >= pairs,
           "moe_route_align: the lists are too short for the step")
     _launch("lrs_moe_route_align", _dev(logits, "logits"), logits.stride(0), None if bias is None else _dev(bias, "bias"), _dev(ids, "ids"),
-            _dev(weights, "weights"), tokens, experts, top, _dev(sorted_pairs, "sorted_pairs"), sorted_pairs.numel(), _dev(place, "place"),
+            _dev(weights, "weights"), tokens, experts, identity, top, _dev(sorted_pairs, "sorted_pairs"), sorted_pairs.numel(), _dev(place, "place"),
             _dev(tile_expert, "tile_expert"), tiles, *rule.words(), _stream())
 
 
@@ -1704,12 +1709,15 @@ def moe_experts(out: torch.Tensor, a: torch.Tensor, w: torch.Tensor, sorted_pair
 
 def moe_combine(residual: torch.Tensor, rows: torch.Tensor, place: torch.Tensor, weights: torch.Tensor | None, norm_weight: torch.Tensor | None,
                 eps: float = 0.0, rounded: torch.Tensor | None = None, layer_norm_alpha: float | None = None, top: int | None = None,
-                extra: torch.Tensor | None = None) -> None:
+                extra: torch.Tensor | None = None, store: bool = False, itself: torch.Tensor | None = None,
+                next_norm: tuple | None = None) -> None:
     """residual [T, H] += sum over a token's choices of weights[t, c] * rows[place[t, c]]; with norm_weight: the RMS
     norm (weight norm_weight, eps) of that sum instead of the sum itself; with layer_norm_alpha as well: residual becomes
     the layer norm (norm_weight, eps) of layer_norm_alpha * residual + sum.  rounded: bfloat16 [T, H] that receives the
     updated rows as well.  weights None (then `top` says how many choices a token has): every choice counts once.  extra
-    (float32 [T, H]): rows added to a token's sum before any norm (what a part that runs for every token gave out)."""
+    (float32 [T, H]): rows added to a token's sum before any norm (what a part that runs for every token gave out).  store:
+    residual = the sum (no norm).  itself [T, H]: what a choice without a row (place -1) stands for, the token's own input.
+    next_norm (weight float32 [H], eps, buffer [T, H]; with an RMS norm): the buffer receives the RMS norm of the updated rows."""
     if weights is not None:
         tokens, top = weights.shape
     else:
@@ -1724,26 +1732,45 @@ def moe_combine(residual: torch.Tensor, rows: torch.Tensor, place: torch.Tensor,
           "moe_combine: extra rows must be contiguous float32 [T, H]")
     _need(norm_weight is None or (norm_weight.numel() == hidden and norm_weight.is_contiguous()), "moe_combine: norm weight must hold H values")
     _need(layer_norm_alpha is None or norm_weight is not None, "moe_combine: a layer norm needs its weight")
+    _need(itself is None or (itself.dim() == 2 and itself.shape[0] >= tokens and itself.shape[1] == hidden and itself.stride(1) == 1), "moe_combine: the tokens' own rows must be [T, H]")
+    follows = (None, 0.0, None, 0)
+    if next_norm is not None:
+        next_weight, next_eps, normed = next_norm
+        _need(norm_weight is not None and next_weight.dtype == torch.float32 and next_weight.numel() == hidden and next_weight.is_contiguous()
+              and normed.shape == (tokens, hidden) and normed.is_contiguous(), "moe_combine: the norm that follows needs a float32 weight [H] and a contiguous [T, H] buffer")
+        follows = (_dev(next_weight, "next_weight"), next_eps, _dev(normed, "normed"), dtype_code(normed.dtype))
     _launch("lrs_moe_combine", _dev(residual, "residual"), _dev(rows, "rows"), tokens, hidden, _dev(place, "place"), None if weights is None else _dev(weights, "weights"), top,
             None if norm_weight is None else _dev(norm_weight, "norm_weight"), 0 if norm_weight is None else dtype_code(norm_weight.dtype), eps,
             _rounded(rounded, tokens, hidden, "moe_combine"), int(layer_norm_alpha is not None), 0.0 if layer_norm_alpha is None else layer_norm_alpha,
-            None if extra is None else _dev(extra, "extra"), _stream())
+            None if extra is None else _dev(extra, "extra"), int(store), None if itself is None else _dev(itself, "itself"),
+            0 if itself is None else dtype_code(itself.dtype), 0 if itself is None else _rows(itself, "itself"), *follows, _stream())
 
 
 # ------------------------------------------------------------------- latent attention
 def latent_prep(proj: torch.Tensor, q_col: int, kv_col: int, heads: int, dim: int, rot: int, rank: int, norm_weight: torch.Tensor, eps: float,
-                cos: torch.Tensor | None, sin: torch.Tensor | None, pages: torch.Tensor, slots: torch.Tensor, queries: torch.Tensor,
-                value_pages: torch.Tensor | None = None) -> None:
+                cos: torch.Tensor | None, sin: torch.Tensor | None, pages: torch.Tensor, slots: torch.Tensor, queries: torch.Tensor | None,
+                value_pages: torch.Tensor | None = None, query_latent: tuple | None = None) -> None:
     """Per token of proj [T, columns]: the RMS norm (norm_weight, eps) of the `rank` latent values at column kv_col and the
     rotation (pairs 2i, 2i + 1; cos, sin [T, rot / 2], None: none) of the `rot` shared key values behind them, written into
     the token's row of pages [P, 1, page, rank + rot] (slots[t] < 0: not kept); and the rotation of the last `rot` of the
     dim + rot values of every head's query (from column q_col on) into queries [T, heads, rank + rot][..., rank:].
-    value_pages [P, 1, rank, page]: receives the normed latent values as well, transposed inside a page."""
+    value_pages [P, 1, rank, page]: receives the normed latent values as well, transposed inside a page.
+    query_latent (weight [q_rank], buffer [T, >= q_rank] of the rows' dtype; heads 0 and queries None then): column q_col begins the
+    q_rank latent values the queries will be made of; their RMS norm (weight of norm_weight's dtype, eps) goes into the buffer, zeros
+    into the columns behind it."""
     tokens, width = proj.shape[0], rank + rot
-    _need(proj.dim() == 2 and proj.stride(1) == 1 and proj.shape[1] >= max(q_col + heads * (dim + rot), kv_col + width), "latent_prep: proj rows are too short")
+    q_rank, of_queries = 0, (0, None, None, 0)
+    if query_latent is not None:
+        q_norm, q_rows = query_latent
+        q_rank = q_norm.numel()
+        _need(heads == 0 and queries is None and q_norm.dtype == norm_weight.dtype and q_norm.is_contiguous(), "latent_prep: queries, or the latent values they are made of with a weight of the other norm's dtype")
+        _need(q_rows.dim() == 2 and q_rows.is_contiguous() and q_rows.shape[0] == tokens and q_rows.shape[1] >= q_rank and q_rows.dtype == proj.dtype,
+              f"latent_prep: the normalised latent rows of the queries need a contiguous [{tokens}, >= {q_rank}] buffer of the rows' dtype")
+        of_queries = (q_rank, _dev(q_norm, "q_norm"), _dev(q_rows, "q_latent"), q_rows.shape[1])
+    _need(proj.dim() == 2 and proj.stride(1) == 1 and proj.shape[1] >= max(q_col + q_rank + heads * (dim + rot), kv_col + width), "latent_prep: proj rows are too short")
     _need(pages.dim() == 4 and pages.shape[1] == 1 and pages.shape[3] == width and pages.is_contiguous() and pages.dtype == proj.dtype,
           f"latent_prep: pages must be contiguous [P, 1, page, {width}] of the rows' dtype")
-    _need(queries.shape == (tokens, heads, width) and queries.is_contiguous() and queries.dtype == proj.dtype, f"latent_prep: queries must be [{tokens}, {heads}, {width}]")
+    _need(queries is None or (queries.shape == (tokens, heads, width) and queries.is_contiguous() and queries.dtype == proj.dtype), f"latent_prep: queries must be [{tokens}, {heads}, {width}]")
     _need(value_pages is None or (value_pages.shape == (pages.shape[0], 1, rank, pages.shape[2]) and value_pages.is_contiguous() and value_pages.dtype == pages.dtype),
           f"latent_prep: value pages must be contiguous [P, 1, {rank}, page] of the pages' dtype")
     _need(norm_weight.numel() == rank and norm_weight.is_contiguous(), f"latent_prep: the norm weight must hold {rank} values")
@@ -1754,18 +1781,26 @@ def latent_prep(proj: torch.Tensor, q_col: int, kv_col: int, heads: int, dim: in
     _launch("lrs_latent_prep", _dev(proj, "proj"), proj.stride(0), dtype_code(proj.dtype), tokens, q_col, kv_col, heads, dim, rot, rank,
             _dev(norm_weight, "norm_weight"), dtype_code(norm_weight.dtype), eps, None if cos is None else _dev(cos, "cos"),
             None if sin is None else _dev(sin, "sin"), _dev(pages, "pages"), None if value_pages is None else _dev(value_pages, "value_pages"), pages.shape[2],
-            _dev(slots, "slots"), _dev(queries, "queries"), heads * width, _stream())
+            _dev(slots, "slots"), None if queries is None else _dev(queries, "queries"), heads * width, *of_queries, _stream())
 
 
-def head_gemm(out: torch.Tensor, a: torch.Tensor, w: torch.Tensor, transposed: bool) -> None:
+def head_gemm(out: torch.Tensor, a: torch.Tensor, w: torch.Tensor, transposed: bool, rotate: tuple | None = None,
+              gate: torch.Tensor | None = None) -> None:
     """out [T, heads, n] = per head h: w[h] a[t, h] with w [heads, n, k], or w[h]^T a[t, h] with w [heads, k, n] if `transposed`.
-    out and a may be views with strides of their own between tokens and heads."""
-    tokens, heads, n = out.shape
-    k = a.shape[2]
+    out and a may be views with strides of their own between tokens and heads.
+    rotate (cos, sin float32 [T, rot / 2]): a and out have rot values more a head, behind the k inputs and the n outputs; they are
+    rotated in pairs (2i, 2i + 1) on the way.  gate [T, heads * n] (rows of any stride): out is multiplied by its sigmoid."""
+    rot = 0 if rotate is None else 2 * rotate[0].shape[1]
+    tokens, heads, n = out.shape[0], out.shape[1], out.shape[2] - rot
+    k = a.shape[2] - rot
+    for t in rotate or ():
+        _need(t.dtype == torch.float32 and t.shape == (tokens, rot // 2) and t.is_contiguous(), f"head_gemm: rotation tables must be float32 [{tokens}, {rot // 2}]")
+    _need(gate is None or (gate.shape == (tokens, heads * n) and gate.stride(1) == 1 and gate.dtype == out.dtype), f"head_gemm: gate must be [{tokens}, {heads * n}] of the rows' dtype")
     _need(a.shape[:2] == (tokens, heads) and a.stride(2) == 1 and out.stride(2) == 1 and a.dtype == out.dtype == w.dtype, "head_gemm: a [T, heads, k] and out [T, heads, n] of the weights' dtype")
     _need(w.is_contiguous() and w.shape == ((heads, k, n) if transposed else (heads, n, k)), f"head_gemm: w must be contiguous [{heads}, {k if transposed else n}, {n if transposed else k}]")
     _launch("lrs_head_gemm", _dev(out, "out"), out.stride(0), out.stride(1), _dev(a, "a"), a.stride(0), a.stride(1), _dev(w, "w"), n * k, int(transposed),
-            dtype_code(w.dtype), tokens, heads, n, k, _stream())
+            dtype_code(w.dtype), tokens, heads, n, k, rot, *((_dev(rotate[0], "cos"), _dev(rotate[1], "sin")) if rot else (None, None)),
+            None if gate is None else _dev(gate, "gate"), 0 if gate is None else _rows(gate, "gate"), _stream())
 
 
 def latent_attention(out: torch.Tensor, queries: torch.Tensor, pages: torch.Tensor, block_table: torch.Tensor, token_request: torch.Tensor,

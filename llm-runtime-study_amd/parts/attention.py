@@ -36,8 +36,13 @@ And with the norm over the projection: `query_temperature` (coef, every) multipl
 1 + coef * ln(floor((p + 1) / every) + 1); `value_mix` mixes a layer's values with those of an earlier layer of the same token,
 v <- (1 - lambda) v + lambda v_first with a learned lambda, before they are cached ("first": the layer whose values the others take,
 "later": a layer that takes them; they stay in a buffer of the step); `distance_bias` takes rate_h * ln(1 + reach_h * (i - j)) off
-head h's score of query i and key j; a number for `sink` is a sink of that score in every head instead of a learned one.  Values
+head h's score of query i and key j (`"linear"`: slope_h * (i - j) with the fixed slopes 2^(-8 (h + 1) / heads)); a number for `sink` is a sink of that score in every head instead of a learned one.  Values
 narrower than keys (a multiple of 16) run on the matrix cores too.
+
+`chunk` in place of a window: position i sees position j <= i only in its own chunk of that many positions, counted from position 0.
+Heads that need no preparation at all (no norm, rotation, bias, temperature or mixed values) stay where the product left them:
+only their keys and values pass through a kernel on their way into the pages, and in decode steps of few rows the attention kernel
+stores those too.
 """
 
 from __future__ import annotations
@@ -47,7 +52,7 @@ import math
 import torch
 
 from ..kernels import ops
-from .base import PagedKVNeed, Part, PartSpec, TensorSpec, create, length_class, register
+from .base import PagedKVNeed, Part, PartSpec, TensorSpec, create, length_class, reach_of, register
 from .linear import ScaledRows, kernels_of, linear, materialize, rows_of, workspace_of
 
 
@@ -69,7 +74,7 @@ class GQAAttention(Part):
                  kv_shared: bool = False, values_from_keys: bool = False, norm_over: str = "head", value_dim: int | None = None,
                  keep_first: int = 0, output_gate: bool | str = False, unit_norm_after_rotation: bool = False,
                  sink: bool | float = False, score_cap: float | None = None, query_temperature: tuple | None = None,
-                 value_mix: str | None = None, distance_bias: bool = False):
+                 value_mix: str | None = None, distance_bias: bool | str = False, chunk: int | None = None):
         for name, value in (("hidden_size", hidden_size), ("num_heads", num_heads), ("num_kv_heads", num_kv_heads), ("head_dim", head_dim)):
             if value <= 0:
                 raise ValueError(f"{name} must be positive, got {value}")
@@ -77,8 +82,8 @@ class GQAAttention(Part):
             raise ValueError(f"num_heads must be divisible by num_kv_heads, got {num_heads} and {num_kv_heads}")
         if scale is not None and (not math.isfinite(scale) or scale <= 0):
             raise ValueError(f"scale must be finite and positive, got {scale}")
-        if window is not None and window <= 0:
-            raise ValueError(f"window must be positive when given, got {window}")
+        # what a query sees: the kernels' word for it, and the most positions that can be (None: all)
+        self.reach, self.chunk, self.span = reach_of(window, chunk), chunk, window if chunk is None else chunk
         if qk_norm and qk_norm_eps <= 0:
             raise ValueError(f"qk_norm_eps must be positive, got {qk_norm_eps}")
         self.hidden_size, self.num_heads, self.num_kv_heads, self.head_dim = hidden_size, num_heads, num_kv_heads, head_dim
@@ -109,12 +114,17 @@ class GQAAttention(Part):
             raise ValueError(f"the query temperature's step must be positive, got {query_temperature[1]}")
         if value_mix not in (None, "first", "later"):
             raise ValueError(f"value_mix must be None, 'first' or 'later', got {value_mix!r}")
+        if distance_bias not in (False, True, "linear"):
+            raise ValueError(f"distance_bias must be False, True (learned, with a logarithm) or 'linear' (fixed slopes), got {distance_bias!r}")
         self.query_temperature, self.value_mix, self.distance_bias = query_temperature, value_mix, distance_bias
         self.neighbours = getattr(self.position, "pairing", "halves") == "interleaved"
         # the forms that the kernels preparing whole rows serve (see the module's text)
         self.whole_rows = bool((qk_norm and norm_over == "projection") or self.value_dim != head_dim or keep_first > 0 or output_gate
                                or unit_norm_after_rotation or self.has_sink or self.sink_score is not None or score_cap is not None or self.neighbours
                                or query_temperature is not None or value_mix is not None or distance_bias)
+        # heads that no kernel has to touch between the product and the attention (see the module's text)
+        self.heads_as_projected = bool(self.whole_rows and not (qk_norm or bias or unit_norm_after_rotation or query_temperature is not None
+                                                               or value_mix is not None) and position.kind == "none")
         if (unit_norm_after_rotation or self.neighbours) and (query_temperature is not None or value_mix is not None):
             raise ValueError("a query temperature and mixed values are made by the kernel that normalises over the projection")
         if self.whole_rows and (kv_shared or values_from_keys or (qk_norm and norm_over == "head")):
@@ -141,7 +151,7 @@ class GQAAttention(Part):
             specs["sink"] = TensorSpec((self.num_heads,), role="bias")
         if self.value_mix is not None:      # (the layer the others take their values from has no use for its own)
             specs["value_mix"] = TensorSpec((), role="bias", optional=self.value_mix == "first")
-        if self.distance_bias:              # drawn around one at random: a reach must not be negative
+        if self.distance_bias is True:      # drawn around one at random: a reach must not be negative
             specs["distance_rate"] = TensorSpec((self.num_heads,), role="norm")
             specs["distance_reach"] = TensorSpec((self.num_heads,), role="norm")
         specs["o_proj.weight"] = TensorSpec((h, self.num_heads * self.value_dim))
@@ -168,7 +178,10 @@ class GQAAttention(Part):
             self.sinks = torch.full((self.num_heads,), self.sink_score, dtype=torch.float32, device=self.w_qkv.device)
         if self.value_mix == "later":
             self.mix = weights["value_mix"].float().reshape(1).contiguous()
-        if self.distance_bias:
+        if self.distance_bias == "linear":
+            slopes = 2.0 ** (-8.0 * torch.arange(1, self.num_heads + 1, dtype=torch.float64) / self.num_heads)
+            self.distance = slopes.float().to(self.w_qkv.device)
+        elif self.distance_bias:
             self.distance = torch.stack((weights["distance_rate"].float(), weights["distance_reach"].float())).contiguous()
         self.w_o = weights["o_proj.weight"].to(dtype).contiguous()
         if self.qk_norm:
@@ -181,18 +194,16 @@ class GQAAttention(Part):
         return (self.w_qkv.numel() + self.w_o.numel()) * self.w_o.element_size()
 
     def flops(self, tokens, pairs):
-        if self.window is not None:
-            pairs = min(pairs, tokens * self.window)
+        if self.span is not None:
+            pairs = min(pairs, tokens * self.span)
         # the projections, then scores and weighted values: two products of head_dim per pair and query head
         return super().flops(tokens, pairs) + 2.0 * pairs * self.num_heads * (self.head_dim + self.value_dim)
 
     def cache_need(self):
         if self.kv_shared:
             return None
-        if self.value_dim != self.head_dim or self.keep_first:
-            return PagedKVNeed(self.num_kv_heads, self.head_dim, self.window, value_dim=None if self.value_dim == self.head_dim else self.value_dim,
-                               keep_first=self.keep_first)
-        return PagedKVNeed(self.num_kv_heads, self.head_dim, self.window)
+        return PagedKVNeed(self.num_kv_heads, self.head_dim, self.window, value_dim=None if self.value_dim == self.head_dim else self.value_dim,
+                           keep_first=self.keep_first, chunk=self.chunk)
 
     @staticmethod
     def _decode_splits(workgroups: int, longest: int, bound: int, page_size: int) -> int:
@@ -305,19 +316,19 @@ class GQAAttention(Part):
                         cache.k_pages, cache.v_pages, group.slots, group.page_size, skip_q=queries_raw is not None)
         if decode:
             longest, bound = ctx.max_k, ctx.max_k_bound
-            if self.window is not None:
-                longest, bound = min(longest, self.window + 32), min(bound, self.window + 64)
+            if self.span is not None:
+                longest, bound = min(longest, self.span + 32), min(bound, self.span + 64)
             splits = self._decode_splits(t * kv_heads, longest, bound, group.page_size)
             part_o = part_ml = None
             if splits > 1:
                 part_o = ctx.scratch("attn_part_o", (t, nq * splits * d), torch.float32)
                 part_ml = ctx.scratch("attn_part_ml", (t, nq * splits * 2), torch.float32)
             ops.attention_decode(out, qkv, cache.k_pages, cache.v_pages, group.block_table, ctx.token_slot, ctx.positions,
-                                 nq, self.scale, self.window or 0, splits, part_o, part_ml, ctx.max_k_bound, prepare,
+                                 nq, self.scale, self.reach, splits, part_o, part_ml, ctx.max_k_bound, prepare,
                                  form=1)   # the next tile on its way while one is worked on, the first one before the query is prepared (measured: 0.6 % of a step)
         elif ops.attention_decode_supported(ctx.dtype, nq, kv_heads, d, group.page_size):
             # sized by the step's coarse bound of the longest context, the same for every step of one shape
-            longest = ctx.max_k_bound if self.window is None else min(ctx.max_k_bound, self.window + 64)
+            longest = ctx.max_k_bound if self.span is None else min(ctx.max_k_bound, self.span + 64)
             singles = ctx.single_rows
             if singles:
                 # the single tokens at the head of a mixed step (decoding requests beside a prompt portion) go to the
@@ -338,7 +349,7 @@ class GQAAttention(Part):
                     first = ops.DecodePrepare(self.q_norm, self.k_norm, self.qk_norm_eps, None if parted is None else parted[0],
                                               None if parted is None else parted[1], 0)
                 ops.attention_decode(out[:singles], qkv[:singles], cache.k_pages, cache.v_pages, group.block_table, ctx.token_slot,
-                                     ctx.positions, nq, self.scale, self.window or 0, splits, part_o, part_ml, ctx.max_k_bound, first, form=1)
+                                     ctx.positions, nq, self.scale, self.reach, splits, part_o, part_ml, ctx.max_k_bound, first, form=1)
             rest = ctx.memo.get("rows_after_singles")
             if rest is None:
                 rest = ctx.memo["rows_after_singles"] = (ctx.token_slot[singles:], ctx.positions[singles:])
@@ -350,11 +361,11 @@ class GQAAttention(Part):
                 part_o = ctx.scratch("attn_part_o", (t - singles, nq * splits * d), torch.float32)
                 part_ml = ctx.scratch("attn_part_ml", (t - singles, nq * splits * 2), torch.float32)
             ops.attention_prefill(out[singles:], qkv[singles:], cache.k_pages, cache.v_pages, group.block_table, rest[0], rest[1],
-                                  ctx.qblock_token0, ctx.qblock_count, nq, self.scale, self.window or 0, ctx.max_qblock, ctx.max_k_bound,
+                                  ctx.qblock_token0, ctx.qblock_count, nq, self.scale, self.reach, ctx.max_qblock, ctx.max_k_bound,
                                   splits, part_o, part_ml, queries_raw)
         else:
             ops.attention(out, qkv, cache.k_pages, cache.v_pages, group.block_table, ctx.token_slot, ctx.positions,
-                          nq, self.scale, self.window or 0)
+                          nq, self.scale, self.reach)
         return linear(ctx, residual, out, self.w_o, accumulate=accumulate, then_norm=then_norm)
 
     def _forward_whole_rows(self, ctx, x, residual, cache, group, cos, sin, then_norm, accumulate):
@@ -365,7 +376,13 @@ class GQAAttention(Part):
         qkv = ctx.scratch("attn_qkvg", (t, self.w_qkv.shape[0]), ctx.dtype)
         linear(ctx, qkv, x, self.w_qkv)
         self.hand_out_carried(ctx, qkv)
-        if self.unit_after or self.neighbours:
+        cores = ops.attention_decode_supported(ctx.dtype, nq, nkv, d, group.page_size, dv)
+        prepare = None
+        if self.heads_as_projected and cores and ctx.all_decode and t <= self.PREPARE_INSIDE_ROWS and dv == d and not self.keep_first:
+            prepare = ops.DecodePrepare(None, None, 0.0, None, None, nkv)        # the attention kernel stores the new keys and values
+        elif self.heads_as_projected:
+            ops.qkv_norm_prep(qkv[:, nq * d:], 0, nkv, d, dv, None, None, 0.0, None, None, cache.k_pages, cache.v_pages, group.slots, group.page_size)
+        elif self.unit_after or self.neighbours:
             ops.rotate_unit_prep(qkv, nq, nkv, d, dv, self.qk_norm_eps, self.unit_after, cos, sin, self.neighbours, cache.k_pages, cache.v_pages,
                                  group.slots, group.page_size, bias=self.b_late)
         else:
@@ -378,22 +395,21 @@ class GQAAttention(Part):
         # gate a value by a kernel of its own behind them
         gates = qkv[:, gate_at:gate_at + nq] if self.output_gate == "head" else None
         out = ctx.scratch("attn_out", (t, nq * dv), ctx.dtype)
-        cores = ops.attention_decode_supported(ctx.dtype, nq, nkv, d, group.page_size, dv)
         extra = 1 if self.keep_first else 0      # the kept first positions' share is one more partial result for the merge
         if cores and ctx.all_decode:
             longest, bound = ctx.max_k, ctx.max_k_bound
-            if self.window is not None:
-                longest, bound = min(longest, self.window + 32), min(bound, self.window + 64)
+            if self.span is not None:
+                longest, bound = min(longest, self.span + 32), min(bound, self.span + 64)
             splits = self._decode_splits(t * nkv, longest, bound, group.page_size)
             part_o = part_ml = None
             if splits + extra > 1:
                 part_o = ctx.scratch("attn_part_o", (t, nq * (splits + extra) * dv), torch.float32)
                 part_ml = ctx.scratch("attn_part_ml", (t, nq * (splits + extra) * 2), torch.float32)
             ops.attention_decode(out, qkv, cache.k_pages, cache.v_pages, group.block_table, ctx.token_slot, ctx.positions,
-                                 nq, self.scale, self.window or 0, splits, part_o, part_ml, ctx.max_k_bound, None, form=1,
+                                 nq, self.scale, self.reach, splits, part_o, part_ml, ctx.max_k_bound, prepare, form=1,
                                  keep_first=self.keep_first, gates=gates, **more)
         elif cores:
-            longest = ctx.max_k_bound if self.window is None else min(ctx.max_k_bound, self.window + 64)
+            longest = ctx.max_k_bound if self.span is None else min(ctx.max_k_bound, self.span + 64)
             singles = ctx.single_rows
             if singles:
                 splits = self._decode_splits(singles * nkv, longest, ctx.max_k_bound, group.page_size)
@@ -402,7 +418,7 @@ class GQAAttention(Part):
                     part_o = ctx.scratch("attn_single_part_o", (singles, nq * (splits + extra) * dv), torch.float32)
                     part_ml = ctx.scratch("attn_single_part_ml", (singles, nq * (splits + extra) * 2), torch.float32)
                 ops.attention_decode(out[:singles], qkv[:singles], cache.k_pages, cache.v_pages, group.block_table, ctx.token_slot,
-                                     ctx.positions, nq, self.scale, self.window or 0, splits, part_o, part_ml, ctx.max_k_bound, None, form=1,
+                                     ctx.positions, nq, self.scale, self.reach, splits, part_o, part_ml, ctx.max_k_bound, None, form=1,
                                      keep_first=self.keep_first, gates=None if gates is None else gates[:singles], **more)
             rest = ctx.memo.get("rows_after_singles")
             if rest is None:
@@ -413,11 +429,11 @@ class GQAAttention(Part):
                 part_o = ctx.scratch("attn_part_o", (t - singles, nq * (splits + extra) * dv), torch.float32)
                 part_ml = ctx.scratch("attn_part_ml", (t - singles, nq * (splits + extra) * 2), torch.float32)
             ops.attention_prefill(out[singles:], qkv[singles:], cache.k_pages, cache.v_pages, group.block_table, rest[0], rest[1],
-                                  ctx.qblock_token0, ctx.qblock_count, nq, self.scale, self.window or 0, ctx.max_qblock, ctx.max_k_bound,
+                                  ctx.qblock_token0, ctx.qblock_count, nq, self.scale, self.reach, ctx.max_qblock, ctx.max_k_bound,
                                   splits, part_o, part_ml, None, keep_first=self.keep_first, gates=None if gates is None else gates[singles:], **more)
         else:
             ops.attention(out, qkv, cache.k_pages, cache.v_pages, group.block_table, ctx.token_slot, ctx.positions, nq, self.scale,
-                          self.window or 0, self.keep_first, gates=gates, **more)
+                          self.reach, self.keep_first, gates=gates, **more)
         if self.output_gate is True:
             ops.sigmoid_gate(out, qkv[:, gate_at:gate_at + self.gate_width])
         return linear(ctx, residual, out, self.w_o, accumulate=accumulate, then_norm=then_norm)

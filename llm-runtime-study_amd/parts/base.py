@@ -54,6 +54,12 @@ Optional, each announced by a class attribute (a part without it is simply given
                               the product's output (in that buffer's dtype).  A block whose residual is gated by a matrix of
                               the sublayer's input saves a launch this way
 
+  can_overwrite = True        mixer / feed_forward: forward(..., accumulate=False) stores its output into the float32 rows it is
+                              given instead of adding to them
+  applies_output_norm = True  feed_forward: forward(..., output_norm=norm) adds the RMS norm of its output into the stream itself
+  leaves_next_norm = True     ... and forward(..., next_norm=(weight, eps, buffer)) beside it leaves the RMS norm of the new stream
+                              in `buffer`, the input of the sublayer that runs next
+
 A part may also say how its steps can be run again without it (both default to no):
 
   graph_safe = True           it launches only kernels on preallocated buffers, and reads the step's data from
@@ -204,6 +210,18 @@ class PagedKVNeed:
     dtype: torch.dtype | None = None
     value_dim: int | None = None
     keep_first: int = 0         # with a window: the first positions of a sequence stay visible for good, so their pages are never given back
+    chunk: int | None = None    # instead of a window: a position is seen by later ones of its own chunk only (chunks of this many, from position 0 on)
+
+    @property
+    def span(self) -> int | None:
+        """The most positions up to its own that a query sees (None: all)."""
+        return self.window if self.chunk is None else self.chunk
+
+    def first_needed(self, position: int) -> int:
+        """The first position that a query at `position`, or any later one, sees (kept first positions aside)."""
+        if self.chunk is not None:
+            return position - position % self.chunk
+        return 0 if self.window is None else max(0, position - self.window + 1)
 
 
 @dataclass(frozen=True)
@@ -221,6 +239,27 @@ class BothNeeds:
 
     paged: PagedKVNeed
     state: StateNeed
+
+
+def reach_of(window: int | None, chunk: int | None) -> int:
+    """What the attention kernels take as their `window`: a sliding window's size, minus a chunk's, 0 for all earlier positions."""
+    if window is not None and chunk is not None:
+        raise ValueError("a query sees a window or its chunk, not both")
+    for name, size in (("window", window), ("chunk", chunk)):
+        if size is not None and size <= 0:
+            raise ValueError(f"{name} must be positive when given, got {size}")
+    return -chunk if chunk is not None else window or 0
+
+
+@dataclass(frozen=True)
+class BoundNorm:
+    """An RMS norm as its weight (float32) and eps, for a part that applies the norm of its own output (`applies_output_norm`)."""
+
+    weight: Any
+    eps: float
+
+    def rms_parameters(self):
+        return self.weight, self.eps
 
 
 class Part:

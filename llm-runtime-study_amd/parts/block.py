@@ -29,7 +29,7 @@ scaled after it:
 The gate's matrix is stacked behind the sublayer's first product where the sublayer can carry it, the scale is part of the second
 norm's weight, and one kernel (`gated_norm_add`) gates, normalises, adds into the stream and leaves the norm that comes next, in this
 layer or the next one, beside it.  Gate and scale are parameters of the block: with neither it is the plain arrangement of norms on
-both sides.
+both sides (a feed-forward that says `leaves_next_norm` then does all of that in the kernel that sums its own output up).
 """
 
 from __future__ import annotations
@@ -37,7 +37,7 @@ from __future__ import annotations
 import torch
 
 from ..kernels import ops
-from .base import Part, PartSpec, TensorSpec, create, flops_of, register, under
+from .base import BoundNorm, Part, PartSpec, TensorSpec, create, flops_of, register, under
 from .linear import linear, materialize
 
 
@@ -473,6 +473,10 @@ class SandwichBlock(ParallelBlock):
     def _update(self, ctx, which, part, x, h, more, following):
         """h += scale * norm(part(x) * gate(x)); returns the following norm of the new stream, if that is one this kernel makes."""
         weight, eps, matrix, bias = self._bound[which]
+        following_norm = self._following(ctx, h, following)
+        if not self.gated and getattr(part, "leaves_next_norm", False):
+            part.forward(ctx, x, h, *more, output_norm=BoundNorm(weight, eps), next_norm=following_norm)
+            return None if following_norm is None else following_norm[2]
         y = ctx.scratch("sublayer_out", tuple(h.shape), torch.float32)
         gate = None
         ctx.memo.pop("carried_rows", None)
@@ -482,16 +486,21 @@ class SandwichBlock(ParallelBlock):
             linear(ctx, gate, materialize(ctx, x), matrix)
         elif self.gated:
             gate = ctx.memo.pop("carried_rows")
-        parameters = getattr(following, "rms_parameters", None)
-        if parameters is None:
+        if following_norm is None:
             ops.gated_norm_add(h, y, gate, bias, weight, eps)
             return None
-        next_weight, next_eps = parameters()
-        turn = ctx.memo["normed_stream_turn"] = 1 - ctx.memo.get("normed_stream_turn", 0)     # not the buffer x lies in
+        ops.gated_norm_add(h, y, gate, bias, weight, eps, *following_norm)
+        return following_norm[2]
+
+    def _following(self, ctx, h, norm):
+        """(weight, eps, buffer) of the norm that comes next, if it is one the kernels here make; else None."""
+        parameters = getattr(norm, "rms_parameters", None)
+        if parameters is None:
+            return None
+        weight, eps = parameters()
+        turn = ctx.memo["normed_stream_turn"] = 1 - ctx.memo.get("normed_stream_turn", 0)     # not the buffer the sublayer's input lies in
         normed = ctx.scratch(f"stream_normed{turn}", tuple(h.shape), ctx.dtype)
-        next_weight = next_weight if next_weight.dtype == torch.float32 else self._weight_f32(following, next_weight)
-        ops.gated_norm_add(h, y, gate, bias, weight, eps, next_weight, next_eps, normed)
-        return normed
+        return weight if weight.dtype == torch.float32 else self._weight_f32(norm, weight), eps, normed
 
 
 register("block", "sandwich", SandwichBlock)

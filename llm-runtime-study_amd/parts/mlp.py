@@ -79,7 +79,7 @@ register("feed_forward", "swiglu", SwiGLU)
 
 class DenseMLP(Part):
     """down(act(up(x))): two bias-free projections, `activation` between them: "gelu" (the exact one, 0.5 z (1 + erf(z / sqrt 2))),
-    "gelu_tanh", "silu" or "relu" (kernels/ops.py, ACTIVATIONS), or "xielu", which has two learned numbers (p, q): with z = up(x),
+    "gelu_tanh", "silu", "relu" or "relu_squared" (kernels/ops.py, ACTIVATIONS), or "xielu", which has two learned numbers (p, q): with z = up(x),
     softplus(p) z^2 + z / 2 for z > 0 and (1/2 + softplus(q)) (exp(z) - 1 - z) + z / 2 otherwise.  The down projection adds into the float32 rows it is given, or
     stores into them with `accumulate=False`."""
 
