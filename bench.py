@@ -6,6 +6,7 @@
     python bench.py --design kaposun [--shape 8b] [--layers 8] ...     # the same for the Kaposun design
     python bench.py --design felosun [--shape 8b] [--layers 8] ...     # the Felosun design beside a Nobodra model of attention layers and experts of equal sizes
     python bench.py --design mutolix [--shape 8b] [--layers 8] ...     # the Mutolix design beside a Kaposun model of state space and attention layers of equal sizes
+    python bench.py --design tamilix [--shape 8b] [--layers 8] ...     # the Tamilix design beside Felosun (attention, experts) and Napizen (latent attention) models of equal sizes
 
 A step is one decode step of the whole engine (scheduler, step function, sampling) at the
 given batch; `value` is decoded tokens per second.  The same line carries the prefill rate
@@ -30,7 +31,7 @@ if str(ROOT) not in sys.path:
 HBM_PEAK = 8.0e12
 FLOP_PEAK = {"bf16": 2.5e15, "fp32": 157.3e12}
 
-from llm_runtime_study_amd.benchmarks.shapes import QWEN3_8B, SHAPES, felosun_like, kaposun_like, mutolix_like, napizen_like, nobodra_like  # noqa: E402  (layer sizes of the 8B, 14B and 32B models)
+from llm_runtime_study_amd.benchmarks.shapes import QWEN3_8B, SHAPES, felosun_like, kaposun_like, mutolix_like, napizen_like, nobodra_like, tamilix_like  # noqa: E402  (layer sizes of the 8B, 14B and 32B models)
 
 FULL_LAYERS = QWEN3_8B["num_hidden_layers"]
 BENCHMARK_CONTEXT = 4096      # tokens a request's cache can hold at the least: the benchmark context of the 8B configuration
@@ -50,8 +51,8 @@ def parse_args():
     parser.add_argument("--num-pages", type=int, default=None, help="pages of the cache pool (default: max-seq-len tokens for every request of the largest batch)")
     parser.add_argument("--shape", choices=tuple(SHAPES), default="8b", help="layer sizes: Qwen3-8B (default), 14B or 32B")
     parser.add_argument("--layers", type=int, default=None, help="fewer layers than the shape has (reported in config)")
-    parser.add_argument("--design", choices=("qwen3", "nobodra", "napizen", "kaposun", "felosun", "mutolix"), default="qwen3",
-                        help="measure that design at the shape's layer sizes (8 layers unless --layers says otherwise) and, beside it, the shape itself (felosun, mutolix: the design nearest to it) with as many layers")
+    parser.add_argument("--design", choices=("qwen3", "nobodra", "napizen", "kaposun", "felosun", "mutolix", "tamilix"), default="qwen3",
+                        help="measure that design at the shape's layer sizes (8 layers unless --layers says otherwise) and, beside it, the shape itself (felosun, mutolix, tamilix: the designs nearest to it) with as many layers")
     parser.add_argument("--dtype", choices=("bfloat16", "float32"), default="bfloat16")
     parser.add_argument("--no-points", action="store_true", help="skip the batch 1 and 64 decode points")
     parser.add_argument("--temperature", type=float, default=0.0, help="draw the tokens at this temperature instead of taking the largest logit (reported in config)")
@@ -190,7 +191,8 @@ def prefill_entry(engine, tokens: int, dtype_name: str, seed: int) -> dict:
 def step_bytes(engine, batch: int, mean_context: float) -> float:
     """Bytes a decode step of `batch` requests must read (and, for states, write back): the weights in use, the cached
     keys and values inside every layer's window, every request's state rows.  A layer of routed experts reads the experts
-    that the batch's tokens choose between them: experts * (1 - (1 - top / experts) ** batch) of them on average."""
+    that the batch's tokens choose between them: experts * (1 - (1 - top / choices) ** batch) of them on average, `choices` being the
+    outputs of the router (identity experts, which have no weights, among them).  A layer in chunks reads the chunk a request is in."""
     import math
 
     from llm_runtime_study_amd.parts import BothNeeds, PagedKVNeed, StateNeed
@@ -201,11 +203,12 @@ def step_bytes(engine, batch: int, mean_context: float) -> float:
         total += layer.weight_bytes()
         ff = getattr(layer, "feed_forward", None)
         if ff is not None and hasattr(ff, "num_experts"):
-            hit = ff.num_experts * (1.0 - (1.0 - ff.top / ff.num_experts) ** batch)
-            total += (hit - ff.top) * (3 if getattr(ff, "gated", False) else 2) * ff.hidden_size * ff.intermediate_size * ff.up.element_size()
+            hit = ff.num_experts * (1.0 - (1.0 - ff.top / ff.choices) ** batch)
+            total += (hit - ff.top * ff.num_experts / ff.choices) * (3 if getattr(ff, "gated", False) else 2) * ff.hidden_size * ff.intermediate_size * ff.up.element_size()
         for need in ((need.paged, need.state) if isinstance(need, BothNeeds) else (need,)):
             if isinstance(need, PagedKVNeed):
                 held = mean_context if need.window is None else min(mean_context, need.window + need.keep_first)
+                held = held if need.chunk is None else mean_context % need.chunk
                 kept = need.head_dim + (need.head_dim if need.value_dim is None else need.value_dim)
                 total += batch * held * need.num_kv_heads * kept * (2 if engine.dtype == torch_bfloat16() else 4)
             elif isinstance(need, StateNeed):
@@ -242,7 +245,7 @@ def measure_design(args, config, dtype_name: str, max_seq_len: int, max_batch: i
 
 
 def design_main(args) -> int:
-    """--design nobodra | napizen | kaposun | felosun | mutolix: the design at the shape's layer sizes, and the shape itself with as many layers, one after the other."""
+    """--design nobodra | napizen | kaposun | felosun | mutolix | tamilix: the design at the shape's layer sizes, and the shape itself with as many layers, one after the other."""
     import gc
 
     import torch
@@ -254,20 +257,28 @@ def design_main(args) -> int:
     max_batch = args.batch if args.no_points else max(args.batch, 64)
     max_seq_len = args.max_seq_len or max(BENCHMARK_CONTEXT, args.context + args.steps + warmup_room(args.warmup, max(args.decode_steps_per_launch, 1))
                                           + decode_lead(max_batch, args.context, max(2048, args.prefill_tokens)) + max_batch + 64, args.prefill_tokens + 1)
-    name = {"nobodra": "Nobodra", "napizen": "Napizen", "kaposun": "Kaposun", "felosun": "Felosun", "mutolix": "Mutolix"}[args.design]
-    raw = {"nobodra": nobodra_like, "napizen": napizen_like, "kaposun": kaposun_like, "felosun": felosun_like, "mutolix": mutolix_like}[args.design](SHAPES[args.shape], layers)
+    name = {"nobodra": "Nobodra", "napizen": "Napizen", "kaposun": "Kaposun", "felosun": "Felosun", "mutolix": "Mutolix", "tamilix": "Tamilix"}[args.design]
+    raw = {"nobodra": nobodra_like, "napizen": napizen_like, "kaposun": kaposun_like, "felosun": felosun_like, "mutolix": mutolix_like, "tamilix": tamilix_like}[args.design](SHAPES[args.shape], layers)
     mine = measure_design(args, config_from_dict(raw), dtype_name, max_seq_len, max_batch)
     gc.collect()
     torch.cuda.empty_cache()
     # Felosun stands beside the model nearest to it: Nobodra's layers of windowed attention and routed experts (the same block that
     # normalises outputs), at equal sizes; the others beside the dense shape itself
-    # and Mutolix beside Kaposun's state space layers and its attention with a norm over the projection, in Mutolix's order
+    # and Mutolix beside Kaposun's state space layers and its attention with a norm over the projection, in Mutolix's order; Tamilix
+    # beside Felosun (grouped-query attention with sinks, clamped experts and a shared one), and Napizen (latent attention) as a third
     shape = SHAPES[args.shape]
     beside_raw, beside_name = {
         "felosun": lambda: (nobodra_like(shape, layers, attention_only=True), "Nobodra, attention layers only, at the same sizes"),
+        "tamilix": lambda: (felosun_like(shape, layers), "Felosun at the same sizes"),
         "mutolix": lambda: (kaposun_like(shape, layers, order="ends"), "Kaposun, state space and attention layers, at the same sizes"),
     }.get(args.design, lambda: (dict(shape, num_hidden_layers=layers), f"Qwen3-{args.shape.upper()} shape"))()
     beside = measure_design(args, config_from_dict(beside_raw), dtype_name, max_seq_len, max_batch)
+    third = {}
+    if args.design == "tamilix":
+        gc.collect()
+        torch.cuda.empty_cache()
+        third = {"beside_latent": {"model": f"Napizen at the same sizes, {layers} layers",
+                                   **measure_design(args, config_from_dict(napizen_like(shape, layers)), dtype_name, max_seq_len, max_batch)}}
     main_point = mine[f"decode_b{args.batch}"]
     line = {
         "metric": f"decode tok/s at batch {args.batch} ({name} at Qwen3-{args.shape.upper()} layer sizes, {layers} layers)",
@@ -277,11 +288,12 @@ def design_main(args) -> int:
         "config": {"model": f"{name} at Qwen3-{args.shape.upper()} layer sizes", "layers": layers, "width": raw["width"], "layer_kinds": [layer["type"] for layer in raw["layers"]],
                    "mixer": raw["layers"][-1]["mixer"] if layers >= 4 else raw["layers"][0]["mixer"], "first_mixer": raw["layers"][0]["mixer"],
                    **({"third_mixer": raw["layers"][2]["mixer"]} if args.design == "kaposun" and layers >= 3 else {}),
-                   **({"second_mixer": raw["layers"][1]["mixer"]} if args.design == "mutolix" and layers >= 2 else {}),
+                   **({"second_mixer": raw["layers"][1]["mixer"]} if args.design in ("mutolix", "tamilix") and layers >= 2 else {}),
                    "mlp": [raw["layers"][0]["mlp"], raw["layers"][min(1, layers - 1)]["mlp"] if args.design == "mutolix" else raw["layers"][-1]["mlp"]],
                    "global_batch": args.batch, "seq_len": args.context, "max_seq_len": max_seq_len, "prefill_tokens": args.prefill_tokens, "parallelism": "single GPU"},
         args.design: mine,
         "beside": {"model": f"{beside_name}, {layers} layers", **beside},
+        **third,
     }
     print(json.dumps(line))
     return 0

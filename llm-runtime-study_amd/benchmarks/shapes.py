@@ -67,6 +67,24 @@ def napizen_like(shape: dict, layers: int, experts: int = 32, top: int = 8, rank
             "layers": [{"type": "latent_attention", "mixer": mixer, "mlp": routed if index % 2 else dense} for index in range(layers)]}
 
 
+def tamilix_like(shape: dict, layers: int, experts: int = 32, identity: int = 8, top: int = 8, chunk: int = 4096, window: int = 4096, q_rank: int = 1536,
+                 rank: int = 512, rot: int = 64) -> dict:
+    """A Tamilix configuration with the layer sizes of a dense shape above, for measurements beside models of equal sizes: the same
+    width, vocabulary and heads; in turn a layer of attention in chunks and a layer of latent attention behind a window (heads of the
+    shape's size plain and `rot` rotated dims, queries from `q_rank` latent values, `rank` latent values a position, both at most half
+    the width's); every other pair of layers has the dense feed-forward first (two matrices of `intermediate_size` where the shape has
+    three) or felosun_like's experts with a shared one, and `identity` more outputs of the router."""
+    width, heads, kv_heads, dim = shape["hidden_size"], shape["num_attention_heads"], shape["num_key_value_heads"], shape["head_dim"]
+    ff = max(128, round(shape["intermediate_size"] / (top + 1) / 128) * 128)
+    routed = {"kind": "moe", "expert": {"ff": ff, "limit": 7.0}, "router": {"experts": experts, "identity": identity, "top": top}, "shared": {"ff": ff, "limit": 7.0}}
+    dense = {"kind": "dense", "ff": shape["intermediate_size"]}
+    chunked = {"type": "attention", "mixer": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": dim ** -0.5, "mask": {"size": chunk}}}
+    latent = {"type": "latent_attention", "mixer": {"heads": heads, "dim": dim, "rot_dim": rot, "vdim": dim, "q_rank": min(q_rank, width // 2), "kv_rank": min(rank, width // 2),
+                                                    "scale": (dim + rot) ** -0.5, "mask": {"size": window}, "rot": {"base": 500000.0, "dims": rot}}}
+    return {"architecture": "Tamilix", "vocab": shape["vocab_size"], "width": width, "norm": {"eps": 1e-6}, "embedding": {"scale": 1.0},
+            "layers": [dict((chunked, latent)[index % 2], mlp=(dense, routed, routed, dense)[index % 4]) for index in range(layers)]}
+
+
 def mutolix_like(shape: dict, layers: int) -> dict:
     """A Mutolix configuration with the layer sizes of a dense shape above, for measurements beside a model of equal sizes: the same
     width, vocabulary and attention heads; of every four layers the first and the last are matrix memories without feed-forward
