@@ -60,6 +60,23 @@ __device__ __forceinline__ float distance_loss_of(const float* __restrict__ dist
   return form == DISTANCE_LINEAR ? distance[head] * LOG2E * behind : distance_loss(distance[head], distance[nq + head], behind);
 }
 
+// A linear bias makes the scores of a walk towards the query rise by the rate at every position, so a reference point that fits a tile
+// is soon far below the next ones'.  A walk whose weights have grown beyond GROWN raises its reference points by what brings the sums
+// down to 2^-40 (never further: nothing that has been added up is lost) and goes on; `more` is what to add to the reference point, in
+// powers of two, a whole number that the four lanes of a query agree on.
+constexpr float GROWN = 0x1p24f;
+__device__ __forceinline__ float growth_of(float run_sum) {
+  float most = fmaxf(run_sum, __shfl_xor(run_sum, 16, WAVE));
+  most = fmaxf(most, __shfl_xor(most, 32, WAVE));
+  return most >= 1.f ? floorf(__builtin_amdgcn_logf(most)) + 40.f : 0.f;
+}
+
+// The linear form of the bias for four keys in a row, the first of them `behind` positions behind the query.
+__device__ __forceinline__ floatx4 linear_of_four(float rate, float behind) {
+  const float first = -rate * behind;
+  return floatx4{first, first + rate, fmaf(rate, 2.f, first), fmaf(rate, 3.f, first)};
+}
+
 // A gate a head: the head's output times sigmoid(gates[token, head]), the gate values lying in rows of their own stride (the
 // columns of the projection that made them).  Null: no gate.
 template <typename T>
@@ -848,7 +865,8 @@ LRS_API int lrs_attention_decode(void* out, int out_stride, float* part_o, float
 // splits > 1 (few queries over long contexts): the key tiles of every group are divided between
 // `splits` workgroups, which leave unnormalised sums, maxima and weights in part_o / part_ml
 // [tokens, heads, splits, ...] for attention_merge_kernel, as the decode kernel does.
-template <int D, int QB>
+// LINEAR: the linear bias by distance, as instances of their own so that the others keep their registers.
+template <int D, int QB, bool LINEAR>
 __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void attention_prefill_bf16_kernel(
     bf16* __restrict__ out, int out_stride, const bf16* __restrict__ q, int q_stride,
     const bf16* __restrict__ k_pages, const bf16* __restrict__ v_pages,
@@ -857,7 +875,7 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void attention_prefill_bf16_
     const int* __restrict__ qblock_count, int n_blocks, int chunk, int nq, int nkv, int page_size, float scale,
     int window, int splits, int slots, float* __restrict__ part_o, float* __restrict__ part_ml,
     const float* __restrict__ sinks, float softcap, const bf16* __restrict__ gates, int gate_stride, int dv,
-    const float* __restrict__ distance, int distance_form) {
+    const float* __restrict__ distance) {
   constexpr int DS = D / 32, DB = D / 16;
   // Padded LDS rows.  Every fragment is read 16 bytes a lane, 16 rows at a time (the lane's row is col, its
   // piece g), which the LDS serves at its full 256 bytes a cycle when rows lie 32 bytes more than a multiple
@@ -986,14 +1004,31 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void attention_prefill_bf16_
 
     // the head's bias by distance, in units of the unscaled scores
     const int biased = active ? head : head0;
-    const bool linear = distance && distance_form == DISTANCE_LINEAR;
-    const float rate = distance ? distance[biased] * (linear ? 1.f : LN2) / scale : 0.f, reach = distance && !linear ? distance[nq + biased] : 0.f;
-    // the linear form: what the products of keys first .. first + 3 are added to (with a cap on the scores, what is added to them)
-    auto linear_bias = [&](int b, int first) {
-      const float before = -rate * (float)((live[b] ? pos[b] : pos_last) - first);
-      return floatx4{before, fmaf(rate, 1.f, before), fmaf(rate, 2.f, before), fmaf(rate, 3.f, before)};
+    const float rate = distance ? distance[biased] * (LINEAR ? 1.f : LN2) / scale : 0.f, reach = !LINEAR && distance ? distance[nq + biased] : 0.f;
+    // The linear form in two parts: what depends on a key's place in its tile is what the tile's products are added to (the same for
+    // every tile), and what is the same for all of a query's keys in the tile joins the exponents' shift.  With a cap on the scores,
+    // or two blocks of queries (whose registers are all in use), it is taken off whole.
+    const bool in_parts = LINEAR && QB == 1 && !(softcap > 0.f);
+    floatx4 in_tile[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
+    if constexpr (LINEAR && QB == 1) {
+#pragma unroll
+      for (int h = 0; h < 2; ++h)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) in_tile[h][i] = in_parts ? rate * (float)(h * 16 + g * 4 + i) : 0.f;
+    }
+    auto of_tile = [&](int tile, int b) { return in_parts ? -rate * (float)((live[b] ? pos[b] : pos_last) - tile * 32) : 0.f; };
+    bool grown = false;                                        // the weights have left the reference points behind
+    auto raise_reference = [&]() {
+#pragma unroll
+      for (int b = 0; b < QB; ++b) {
+        const float more = growth_of(run_sum[b]), shrink = fast_exp2(-more);
+        run_max[b] += more / scale2;
+        run_sum[b] *= shrink;
+#pragma unroll
+        for (int e = 0; e < DB; ++e) o[b][e] *= shrink;
+      }
+      grown = false;
     };
-    const bool linear_first = linear && !(softcap > 0.f);
     // The three parts of a tile's work.
     // scores: S[key, query] = K Q^T, unscaled (the scale enters with the exponent).
     auto scores = [&](int tile, int buffer, floatx4 (&sc)[QB][2]) {
@@ -1001,7 +1036,7 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void attention_prefill_bf16_
 #pragma unroll
       for (int b = 0; b < QB; ++b)
 #pragma unroll
-        for (int h = 0; h < 2; ++h) sc[b][h] = linear_first ? linear_bias(b, tile * 32 + h * 16 + g * 4) : floatx4{0.f, 0.f, 0.f, 0.f};
+        for (int h = 0; h < 2; ++h) sc[b][h] = in_tile[h];
 #pragma unroll
       for (int h = 0; h < 2; ++h)
 #pragma unroll
@@ -1019,13 +1054,13 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void attention_prefill_bf16_
 #pragma unroll
             for (int i = 0; i < 4; ++i) sc[b][h][i] = capped(sc[b][h][i], cap);
       }
-      if (linear && !linear_first) {
+      if (LINEAR && !in_parts) {
 #pragma unroll
         for (int b = 0; b < QB; ++b)
 #pragma unroll
-          for (int h = 0; h < 2; ++h) sc[b][h] += linear_bias(b, tile * 32 + h * 16 + g * 4);
+          for (int h = 0; h < 2; ++h) sc[b][h] += linear_of_four(rate, (float)((live[b] ? pos[b] : pos_last) - (tile * 32 + h * 16 + g * 4)));
       }
-      if (distance && !linear) { // (a key ahead of the query gives no number here; the mask takes it out)
+      if (!LINEAR && distance) { // (a key ahead of the query gives no number here; the mask takes it out)
 #pragma unroll
         for (int b = 0; b < QB; ++b)
 #pragma unroll
@@ -1051,6 +1086,11 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void attention_prefill_bf16_
 #pragma unroll
       for (int b = 0; b < QB; ++b) {
         float tile_max = -INFINITY;
+        if (in_parts) {
+          const float all = of_tile(tile, b);
+          sc[b][0] += all;
+          sc[b][1] += all;
+        }
 #pragma unroll
         for (int h = 0; h < 2; ++h)
 #pragma unroll
@@ -1089,12 +1129,12 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void attention_prefill_bf16_
           for (int e = 0; e < DB; ++e) o[b][e] *= alpha[b];
       }
     };
-    auto weights = [&](floatx4 (&sc)[QB][2], bf16x8 (&pf)[QB]) -> bool {
+    auto weights = [&](int tile, floatx4 (&sc)[QB][2], bf16x8 (&pf)[QB]) -> bool {
       float sums[QB];
       bool again = false;
 #pragma unroll
       for (int b = 0; b < QB; ++b) {
-        const float shift = -run_max[b] * scale2;                // +inf before the query's first tile: the sum then says "again"
+        const float shift = ((LINEAR && QB == 1 ? of_tile(tile, b) : 0.f) - run_max[b]) * scale2;      // +inf before the query's first tile: the sum then says "again"
         float tile_sum = 0.f;
 #pragma unroll
         for (int h = 0; h < 2; ++h)
@@ -1108,8 +1148,13 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void attention_prefill_bf16_
         again |= !(tile_sum <= 0x1p60f);                         // too large, infinite or not a number
       }
       if (__any(again)) return false;
+      bool large = false;
 #pragma unroll
-      for (int b = 0; b < QB; ++b) run_sum[b] += sums[b];
+      for (int b = 0; b < QB; ++b) {
+        run_sum[b] += sums[b];
+        if constexpr (LINEAR && QB == 1) large |= sums[b] > GROWN;
+      }
+      if constexpr (LINEAR && QB == 1) grown = __any(large);
       return true;
     };
     // values: O^T[dim, query] += V^T P
@@ -1147,17 +1192,23 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void attention_prefill_bf16_
     int tile = first_tile;
     for (;;) {
       bool unfinished = false;
-      for (; tile <= last_tile; ++tile) {
+      for (; tile <= last_tile && !(LINEAR && QB == 1 && grown); ++tile) {
         const int buffer = (tile - first_tile) & 1;
         if (tile < last_tile) fetch(tile + 1, kreg_a, vreg_a);
         scores(tile, buffer, sc);
-        if (tile < whole_begin || tile >= whole_end || !weights(sc, pf)) {
+        if (tile < whole_begin || tile >= whole_end || !weights(tile, sc, pf)) {
           unfinished = true;
           break;
         }
         values(buffer, pf);
         if (tile < last_tile) stash(buffer ^ 1, kreg_a, vreg_a);
         __syncthreads();
+      }
+      if constexpr (LINEAR && QB == 1) {
+        if (grown) {
+          raise_reference();
+          continue;
+        }
       }
       if (!unfinished) break;
       const int buffer = (tile - first_tile) & 1;
@@ -1224,7 +1275,7 @@ __global__ __launch_bounds__(256, D <= 128 ? 2 : 1) void attention_prefill_bf16_
 // linear one, which without a cap is what the products are added to and costs nothing), or the cap and then the bias.
 enum { SCORES_PLAIN = 0, SCORES_CAPPED = 1, SCORES_DISTANCE = 2, SCORES_BOTH = 3, SCORES_LINEAR = 4, SCORES_CAPPED_LINEAR = 5 };
 template <int QB, bool MANY_WAVES, bool IDLE_WAVES, int SCORES>
-__global__ __launch_bounds__(MANY_WAVES ? 512 : 256, MANY_WAVES ? 1 : 2) void attention_prefill_d128_bf16_kernel(
+__global__ __launch_bounds__(MANY_WAVES ? 512 : 256, MANY_WAVES ? 1 : QB == 1 && (SCORES & SCORES_LINEAR) ? 3 : 2) void attention_prefill_d128_bf16_kernel(
     bf16* __restrict__ out, int out_stride, const bf16* __restrict__ q, int q_stride,
     const bf16* __restrict__ k_pages, const bf16* __restrict__ v_pages,
     const int* __restrict__ block_table, int table_stride, const int* __restrict__ token_request,
@@ -1387,11 +1438,19 @@ __global__ __launch_bounds__(MANY_WAVES ? 512 : 256, MANY_WAVES ? 1 : 2) void at
       reach = distance[nq + biased];
     }
     if constexpr (LINEAR) rate = distance[active ? head : head0] / scale;
-    // the linear form for the lane's keys 4 h .. 4 h + 3 of a tile
+    // The linear form in two parts, as in attention_prefill_bf16_kernel: the lane's eight keys' places in their tile, and the tile's
+    // distance from the query, which joins the exponents' shift; or taken off whole.
+    constexpr bool IN_PARTS = LINEAR && !CAPPED && QB == 1, RAISES = LINEAR && QB == 1;
+    floatx4 in_tile[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
+    if constexpr (IN_PARTS) {
+#pragma unroll
+      for (int h = 0; h < 2; ++h)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) in_tile[h][i] = rate * (float)(key_chunk * 8 + h * 4 + i);
+    }
+    auto of_tile = [&](int tile, int b) { return -rate * (float)((live[b] ? pos[b] : pos_last) - tile * 32); };
     auto linear_bias = [&](int tile, int b, int h) {
-      const float before = -rate * (float)((live[b] ? pos[b] : pos_last) - (tile * 32 + key_chunk * 8));
-      return floatx4{fmaf(rate, (float)(4 * h), before), fmaf(rate, (float)(4 * h + 1), before), fmaf(rate, (float)(4 * h + 2), before),
-                     fmaf(rate, (float)(4 * h + 3), before)};
+      return linear_of_four(rate, (float)((live[b] ? pos[b] : pos_last) - (tile * 32 + key_chunk * 8 + h * 4)));
     };
     // what a tile's products are added to
     auto begin_scores = [&](int tile, floatx4 (&sc)[QB][2]) {
@@ -1399,8 +1458,8 @@ __global__ __launch_bounds__(MANY_WAVES ? 512 : 256, MANY_WAVES ? 1 : 2) void at
       for (int b = 0; b < QB; ++b)
 #pragma unroll
         for (int h = 0; h < 2; ++h) {
-          if constexpr (LINEAR && !CAPPED) sc[b][h] = linear_bias(tile, b, h);
-          else sc[b][h] = floatx4{0.f, 0.f, 0.f, 0.f};
+          if constexpr (LINEAR && !CAPPED && !IN_PARTS) sc[b][h] = linear_bias(tile, b, h);
+          else sc[b][h] = in_tile[h];
         }
     };
     auto take_off_linear = [&](int tile, floatx4 (&sc)[QB][2]) {
@@ -1408,6 +1467,18 @@ __global__ __launch_bounds__(MANY_WAVES ? 512 : 256, MANY_WAVES ? 1 : 2) void at
       for (int b = 0; b < QB; ++b)
 #pragma unroll
         for (int h = 0; h < 2; ++h) sc[b][h] += linear_bias(tile, b, h);
+    };
+    bool grown = false;                                        // a linear bias's weights have left the reference points behind
+    auto raise_reference = [&]() {
+#pragma unroll
+      for (int b = 0; b < QB; ++b) {
+        const float more = growth_of(run_sum[b]), shrink = fast_exp2(-more);
+        run_max[b] += more / scale2;
+        run_sum[b] *= shrink;
+#pragma unroll
+        for (int e = 0; e < DB; ++e) o[b][e] *= shrink;
+      }
+      grown = false;
     };
     auto take_off_distance = [&](int tile, floatx4 (&sc)[QB][2]) {
 #pragma unroll
@@ -1444,6 +1515,11 @@ __global__ __launch_bounds__(MANY_WAVES ? 512 : 256, MANY_WAVES ? 1 : 2) void at
 #pragma unroll
       for (int b = 0; b < QB; ++b) {
         float tile_max = -INFINITY;
+        if constexpr (IN_PARTS) {
+          const float all = of_tile(tile, b);
+          sc[b][0] += all;
+          sc[b][1] += all;
+        }
 #pragma unroll
         for (int h = 0; h < 2; ++h)
 #pragma unroll
@@ -1500,7 +1576,7 @@ __global__ __launch_bounds__(MANY_WAVES ? 512 : 256, MANY_WAVES ? 1 : 2) void at
       begin_scores(next_tile, next);
 #pragma unroll
       for (int b = 0; b < QB; ++b) {
-        shift[b] = -run_max[b] * scale2;                         // +inf before the query's first tile: the sum then says "again"
+        shift[b] = ((IN_PARTS ? of_tile(next_tile - 1, b) : 0.f) - run_max[b]) * scale2;      // +inf before the query's first tile: the sum then says "again"
         tile_sum[b] = 0.f;
       }
       __builtin_amdgcn_sched_barrier(0);
@@ -1525,6 +1601,12 @@ __global__ __launch_bounds__(MANY_WAVES ? 512 : 256, MANY_WAVES ? 1 : 2) void at
       if (__any(again)) return false;
 #pragma unroll
       for (int b = 0; b < QB; ++b) run_sum[b] += tile_sum[b];
+      if constexpr (RAISES) {
+        bool large = false;
+#pragma unroll
+        for (int b = 0; b < QB; ++b) large |= tile_sum[b] > GROWN;
+        grown = __any(large);
+      }
       if constexpr (CAPPED) cap_scores(next);
       if constexpr (DISTANCE) take_off_distance(next_tile, next);
       if constexpr (LINEAR && CAPPED) take_off_linear(next_tile, next);
@@ -1617,7 +1699,7 @@ __global__ __launch_bounds__(MANY_WAVES ? 512 : 256, MANY_WAVES ? 1 : 2) void at
       bool asked = false;                                      // the turn's fetches have been asked for already
       // one way out of the inner loop only, at its top, before anything of the turn has happened to the accumulators
       for (;;) {
-        if (asked || tile < fast_begin || tile >= fast_end) break;
+        if (asked || tile < fast_begin || tile >= fast_end || (RAISES && grown)) break;
         ask_ahead(std::true_type{});
         if (!weights_beside_scores(tile + 1, stage == STAGES - 1 ? 0 : stage + 1, sa, sb, pf)) {
           asked = true;
@@ -1627,6 +1709,12 @@ __global__ __launch_bounds__(MANY_WAVES ? 512 : 256, MANY_WAVES ? 1 : 2) void at
         turn_over(4);
 #pragma unroll
         for (int b = 0; b < QB; ++b) sa[b][0] = sb[b][0], sa[b][1] = sb[b][1];
+      }
+      if constexpr (RAISES) {
+        if (grown && !asked) {
+          raise_reference();
+          continue;
+        }
       }
       const bool unfinished = tile <= last_tile;
       if (!unfinished) break;
@@ -1753,11 +1841,16 @@ LRS_API int lrs_attention_prefill(void* out, int out_stride, const void* q, int 
   LRS_REQUIRE(d == 128 || table_lds <= 24 * 1024, "attention_prefill: a context of %d tokens needs more block table entries than fit LDS", max_context);
   hipStream_t s = (hipStream_t)stream;
 #define LAUNCH2(D, QB)                                                                                               \
-  attention_prefill_bf16_kernel<D, QB><<<grid, block, table_lds, s>>>((bf16*)out, out_stride, (const bf16*)q, q_stride, \
+  do {                                                                                                               \
+    if (distance && distance_form == DISTANCE_LINEAR) LAUNCH3(D, QB, true);                                          \
+    else LAUNCH3(D, QB, false);                                                                                      \
+  } while (0)
+#define LAUNCH3(D, QB, LINEAR)                                                                                       \
+  attention_prefill_bf16_kernel<D, QB, LINEAR><<<grid, block, table_lds, s>>>((bf16*)out, out_stride, (const bf16*)q, q_stride, \
                                                               (const bf16*)k_pages, (const bf16*)v_pages, block_table, \
                                                               table_stride, token_request, positions, qblock_token0, \
                                                               qblock_count, n_blocks, chunk, nq, nkv, page_size, scale, window, \
-                                                              splits, slots, part_o, part_ml, own_sinks, softcap, own_gates, gate_stride, dv, distance, distance_form)
+                                                              splits, slots, part_o, part_ml, own_sinks, softcap, own_gates, gate_stride, dv, distance)
 #define LAUNCH(D)                                \
   if (max_count <= 16) LAUNCH2(D, 1);            \
   else LAUNCH2(D, 2)
@@ -1804,6 +1897,7 @@ LRS_API int lrs_attention_prefill(void* out, int out_stride, const void* q, int 
   }
 #undef LAUNCH
 #undef LAUNCH2
+#undef LAUNCH3
   if (lrs_check_launch("attention_prefill")) return 1;
   if (keep_first > 0) {
     launch_attention_kept((const bf16*)q, q_stride, (const bf16*)k_pages, (const bf16*)v_pages, block_table, table_stride, token_request,

@@ -252,14 +252,26 @@ __global__ __launch_bounds__(256) void head_gemm_bf16_kernel(bf16* __restrict__ 
   const int lane = threadIdx.x % WAVE, wave = threadIdx.x / WAVE, col = lane & 15, g = lane >> 4;
   const int h = blockIdx.z, n0 = blockIdx.y * 64, t0 = blockIdx.x * 64 + wave * 16;
   if (t0 >= tokens) return;
-  if (ex.rot && blockIdx.y == 0) {
-    const int half = ex.rot / 2;
-    for (int i = lane; i < 16 * half; i += WAVE) {
+  if (n0 >= n) {               // the workgroups behind the outputs' (launched where there is something to rotate)
+    const int half = ex.rot / 2, count = min(16, tokens - t0);
+    for (int i = lane; i < count * half; i += WAVE) {
       const int at = t0 + i / half;
-      if (at < tokens) rotate_behind(ex, out + (int64_t)at * out_token + (int64_t)h * out_head, a + (int64_t)at * a_token + (int64_t)h * a_head, at, n, k, i % half);
+      rotate_behind(ex, out + (int64_t)at * out_token + (int64_t)h * out_head, a + (int64_t)at * a_token + (int64_t)h * a_head, at, n, k, i % half);
     }
+    return;
   }
   const int t = t0 + col;
+  // the gate's values of the lane's outputs, on their way while the product is made
+  bf16 gates[4][4];
+  if (ex.gate) {
+#pragma unroll
+    for (int c = 0; c < 4; ++c)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int row = t0 + 4 * g + i, nn = n0 + 16 * c + col;
+        gates[c][i] = row < tokens && nn < n ? ex.gate[(int64_t)row * ex.gate_stride + (int64_t)h * n + nn] : (bf16)0.f;
+      }
+  }
   const bf16* a_row = a + (int64_t)(t < tokens ? t : tokens - 1) * a_token + (int64_t)h * a_head + g * 8;
   const bf16* w_row = w + (int64_t)h * w_head + (int64_t)(n0 + col) * k + g * 8;
   floatx4 acc[4] = {};
@@ -284,7 +296,7 @@ __global__ __launch_bounds__(256) void head_gemm_bf16_kernel(bf16* __restrict__ 
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
       const int row = t0 + 4 * g + i, nn = n0 + 16 * c + col;
-      if (row < tokens && nn < n) out[(int64_t)row * out_token + (int64_t)h * out_head + nn] = (bf16)gated_value(ex, acc[c][i], row, h, n, nn);
+      if (row < tokens && nn < n) out[(int64_t)row * out_token + (int64_t)h * out_head + nn] = (bf16)(ex.gate ? acc[c][i] / (1.0f + __expf(-(float)gates[c][i])) : acc[c][i]);
     }
 }
 
@@ -543,8 +555,8 @@ LRS_API int lrs_head_gemm(void* out, int out_token, int out_head, const void* a,
   LRS_REQUIRE(k <= 4096, "head_gemm: k %d above the supported 4096", k);
   hipStream_t s = (hipStream_t)stream;
   if (dtype == LRS_BF16 && !trans && k % 8 == 0 && a_token % 8 == 0 && a_head % 8 == 0 && (uintptr_t)a % 16 == 0 && (uintptr_t)w % 16 == 0 &&
-      (n + 63) / 64 <= 65535) {
-    head_gemm_bf16_kernel<<<dim3((tokens + 63) / 64, (n + 63) / 64, heads), 256, 0, s>>>((bf16*)out, out_token, out_head, (const bf16*)a, a_token, a_head,
+      (n + 63) / 64 < 65535) {
+    head_gemm_bf16_kernel<<<dim3((tokens + 63) / 64, (n + 63) / 64 + (rot > 0), heads), 256, 0, s>>>((bf16*)out, out_token, out_head, (const bf16*)a, a_token, a_head,
                                                                                        (const bf16*)w, w_head, tokens, n, k,
                                                                                        HeadExtras<bf16>{rot, cosv, sinv, (const bf16*)gate, gate_stride});
     return lrs_check_launch("head_gemm");

@@ -746,6 +746,130 @@ __global__ __launch_bounds__(1024) void moe_combine_kernel(float* __restrict__ r
   }
 }
 
+// The same for rows of up to 8,192 values, a multiple of four: 16 bytes a load, a token's rows four at a time, everything that does
+// not wait for the sum asked for before it is made, the row in registers from the first sum to the last store.
+template <typename TW, int THREADS>
+__global__ __launch_bounds__(THREADS) void moe_combine_vec_kernel(float* __restrict__ residual, const float* __restrict__ rows, int hidden,
+                                                                  const int* __restrict__ place, const float* __restrict__ weights, int top,
+                                                                  const TW* __restrict__ norm_w, float eps, bf16* __restrict__ rounded, int kind,
+                                                                  float alpha, const float* __restrict__ extra, const CombineMore more) {
+  constexpr int PER = 8192 / 4 / THREADS, AT_ONCE = 4;
+  typedef TW w4 __attribute__((ext_vector_type(4)));
+  __shared__ float scratch[16];
+  const int t = blockIdx.x, quads = hidden / 4;
+  const int64_t base = (int64_t)t * hidden;
+  const int* where = place + (int64_t)t * top;
+  floatx4 acc[PER], old[PER], added[PER], self[PER], next_w[PER];
+  w4 nw[PER];
+#pragma unroll
+  for (int p = 0; p < PER; ++p) {
+    const int q = threadIdx.x + p * THREADS;
+    acc[p] = added[p] = self[p] = floatx4{0.f, 0.f, 0.f, 0.f};
+    if (q >= quads) continue;
+    if (kind != COMBINE_STORE) old[p] = *(const floatx4*)(residual + base + 4 * q);
+    if (extra) added[p] = *(const floatx4*)(extra + base + 4 * q);
+    if (norm_w) nw[p] = *(const w4*)(norm_w + 4 * q);
+    if (more.normed) next_w[p] = *(const floatx4*)(more.next_weight + 4 * q);
+    if (more.self) {
+      const int64_t at = (int64_t)t * more.self_stride + 4 * q;
+      if (more.self_f32) self[p] = *(const floatx4*)((const float*)more.self + at);
+      else {
+        const bf16x4 v = *(const bf16x4*)((const bf16*)more.self + at);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) self[p][i] = (float)v[i];
+      }
+    }
+  }
+  for (int c0 = 0; c0 < top; c0 += AT_ONCE) {
+    float share[AT_ONCE];
+    int row[AT_ONCE];
+#pragma unroll
+    for (int c = 0; c < AT_ONCE; ++c) {      // (past the last choice: the last one once more, weighing nothing)
+      const int at = c0 + c < top ? c0 + c : top - 1;
+      row[c] = where[at];
+      share[c] = c0 + c >= top ? 0.f : weights ? weights[(int64_t)t * top + at] : 1.f;
+    }
+#pragma unroll
+    for (int p = 0; p < PER; ++p) {
+      const int q = threadIdx.x + p * THREADS;
+      if (q >= quads) continue;
+      floatx4 v[AT_ONCE];
+#pragma unroll
+      for (int c = 0; c < AT_ONCE; ++c) v[c] = row[c] < 0 ? self[p] : *(const floatx4*)(rows + (int64_t)row[c] * hidden + 4 * q);
+#pragma unroll
+      for (int c = 0; c < AT_ONCE; ++c)
+        if (c0 + c < top) {
+#pragma unroll
+          for (int i = 0; i < 4; ++i) acc[p][i] = fmaf(share[c], v[c][i], acc[p][i]);
+        }
+    }
+  }
+  float ss = 0.f;
+#pragma unroll
+  for (int p = 0; p < PER; ++p) {
+    if (threadIdx.x + p * THREADS >= quads) continue;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      if (extra) acc[p][i] += added[p][i];
+      if (kind == COMBINE_LAYERNORM) {
+        acc[p][i] = fmaf(alpha, old[p][i], acc[p][i]);
+        ss += acc[p][i];
+      } else {
+        ss = fmaf(acc[p][i], acc[p][i], ss);
+      }
+    }
+  }
+  auto store = [&](int p, const floatx4& v) {
+    const int q = threadIdx.x + p * THREADS;
+    *(floatx4*)(residual + base + 4 * q) = v;
+    if (rounded) *(bf16x4*)(rounded + base + 4 * q) = bf16x4{(bf16)v[0], (bf16)v[1], (bf16)v[2], (bf16)v[3]};
+  };
+  float mean = 0.f, inv = 1.f;
+  if (kind == COMBINE_LAYERNORM) {
+    mean = block_sum(ss, scratch) / (float)hidden;
+    float sq = 0.f;
+#pragma unroll
+    for (int p = 0; p < PER; ++p) {
+      if (threadIdx.x + p * THREADS >= quads) continue;
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const float d = acc[p][i] - mean;
+        sq = fmaf(d, d, sq);
+      }
+    }
+    inv = 1.0f / sqrtf(block_sum(sq, scratch) / (float)hidden + eps);
+  } else if (kind == COMBINE_ADD_RMS) {
+    inv = 1.0f / sqrtf(block_sum(ss, scratch) / (float)hidden + eps);
+  }
+  float next = 0.f;
+#pragma unroll
+  for (int p = 0; p < PER; ++p) {
+    if (threadIdx.x + p * THREADS >= quads) continue;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      float v = acc[p][i];
+      if (kind == COMBINE_LAYERNORM) v = (v - mean) * inv * (float)nw[p][i];
+      else if (kind == COMBINE_ADD_RMS) v = old[p][i] + v * inv * (float)nw[p][i];
+      else if (kind == COMBINE_ADD) v = old[p][i] + v;
+      acc[p][i] = v;
+      next = fmaf(v, v, next);
+    }
+    store(p, acc[p]);
+  }
+  if (more.normed == nullptr) return;
+  const float next_inv = 1.0f / sqrtf(block_sum(next, scratch) / (float)hidden + more.next_eps);
+#pragma unroll
+  for (int p = 0; p < PER; ++p) {
+    const int q = threadIdx.x + p * THREADS;
+    if (q >= quads) continue;
+    floatx4 v;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) v[i] = acc[p][i] * next_inv * next_w[p][i];
+    if (more.normed_f32) *(floatx4*)((float*)more.normed + base + 4 * q) = v;
+    else *(bf16x4*)((bf16*)more.normed + base + 4 * q) = bf16x4{(bf16)v[0], (bf16)v[1], (bf16)v[2], (bf16)v[3]};
+  }
+}
+
 }  // namespace
 
 // Rows of a tile of the grouped products: 32, or 128 once the step brings every expert 48 rows and more on average: what
@@ -895,6 +1019,18 @@ LRS_API int lrs_moe_combine(float* residual, const float* rows, int tokens, int 
   const size_t lds = (size_t)(hidden + 16 + 2 * top) * sizeof(float);
   LRS_REQUIRE(lds <= 64 * 1024, "moe_combine: a width of %d with %d choices is too much", hidden, top);
   hipStream_t s = (hipStream_t)stream;
+  const int w_item = norm_dtype == LRS_BF16 ? 2 : 4, self_item = self_dtype == LRS_F32 ? 4 : 2, n_item = normed_dtype == LRS_F32 ? 4 : 2;
+  const bool vec = hidden % 4 == 0 && hidden <= 8192 && ((uintptr_t)residual | (uintptr_t)rows | (uintptr_t)extra | (uintptr_t)next_weight) % 16 == 0 &&
+                   (uintptr_t)norm_w % (4 * w_item) == 0 && (uintptr_t)self % (4 * self_item) == 0 && self_stride % 4 == 0 &&
+                   (uintptr_t)normed % (4 * n_item) == 0 && (uintptr_t)rounded % 8 == 0;
+  if (vec) {
+#define VEC(TW, THREADS) \
+  moe_combine_vec_kernel<TW, THREADS><<<tokens, THREADS, 0, s>>>(residual, rows, hidden, place, weights, top, (const TW*)norm_w, eps, (bf16*)rounded, kind, alpha, extra, more)
+    if (norm_w && norm_dtype == LRS_BF16) { if (hidden > 2048) VEC(bf16, 1024); else VEC(bf16, 512); }
+    else { if (hidden > 2048) VEC(float, 1024); else VEC(float, 512); }
+#undef VEC
+    return lrs_check_launch("moe_combine");
+  }
   const int threads = hidden >= 2048 ? 1024 : 256;
   if (norm_w && norm_dtype == LRS_BF16)
     moe_combine_kernel<bf16><<<tokens, threads, lds, s>>>(residual, rows, hidden, place, weights, top, (const bf16*)norm_w, eps, (bf16*)rounded, kind, alpha, extra, more);
